@@ -8,7 +8,8 @@
 // of the sequence).  With a window, the first `keep_first` keys of a sequence may stay visible to
 // every later query (t < keep_first), and a head may have a sink: one more term exp(sink_h) in the
 // softmax's denominator, with no key and no value.  The output may be gated: out * sigmoid(gate),
-// gate a matrix of out's shape.  A value head may have another size (vd) than a query and key
+// gate a matrix of out's shape.  Values may have been cached turned by their own position; the output is then turned
+// back by the query's (`turns`), before the gate.  A value head may have another size (vd) than a query and key
 // head (hd); the bfloat16 MFMA kernels take equal sizes, the others both.  Head
 // h reads kv head h / (n_heads / n_kv_heads) (attention.rs:432-438).  Scores,
 // softmax and the output sum are float32, in the one-pass form of
@@ -47,6 +48,7 @@ struct AttnArgs {
     int gate_per_head;   // 1: the gate is [tokens, n_heads], one number for all of a head's outputs
     float softcap;       // > 0: a scaled score s becomes softcap * tanh(s / softcap)
     const float* slopes; // [n_heads] or null: the score of key t for the query at p then loses slopes[h] * (p - t)
+    const float2* turns; // [tokens, vd / 2] (cos, sin) or null: output pair (2m, 2m + 1) is turned back by that angle
     int bs_shift;        // log2(bs) if bs is a power of two, else -1
     int n_items;
     float scale;
@@ -121,6 +123,20 @@ __device__ __forceinline__ void store_out(const AttnArgs& a, int tok, int h, int
         v *= 1.f / (1.f + expf(-gv));
     }
     from_float((T*)a.out + (size_t)tok * a.ldo + (size_t)h * a.vd + d, v);
+}
+
+// Values that were cached turned by their own position (pairs 2m, 2m + 1 of a head): the output of the query at token
+// tok is turned back by the query's angle, after the softmax and before any gate.  `v` is output element d, `other`
+// its partner d ^ 1.
+__device__ __forceinline__ float turned_back(const AttnArgs& a, int tok, int d, float v, float other) {
+    const float2 cs = a.turns[(size_t)tok * (a.vd >> 1) + (d >> 1)];
+    return fmaf(v, cs.x, (d & 1) ? -(other * cs.y) : other * cs.y);
+}
+// store_out from kernels whose lanes hold neighbouring output elements (lane l ^ 1 holds d ^ 1, and both are here)
+template <typename T>
+__device__ __forceinline__ void store_lane(const AttnArgs& a, int tok, int h, int d, float v) {
+    if (a.turns) v = turned_back(a, tok, d, v, lane_pair_other(v));
+    store_out<T>(a, tok, h, d, v);
 }
 
 // block of the table and slot in its page of key t (a shift when the page size is a power of two)
@@ -264,7 +280,7 @@ __global__ __launch_bounds__(64) void attn_tile_kernel(AttnArgs a) {
         if (d < a.vd) {
 #pragma unroll
             for (int i = 0; i < TQ; ++i)
-                if (i < n) store_out<T>(a, tok0 + i, h, d, o[dd][i] * finish_row<false>(a, h, m[i], l[i]));
+                if (i < n) store_lane<T>(a, tok0 + i, h, d, o[dd][i] * finish_row<false>(a, h, m[i], l[i]));
         }
     }
 }
@@ -396,7 +412,7 @@ __global__ __launch_bounds__(128) void attn_decode_merge_kernel(AttnArgs a) {
             const float v = (w > 0.f) ? po[(size_t)s * hd + d] : 0.f;   // an empty chunk wrote nothing
             acc = fmaf(w, v, acc);
         }
-        store_out<T>(a, tok, h, d, acc * fin);
+        store_lane<T>(a, tok, h, d, acc * fin);
     }
 }
 
@@ -751,7 +767,7 @@ __global__ __launch_bounds__(64) void attn_mfma_tile_kernel(AttnArgs a) {
 #pragma unroll
             for (int cb = 0; cb < WaveAttn<HD>::CB; ++cb) {
                 const int d = 16 * cb + li;
-                if (d < a.vd) store_out<bf16>(a, tok0 + row, h, d, w.o[cb][r] * fr);
+                if (d < a.vd) store_lane<bf16>(a, tok0 + row, h, d, w.o[cb][r] * fr);
             }
         }
     }
@@ -830,7 +846,7 @@ __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(Att
 #pragma unroll
                 for (int cb = 0; cb < WaveAttn<HD>::CB; ++cb) {
                     const int d = 16 * cb + li;
-                    if (d < a.vd) store_out<bf16>(a, tok, h, d, w.o[cb][r] * fin);
+                    if (d < a.vd) store_lane<bf16>(a, tok, h, d, w.o[cb][r] * fin);
                 }
             } else {
                 float* po = a.part_o + (((size_t)item * a.nh + h) * a.splits + split) * a.vd;
@@ -885,6 +901,23 @@ __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(Att
     const bool last = a.splits == 1;
     const float fin = last ? finish_row<true>(a, h, m, l) : 1.f;
     float* po = a.part_o + (((size_t)item * a.nh + h) * a.splits + split) * vd;
+    if (last && a.turns) {      // pairs of columns, which are turned back together
+        for (int d = 2 * sub; d < vd; d += 2 * per_row) {
+            float o0 = 0.f, o1 = 0.f;
+#pragma unroll
+            for (int u = 0; u < 8; ++u)
+                if (u < n_waves) {
+                    const float* src = wave_out + ((size_t)u * n + row) * stride + d;
+                    o0 += f[u] * src[0];
+                    o1 += f[u] * src[1];
+                }
+            o0 *= fin;
+            o1 *= fin;
+            store_out<bf16>(a, tok, h, d, turned_back(a, tok, d, o0, o1));
+            store_out<bf16>(a, tok, h, d + 1, turned_back(a, tok, d + 1, o1, o0));
+        }
+        return;
+    }
     for (int d = sub; d < vd; d += per_row) {
         float o = 0.f;
 #pragma unroll
@@ -1090,7 +1123,7 @@ __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(
 #pragma unroll
             for (int cb = 0; cb < CB; ++cb) {
                 const int d = 16 * cb + li;
-                if (d < vd) store_out<bf16>(a, tok0 + row, h, d, o[cb][r] * fr);
+                if (d < vd) store_lane<bf16>(a, tok0 + row, h, d, o[cb][r] * fr);
             }
         }
     }
@@ -1306,7 +1339,7 @@ __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(Att
         const float fr = __shfl(fin, row, 64);
         if (row < n) {
 #pragma unroll
-            for (int cb = 0; cb < CB; ++cb) store_out<bf16>(a, tok0 + row, h, 16 * cb + li, o[cb][r] * fr);
+            for (int cb = 0; cb < CB; ++cb) store_lane<bf16>(a, tok0 + row, h, 16 * cb + li, o[cb][r] * fr);
         }
     }
 }
@@ -1359,8 +1392,9 @@ FX_API int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void*
                          const int* positions, const int* item_seq, const int* item_tok, const int* item_n,
                          int n_items, int nh, int nkv, int hd, int bs, int window, float scale, int tile_q,
                          int vd, int mask_chunk, int keep_first, const float* sinks, const void* gate, long ldg,
-                         float softcap, const float* slopes, int gate_per_head) {
+                         float softcap, const float* slopes, int gate_per_head, const float* turns) {
     if (vd <= 0) vd = hd;
+    FX_REQUIRE(!turns || vd % 2 == 0, "attn_tiles: outputs that are turned back come in pairs, a value head has %d", vd);
     FX_REQUIRE(softcap >= 0.f && softcap < INFINITY, "attn_tiles: a cap of %g on the scores", (double)softcap);
     if (check_common("attn_tiles", dtype, nh, nkv, hd, bs, window, scale, vd, mask_chunk, keep_first)) return 1;
     FX_REQUIRE(tile_q == 64 || (tile_q == 128 && wide_items_ok(dtype, hd, bs) && mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd)),
@@ -1374,7 +1408,7 @@ FX_API int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void*
     a.vd = vd; a.mask_chunk = mask_chunk;
     a.keep_first = window > 0 ? keep_first : 0; a.sinks = sinks; a.gate = gate; a.ldg = ldg;
     a.gate_per_head = gate_per_head ? 1 : 0;
-    a.softcap = softcap; a.slopes = slopes;
+    a.softcap = softcap; a.slopes = slopes; a.turns = (const float2*)turns;
     a.bs_shift = log2_or_minus_one(bs);
     a.n_items = n_items;
     dim3 grid(n_items * 4, nh), grid_blocks(8 * ceil_div((long)n_items * nh, 8));     // a wave per 16 queries / a block per item
@@ -1424,10 +1458,10 @@ static int attn_decode_launch(void* stream, int dtype, const void* q, long ldq, 
                               int nh, int nkv, int hd, int bs, int window, float scale,
                               float* part_o, float* part_ml, int splits, int chunk, int waves, int vd = 0, int mask_chunk = 0,
                               int keep_first = 0, const float* sinks = nullptr, const void* gate = nullptr, long ldg = 0,
-                              float softcap = 0.f, const float* slopes = nullptr, int gate_per_head = 0) {
+                              float softcap = 0.f, const float* slopes = nullptr, int gate_per_head = 0, const float* turns = nullptr) {
     if (vd <= 0) vd = hd;
     AttnArgs a = {};
-    a.softcap = softcap; a.slopes = slopes; a.gate_per_head = gate_per_head ? 1 : 0;
+    a.softcap = softcap; a.slopes = slopes; a.gate_per_head = gate_per_head ? 1 : 0; a.turns = (const float2*)turns;
     a.q = q; a.ldq = ldq; a.out = out; a.ldo = ldo; a.k_pages = k_pages; a.v_pages = v_pages;
     a.block_table = block_table; a.max_blocks = max_blocks; a.positions = positions;
     a.item_seq = item_seq; a.item_tok = item_tok; a.item_n = nullptr;
@@ -1494,14 +1528,15 @@ FX_API int fx_attn_decode(void* stream, int dtype, const void* q, long ldq, void
                           int nh, int nkv, int hd, int bs, int window, float scale,
                           float* part_o, float* part_ml, int splits, int chunk, int waves, int vd, int mask_chunk,
                           int keep_first, const float* sinks, const void* gate, long ldg, float softcap, const float* slopes,
-                          int gate_per_head) {
+                          int gate_per_head, const float* turns) {
+    FX_REQUIRE(!turns || (vd > 0 ? vd : hd) % 2 == 0, "attn_decode: outputs that are turned back come in pairs, a value head has %d", vd > 0 ? vd : hd);
     if (attn_decode_check(dtype, nh, nkv, hd, bs, window, scale, splits, chunk)) return 1;
     FX_REQUIRE(softcap >= 0.f && softcap < INFINITY, "attn_decode: a cap of %g on the scores", (double)softcap);
     if (check_common("attn_decode", dtype, nh, nkv, hd, bs, window, scale, vd, mask_chunk, keep_first)) return 1;
     if (n_items <= 0) return 0;
     return attn_decode_launch(stream, dtype, q, ldq, out, ldo, k_pages, v_pages, block_table, max_blocks, positions,
                               item_seq, item_tok, n_items, nh, nkv, hd, bs, window, scale, part_o, part_ml, splits,
-                              chunk, waves, vd, mask_chunk, keep_first, sinks, gate, ldg, softcap, slopes, gate_per_head);
+                              chunk, waves, vd, mask_chunk, keep_first, sinks, gate, ldg, softcap, slopes, gate_per_head, turns);
 }
 
 // ---------------------------------------------------------------------------

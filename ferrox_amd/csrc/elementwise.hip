@@ -49,6 +49,44 @@ FX_API int fx_embed(void* stream, int w_dtype, const void* table, const int* ids
 }
 
 // ---------------------------------------------------------------------------
+// embedding rows brought to unit root mean square and weighted, in one launch:
+//   h[t, :] = x / sqrt(mean(x^2) + eps) * w,   x = table[ids[t], :] * scale
+// float32 sums; the row's second read comes from cache.  One block per token.
+// ---------------------------------------------------------------------------
+template <typename W>
+__global__ __launch_bounds__(256) void embed_rmsnorm_kernel(const W* __restrict__ table, const int* __restrict__ ids, float* __restrict__ h,
+                                                            int H, int V, float scale, const void* __restrict__ w, int w_dtype, float eps) {
+    __shared__ float red[4];
+    const int t = blockIdx.x, id = ids[t];
+    if (id < 0 || id >= V) {       // (the same in every thread; the host rejects such ids)
+        for (int c = threadIdx.x; c < H; c += 256) h[(size_t)t * H + c] = __int_as_float(0x7fc00000);
+        return;
+    }
+    const W* row = table + (size_t)id * H;
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < H; c += 256) {
+        const float x = to_float(row[c]) * scale;
+        ss = fmaf(x, x, ss);
+    }
+    ss = block_sum<4>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)H + eps);
+    for (int c = threadIdx.x; c < H; c += 256) h[(size_t)t * H + c] = to_float(row[c]) * scale * inv * load_as_float(w, w_dtype, c);
+}
+
+FX_API int fx_embed_rmsnorm(void* stream, int t_dtype, const void* table, const int* ids, float* h, int T, int H, int V,
+                            float scale, const void* w, int w_dtype, float eps) {
+    FX_REQUIRE(T >= 0 && H > 0 && V > 0, "embed_rmsnorm: bad sizes T=%d H=%d V=%d", T, H, V);
+    FX_REQUIRE(w && (w_dtype == FX_F32 || w_dtype == FX_BF16), "embed_rmsnorm: a norm weight of float32 or bfloat16");
+    if (T == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    if (t_dtype == FX_F32) embed_rmsnorm_kernel<float><<<T, 256, 0, s>>>((const float*)table, ids, h, H, V, scale, w, w_dtype, eps);
+    else if (t_dtype == FX_BF16) embed_rmsnorm_kernel<bf16><<<T, 256, 0, s>>>((const bf16*)table, ids, h, H, V, scale, w, w_dtype, eps);
+    else return fx_fail("embed_rmsnorm: unknown table dtype %d", t_dtype);
+    FX_CHECK_LAUNCH("embed_rmsnorm");
+    return 0;
+}
+
+// ---------------------------------------------------------------------------
 // Layer norm with weight and bias: y = (x - mean) / sqrt(var + eps) * w + b, var the mean of the squared
 // deviations from the mean (two passes over the row, which the second finds in cache), all in float32.  Input rows are
 // float32 (the residual stream), optionally gathered through `rows`; output is T.  One block per row.
@@ -513,6 +551,40 @@ FX_API int fx_head_norm_kv_write(void* stream, int dtype, const float* qk, long 
 // consecutive tokens, kv head): they norm the eight value heads into LDS and write them as `write_values` does.
 // ---------------------------------------------------------------------------
 #define UNIT_VD_MAX 256
+// the value heads of n <= 8 consecutive tokens from t0 on, staged in LDS, into their transposed pages (every thread of
+// the block calls this, after a barrier)
+template <typename T>
+__device__ __forceinline__ void write_staged_values(const T (*vs)[UNIT_VD_MAX], int kh, int t0, int n, const int* __restrict__ positions,
+                                                    const int* __restrict__ token_seq, const int* __restrict__ block_table,
+                                                    int max_blocks, T* __restrict__ v_pages, int nkv, int bs, int vd) {
+    const int tid = threadIdx.x;
+    const int pos0 = positions[t0], seq0 = token_seq[t0];
+    bool together = sizeof(T) == 2 && n == 8 && (bs & 7) == 0 && (pos0 & 7) == 0;
+    for (int i = 1; together && i < 8; ++i) together = positions[t0 + i] == pos0 + i && token_seq[t0 + i] == seq0;
+    if (together) {      // eight tokens that follow each other in one page: one 16-byte store per value channel
+        const int page = block_table[(size_t)seq0 * max_blocks + pos0 / bs];
+        T* dst = v_pages + ((size_t)page * nkv + kh) * vd * bs + pos0 % bs;
+        for (int d = tid; d < vd; d += 256) {
+            uint16_t e[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) e[i] = *(const uint16_t*)&vs[i][d];
+            uint4 o;
+            o.x = e[0] | ((uint32_t)e[1] << 16);
+            o.y = e[2] | ((uint32_t)e[3] << 16);
+            o.z = e[4] | ((uint32_t)e[5] << 16);
+            o.w = e[6] | ((uint32_t)e[7] << 16);
+            *(uint4*)(dst + (size_t)d * bs) = o;
+        }
+        return;
+    }
+    for (int idx = tid; idx < n * vd; idx += 256) {
+        const int i = idx / vd, d = idx - i * vd;
+        const int t = t0 + i, pos = positions[t];
+        const int page = block_table[(size_t)token_seq[t] * max_blocks + pos / bs];
+        v_pages[(((size_t)page * nkv + kh) * vd + d) * bs + pos % bs] = vs[i][d];
+    }
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void temp_unit_kv_write_kernel(
     const float* __restrict__ qkv, long ld, T* __restrict__ q_out, long ldq, const int* __restrict__ positions,
@@ -564,31 +636,7 @@ __global__ __launch_bounds__(256) void temp_unit_kv_write_kernel(
         }
     }
     __syncthreads();
-    const int pos0 = positions[t0], seq0 = token_seq[t0];
-    bool together = sizeof(T) == 2 && n == 8 && (bs & 7) == 0 && (pos0 & 7) == 0;
-    for (int i = 1; together && i < 8; ++i) together = positions[t0 + i] == pos0 + i && token_seq[t0 + i] == seq0;
-    if (together) {      // eight tokens that follow each other in one page: one 16-byte store per value channel
-        const int page = block_table[(size_t)seq0 * max_blocks + pos0 / bs];
-        T* dst = v_pages + ((size_t)page * nkv + kh) * vd * bs + pos0 % bs;
-        for (int d = tid; d < vd; d += 256) {
-            uint16_t e[8];
-#pragma unroll
-            for (int i = 0; i < 8; ++i) e[i] = *(const uint16_t*)&vs[i][d];
-            uint4 o;
-            o.x = e[0] | ((uint32_t)e[1] << 16);
-            o.y = e[2] | ((uint32_t)e[3] << 16);
-            o.z = e[4] | ((uint32_t)e[5] << 16);
-            o.w = e[6] | ((uint32_t)e[7] << 16);
-            *(uint4*)(dst + (size_t)d * bs) = o;
-        }
-        return;
-    }
-    for (int idx = tid; idx < n * vd; idx += 256) {
-        const int i = idx / vd, d = idx - i * vd;
-        const int t = t0 + i, pos = positions[t];
-        const int page = block_table[(size_t)token_seq[t] * max_blocks + pos / bs];
-        v_pages[(((size_t)page * nkv + kh) * vd + d) * bs + pos % bs] = vs[i][d];
-    }
+    write_staged_values<T>(vs, kh, t0, n, positions, token_seq, block_table, max_blocks, v_pages, nkv, bs, vd);
 }
 
 FX_API int fx_temp_unit_kv_write(void* stream, int dtype, const float* qkv, long ld, void* q_out, long ldq, const int* positions,
@@ -614,6 +662,126 @@ FX_API int fx_temp_unit_kv_write(void* stream, int dtype, const float* qkv, long
     else
         return fx_fail("temp_unit_kv_write: unknown dtype %d", dtype);
     FX_CHECK_LAUNCH("temp_unit_kv_write");
+    return 0;
+}
+
+// ---------------------------------------------------------------------------
+// Sines and cosines of a step's rotation angles, made once for all layers that rotate by the same frequencies:
+// out[t, m] = (cos, sin)(positions[t] * inv_freq[m]), the angle a float32 product.
+// ---------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void angle_table_kernel(const int* __restrict__ positions, const float* __restrict__ inv_freq,
+                                                          float2* __restrict__ out, int n, long total) {
+    const long i = (long)blockIdx.x * 256 + threadIdx.x;
+    if (i >= total) return;
+    const int t = (int)(i / n), m = (int)(i - (long)t * n);
+    float2 cs;
+    sincosf((float)positions[t] * inv_freq[m], &cs.y, &cs.x);
+    out[i] = cs;
+}
+
+FX_API int fx_angle_table(void* stream, const int* positions, const float* inv_freq, float* out, int T, int n) {
+    FX_REQUIRE(T >= 0 && n > 0, "angle_table: bad sizes T=%d n=%d", T, n);
+    FX_REQUIRE(((uintptr_t)out % 8) == 0, "angle_table: the table holds pairs of floats, 8-byte aligned");
+    if (T == 0) return 0;
+    const long total = (long)T * n;
+    angle_table_kernel<<<(unsigned)((total + 255) / 256), 256, 0, (hipStream_t)stream>>>(positions, inv_freq, (float2*)out, n, total);
+    FX_CHECK_LAUNCH("angle_table");
+    return 0;
+}
+
+// ---------------------------------------------------------------------------
+// From the float32 product qkv [T, nh hd | nkv hd | nkv vd] of a token, with its angles as (cos, sin) tables:
+//   q_out       = q, its first `rot` dimensions rotated by qk_turns[t, 0 .. rot/2), times temp[head] (null: 1)
+//   key page    <- k, rotated the same way
+//   value page  <- v, with a table v_turns [T, vd/2] every pair (2m, 2m + 1) of a head turned by angle m; transposed
+// Pairs of q and k are (i, i + rot/2), or (2i, 2i + 1) when `interleaved`; a value's pairs always lie side by side (a
+// caller whose value pairs are halves of the head reorders the rows of its projection, so that they do).
+// q_out and the pages have type T; everything before the one rounding is float32 arithmetic.  The first blocks take
+// (token, head of q or k) a wave each; the blocks after them take (eight consecutive tokens, kv head): they turn the
+// eight value heads into LDS and write them as `write_values` does.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void turned_kv_write_kernel(
+    const float* __restrict__ qkv, long ld, T* __restrict__ q_out, long ldq, const float* __restrict__ temp, const int* __restrict__ positions,
+    const int* __restrict__ token_seq, const int* __restrict__ block_table, int max_blocks, T* __restrict__ k_pages,
+    T* __restrict__ v_pages, int n_tokens, int nh, int nkv, int hd, int vd, int bs, int rot, int interleaved,
+    const float2* __restrict__ qk_turns, const float2* __restrict__ v_turns, int head_blocks) {
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    if ((int)blockIdx.x < head_blocks) {
+        const int units = nh + (k_pages ? nkv : 0);
+        const int r = blockIdx.x * 4 + wave;
+        if (r >= n_tokens * units) return;
+        const int t = r / units, u = r - t * units, half = rot >> 1;
+        const float* x = qkv + (size_t)t * ld + (size_t)u * hd;
+        const float2* turns = qk_turns + (size_t)t * half;
+        T* dst;
+        float factor = 1.f;
+        if (u < nh) {
+            dst = q_out + (size_t)t * ldq + (size_t)u * hd;
+            if (temp) factor = temp[u];
+        } else {
+            const int pos = positions[t];
+            const int page = block_table[(size_t)token_seq[t] * max_blocks + pos / bs];
+            dst = k_pages + (((size_t)page * nkv + (u - nh)) * bs + pos % bs) * hd;
+        }
+        for (int i = lane; i < half; i += 64) {
+            const int ia = interleaved ? 2 * i : i, ib = interleaved ? 2 * i + 1 : i + half;
+            const float2 cs = turns[i];
+            float y0, y1;
+            rotate_pair(x[ia], x[ib], cs.x, cs.y, y0, y1);
+            from_float(dst + ia, y0 * factor);
+            from_float(dst + ib, y1 * factor);
+        }
+        for (int c = rot + lane; c < hd; c += 64) from_float(dst + c, x[c] * factor);
+        return;
+    }
+    if (!v_pages) return;
+    __shared__ T vs[8][UNIT_VD_MAX];
+    const int b = blockIdx.x - head_blocks;
+    const int kh = b % nkv, t0 = (b / nkv) * 8;
+    const int n = min(8, n_tokens - t0);
+    for (int i = wave; i < n; i += 4) {
+        const float* v = qkv + (size_t)(t0 + i) * ld + (size_t)(nh + nkv) * hd + (size_t)kh * vd;
+        if (v_turns) {
+            for (int m = lane; m < (vd >> 1); m += 64) {
+                const float2 cs = v_turns[(size_t)(t0 + i) * (vd >> 1) + m];
+                float y0, y1;
+                rotate_pair(v[2 * m], v[2 * m + 1], cs.x, cs.y, y0, y1);
+                from_float(&vs[i][2 * m], y0);
+                from_float(&vs[i][2 * m + 1], y1);
+            }
+        } else {
+            for (int c = lane; c < vd; c += 64) from_float(&vs[i][c], v[c]);
+        }
+    }
+    __syncthreads();
+    write_staged_values<T>(vs, kh, t0, n, positions, token_seq, block_table, max_blocks, v_pages, nkv, bs, vd);
+}
+
+FX_API int fx_turned_kv_write(void* stream, int dtype, const float* qkv, long ld, void* q_out, long ldq, const float* temp,
+                              const int* positions, const int* token_seq, const int* block_table, int max_blocks, void* k_pages,
+                              void* v_pages, int T, int nh, int nkv, int hd, int vd, int bs, int rot, int interleaved,
+                              const float* qk_turns, const float* v_turns) {
+    FX_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && bs > 0, "turned_kv_write: bad sizes");
+    FX_REQUIRE(hd > 0 && vd > 0 && vd <= UNIT_VD_MAX, "turned_kv_write: head sizes %d and %d (values up to %d)", hd, vd, UNIT_VD_MAX);
+    FX_REQUIRE(rot >= 0 && rot <= hd && rot % 2 == 0 && (rot == 0 || qk_turns), "turned_kv_write: %d rotated dimensions of %d need a table of angles", rot, hd);
+    FX_REQUIRE(!v_turns || vd % 2 == 0, "turned_kv_write: turned values come in pairs, a value head has %d", vd);
+    FX_REQUIRE((((uintptr_t)qk_turns | (uintptr_t)v_turns) % 8) == 0, "turned_kv_write: tables of angles hold pairs of floats, 8-byte aligned");
+    FX_REQUIRE((k_pages == nullptr) == (v_pages == nullptr), "turned_kv_write: key and value pages must come together");
+    FX_REQUIRE(ld >= (long)(nh + nkv) * hd + (long)nkv * vd && ldq >= (long)nh * hd, "turned_kv_write: rows too short");
+    if (T == 0) return 0;
+    const long units = nh + (k_pages ? nkv : 0);
+    const long head_blocks = (T * units + 3) / 4, n_blocks = head_blocks + (v_pages ? (long)((T + 7) / 8) * nkv : 0);
+    FX_REQUIRE(n_blocks < (1L << 31) && T * units < (1L << 31), "turned_kv_write: too many tokens and heads for one launch");
+    hipStream_t s = (hipStream_t)stream;
+#define FX_TURNED(T_) turned_kv_write_kernel<T_><<<(unsigned)n_blocks, 256, 0, s>>>(qkv, ld, (T_*)q_out, ldq, temp, positions, token_seq, \
+        block_table, max_blocks, (T_*)k_pages, (T_*)v_pages, T, nh, nkv, hd, vd, bs, rot, interleaved, (const float2*)qk_turns,            \
+        (const float2*)v_turns, (int)head_blocks)
+    if (dtype == FX_F32) FX_TURNED(float);
+    else if (dtype == FX_BF16) FX_TURNED(bf16);
+    else return fx_fail("turned_kv_write: unknown dtype %d", dtype);
+#undef FX_TURNED
+    FX_CHECK_LAUNCH("turned_kv_write");
     return 0;
 }
 

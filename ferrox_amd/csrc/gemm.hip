@@ -64,7 +64,7 @@ struct GemmArgs {
     const float* rope_freq_factors;   // rot/2 floats or null: the angle of pair i is divided by rope_freq_factors[i]
     int stream_w;  // tiled kernel: the weights are read about once (one row tile a weight matrix): load them non-temporal
     int act;     // EPI_GATED: which activation the gate goes through (ACT_*)
-    float act_limit, act_alpha;   // ACT_SWIGLU_CLAMP: the bound on gate and up, and the sigmoid's slope
+    float act_limit, act_alpha;   // ACT_SWIGLU_CLAMP: the bound on gate and up, and the sigmoid's slope; SACT_SOFTCAP: the cap
     const float* pre_scale;       // EPI_GATED: [.] or null: gate and up of logical row m are multiplied by
     const int* pre_scale_rows;    //   pre_scale[pre_scale_rows ? pre_scale_rows[m] : m] before the activation (a row of A scaled)
     int store_act;   // EPI_STORE: what the product goes through before it is stored (SACT_*), 0 for nothing
@@ -198,9 +198,10 @@ __device__ __forceinline__ float gated_c(float gate, float up, float limit, floa
 }
 // What a stored product (EPI_STORE) may go through on its way out: the activation of a feed-forward without a gate,
 // down(act(up x)).  Uniform over the launch; SACT_NONE costs one scalar compare per element.
-//   SACT_RELU2  max(x, 0)^2
-enum { SACT_NONE = 0, SACT_RELU2 = 1, SACT_RELU = 2, SACT_SILU = 3, SACT_GELU_TANH = 4, SACT_COUNT = 5 };
-__device__ __forceinline__ float stored_f(int act, float x) {
+//   SACT_RELU2    max(x, 0)^2
+//   SACT_SOFTCAP  limit * tanh(x / limit)      (logits kept within +-limit)
+enum { SACT_NONE = 0, SACT_RELU2 = 1, SACT_RELU = 2, SACT_SILU = 3, SACT_GELU_TANH = 4, SACT_SOFTCAP = 5, SACT_COUNT = 6 };
+__device__ __forceinline__ float stored_f(int act, float x, float limit) {
     if (act == SACT_NONE) return x;
     if (act == SACT_RELU2) {
         const float r = fmaxf(x, 0.0f);
@@ -208,6 +209,7 @@ __device__ __forceinline__ float stored_f(int act, float x) {
     }
     if (act == SACT_RELU) return fmaxf(x, 0.0f);
     if (act == SACT_SILU) return silu_f(x);
+    if (act == SACT_SOFTCAP) return limit * tanhf(x / limit);
     return 0.5f * x * (1.0f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
 }
 // what gate and up of logical row m are multiplied by before the activation (1 without a pre-scale)
@@ -398,9 +400,9 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs g) {
                     float v = acc[i][j][r];
                     if (g.bias) v += bias_v[j];
                     if (EPI == EPI_STORE) {
-                        from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_f(g.store_act, v));
+                        from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_f(g.store_act, v, g.act_limit));
                     } else if (EPI == EPI_STORE_F32) {
-                        ((float*)g.C)[(size_t)m * g.ldc + n] = stored_f(g.store_act, v);
+                        ((float*)g.C)[(size_t)m * g.ldc + n] = stored_f(g.store_act, v, g.act_limit);
                     } else {
                         if (g.row_scale) v *= g.row_scale[ml];
                         ((float*)g.C)[(size_t)m * g.ldc + n] += v;
@@ -663,9 +665,9 @@ __global__ __launch_bounds__(512) void gemm_bf16_wide_kernel(GemmArgs g) {
                     float v = acc[i][j][r];
                     if (g.bias) v += bias_v[j];
                     if (EPI == EPI_STORE) {
-                        from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_f(g.store_act, v));
+                        from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_f(g.store_act, v, g.act_limit));
                     } else if (EPI == EPI_STORE_F32) {
-                        ((float*)g.C)[(size_t)m * g.ldc + n] = stored_f(g.store_act, v);
+                        ((float*)g.C)[(size_t)m * g.ldc + n] = stored_f(g.store_act, v, g.act_limit);
                     } else {
                         if (g.row_scale) {
                             v *= scale_of[i][r];
@@ -1109,9 +1111,9 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(GemmArgs g
             }
             if (g.bias) o += bias_v[r];
             if (EPI == EPI_STORE) {
-                from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_f(g.store_act, o));
+                from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_f(g.store_act, o, g.act_limit));
             } else if (EPI == EPI_STORE_F32) {
-                ((float*)g.C)[(size_t)m * g.ldc + n] = stored_f(g.store_act, o);
+                ((float*)g.C)[(size_t)m * g.ldc + n] = stored_f(g.store_act, o, g.act_limit);
             } else {
                 if (g.row_scale) {
                     o *= row_scale;
@@ -1208,7 +1210,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmArgs g) {
                     if (g.row_scale) v *= g.row_scale[ml];
                     *out += v;
                 } else {
-                    *out = stored_f(g.store_act, v);      // (the host sets store_act for stored products only)
+                    *out = stored_f(g.store_act, v, g.act_limit);      // (the host sets store_act for stored products only)
                 }
             }
         }
@@ -1400,6 +1402,7 @@ FX_API int fx_gemm(void* stream, int dtype, int epi, const void* A, long lda, co
                "gemm: a stored activation (%d) goes with the plain stored product without bias", store_act);
     FX_REQUIRE(!pre_scale || epi == EPI_GATED, "gemm: a scale in front of the activation goes with the gate/up epilogue");
     FX_REQUIRE(act != ACT_SWIGLU_CLAMP || act_limit > 0.f, "gemm: the clamped gate needs a positive limit, got %g", (double)act_limit);
+    FX_REQUIRE(store_act != SACT_SOFTCAP || act_limit > 0.f, "gemm: capped outputs need a positive cap, got %g", (double)act_limit);
     FX_REQUIRE(dtype == FX_F32 || dtype == FX_BF16, "gemm: unknown dtype %d", dtype);
     FX_REQUIRE(epi >= EPI_STORE && epi <= EPI_GATED, "gemm: unknown epilogue %d", epi);
     FX_REQUIRE(M >= 0 && N > 0 && K > 0, "gemm: bad sizes M=%d N=%d K=%d", M, N, K);

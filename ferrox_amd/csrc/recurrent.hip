@@ -1,5 +1,6 @@
-// Recurrent mixers: a short causal convolution with its carried inputs, and the gated delta
-// rule with one decay per key channel, whose state is a [key channels, value channels] matrix per head.
+// Recurrent mixers: a short causal convolution with its carried inputs, mixes of a token with the one before it, and
+// linear recurrences whose state is a [key channels, value channels] matrix per head (the gated delta rule with one
+// decay per key channel, outer products under decays per head or per key channel).
 //
 // Everything that enters the recurrence is float32: the convolved q, k, v, the decays, the step
 // sizes, the state.  A sequence's tokens lie next to each other in the batch: sequence s owns
@@ -554,24 +555,29 @@ FX_API int fx_gated_head_norm(void* stream, int out_dtype, const float* o, long 
 // Lanes, columns, the state's transposed layout, the groups of P tokens that a block of waves brings into LDS a
 // group ahead: as in the delta rule's kernel above; a token's work is one pass over the lane's rows (S updated,
 // then its part of S^T q) and one sum over the lanes of a column.
+// CHANNEL: one forgetting factor per key channel instead, and a read-out that comes before the update, with a bonus
+// u [H, D] that the current token alone gets:
+//   o_t = q_scale (S + diag(u) k_t v_t^T)^T q_t;   S <- diag(keep_t) S + k_t v_t^T            keep: [T, H, D]
+// (the factors travel through LDS beside k and q; no writing factors, no normaliser).
 // Grid: (ceil((V + normalizer) / (NW 64 / LPC)), heads, sequences).
 // ---------------------------------------------------------------------------
-template <int DR, int LPC, bool VEC, int NW>
+template <int DR, int LPC, bool VEC, int NW, bool CHANNEL>
 __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __restrict__ q, long ldq, const float* __restrict__ k, long ldk,
                                                               const float* __restrict__ v, long ldv, const float* __restrict__ keep,
                                                               int keep_const, const float* __restrict__ take, float* __restrict__ out,
                                                               long ldo, float* __restrict__ nq, float* __restrict__ state,
                                                               const int* __restrict__ seq_starts, const int* __restrict__ slots,
-                                                              int H, int G, int D, int V, int VS, float q_scale) {
+                                                              int H, int G, int D, int V, int VS, float q_scale, const float* __restrict__ bonus) {
     constexpr int DP = LPC * DR;                     // rows as a wave holds them
     constexpr int W = VEC ? 4 : 1;                   // floats per load
     constexpr int P = 8;                             // tokens that travel together
     constexpr int NT = NW * 64;
-    constexpr int PIECES = 2 * DP / W;               // loads that bring one token's (k | q)
+    constexpr int OPS = CHANNEL ? 3 : 2;
+    constexpr int PIECES = OPS * DP / W;             // loads that bring one token's (k | q), or (k | q | keep)
     constexpr int NL = (P * PIECES + NT - 1) / NT;   // loads a thread makes per group
     constexpr int COLS = 64 / LPC;
     static_assert(DR % 4 == 0, "a lane's rows are read from LDS in 16-byte pieces");
-    __shared__ __attribute__((aligned(16))) float kq[2][P][2][DP];      // two groups of P tokens x (k, q)
+    __shared__ __attribute__((aligned(16))) float kq[2][P][OPS][DP];      // two groups of P tokens x (k, q (, keep))
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int r = lane % LPC, j = (blockIdx.x * NW + wave) * COLS + lane / LPC;
     const int h = blockIdx.y, s = blockIdx.z, g = h / (H / G);
@@ -591,6 +597,11 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
             for (int e = 0; e < 4; ++e) S[i + e] = (col && r * DR + i + e < D) ? S_g[i + e] : 0.f;
         }
     }
+    float u[CHANNEL ? DR : 1];
+    if constexpr (CHANNEL) {
+#pragma unroll
+        for (int i = 0; i < DR; ++i) u[i] = r * DR + i < D ? bonus[(size_t)h * D + r * DR + i] : 0.f;
+    }
     const float keep_fixed = keep_const ? keep[h] : 0.f;
     float nxt[NL][W], v_nxt[P], a_nxt[P], b_nxt[P];
     auto fetch = [&](int first) {
@@ -600,6 +611,7 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
             const int t = first + p;
             const bool ok = idx < P * PIECES && t < t1 && row < D;
             const float* src = which == 0 ? k + (size_t)t * ldk + (size_t)g * D : q + (size_t)t * ldq + (size_t)g * D;
+            if constexpr (CHANNEL) src = which == 2 ? keep + ((size_t)t * H + h) * D : src;
             if constexpr (VEC) {
                 const float4 x = ok ? *(const float4*)(src + row) : make_float4(0.f, 0.f, 0.f, 0.f);
                 nxt[n][0] = x.x; nxt[n][W - 3] = x.y; nxt[n][W - 2] = x.z; nxt[n][W - 1] = x.w;
@@ -611,8 +623,13 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
         for (int p = 0; p < P; ++p) {
             const bool live = first + p < t1;
             v_nxt[p] = (live && col) ? (ones ? 1.0f : v[(size_t)(first + p) * ldv + (size_t)h * V + j]) : 0.f;
-            a_nxt[p] = live ? (keep_const ? keep_fixed : keep[(size_t)(first + p) * H + h]) : 1.f;
-            b_nxt[p] = live ? (take ? take[(size_t)(first + p) * H + h] : 1.f) : 0.f;
+            if constexpr (CHANNEL) {
+                a_nxt[p] = 1.f;
+                b_nxt[p] = 1.f;
+            } else {
+                a_nxt[p] = live ? (keep_const ? keep_fixed : keep[(size_t)(first + p) * H + h]) : 1.f;
+                b_nxt[p] = live ? (take ? take[(size_t)(first + p) * H + h] : 1.f) : 0.f;
+            }
         }
     };
     auto stage = [&](int slot) {
@@ -646,10 +663,20 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
             for (int i = 0; i < DR; i += 4) {
                 const float4 k4 = *(const float4*)(kk + i), q4 = *(const float4*)(qq + i);
                 const float ka[4] = {k4.x, k4.y, k4.z, k4.w}, qa[4] = {q4.x, q4.y, q4.z, q4.w};
+                if constexpr (CHANNEL) {
+                    const float4 d4 = *(const float4*)(&kq[cur][p][OPS - 1][r * DR] + i);
+                    const float da[4] = {d4.x, d4.y, d4.z, d4.w};
 #pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    S[i + e] = fmaf(ka[e], bv_cur[p], S[i + e] * a_cur[p]);
-                    sq = fmaf(S[i + e], qa[e], sq);
+                    for (int e = 0; e < 4; ++e) {
+                        sq = fmaf(fmaf(u[i + e] * ka[e], bv_cur[p], S[i + e]), qa[e], sq);
+                        S[i + e] = fmaf(ka[e], bv_cur[p], S[i + e] * da[e]);
+                    }
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        S[i + e] = fmaf(ka[e], bv_cur[p], S[i + e] * a_cur[p]);
+                        sq = fmaf(S[i + e], qa[e], sq);
+                    }
                 }
             }
             sq = column_sum<LPC>(sq) * q_scale;
@@ -681,32 +708,49 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
     }
 }
 
-FX_API int fx_gated_outer(void* stream, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
-                          const float* keep, int keep_const, const float* take, float* out, long ldo, float* nq, float* state,
-                          const int* seq_starts, const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale) {
-    FX_REQUIRE(n_seqs >= 0 && H > 0 && G > 0 && H % G == 0, "gated_outer: bad sizes sequences=%d H=%d G=%d", n_seqs, H, G);
-    FX_REQUIRE(D >= 1 && D <= 256 && V >= 1, "gated_outer: key size %d (up to 256) and value size %d", D, V);
-    FX_REQUIRE(ldq >= (long)G * D && ldk >= (long)G * D && ldv >= (long)H * V && ldo >= (long)H * V, "gated_outer: rows too short for %d heads", H);
-    FX_REQUIRE(n_seqs <= 65535 && H <= 65535, "gated_outer: %d sequences of %d heads are more than a launch takes", n_seqs, H);
-    FX_REQUIRE(keep, "gated_outer: the forgetting factors are missing");
+template <bool CHANNEL>
+static int launch_gated_outer(const char* who, void* stream, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
+                              const float* keep, int keep_const, const float* take, float* out, long ldo, float* nq, float* state,
+                              const int* seq_starts, const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale,
+                              const float* bonus) {
+    FX_REQUIRE(n_seqs >= 0 && H > 0 && G > 0 && H % G == 0, "%s: bad sizes sequences=%d H=%d G=%d", who, n_seqs, H, G);
+    FX_REQUIRE(D >= 1 && D <= 256 && V >= 1, "%s: key size %d (up to 256) and value size %d", who, D, V);
+    FX_REQUIRE(ldq >= (long)G * D && ldk >= (long)G * D && ldv >= (long)H * V && ldo >= (long)H * V, "%s: rows too short for %d heads", who, H);
+    FX_REQUIRE(n_seqs <= 65535 && H <= 65535, "%s: %d sequences of %d heads are more than a launch takes", who, n_seqs, H);
+    FX_REQUIRE(keep, "%s: the forgetting factors are missing", who);
     if (n_seqs == 0) return 0;
     const int VS = V + (nq ? 1 : 0);
-    const bool vec = D % 4 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && (((uintptr_t)state | (uintptr_t)q | (uintptr_t)k) % 16) == 0;
+    const bool vec = D % 4 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && (((uintptr_t)state | (uintptr_t)q | (uintptr_t)k | (CHANNEL ? (uintptr_t)keep : 0)) % 16) == 0;
     hipStream_t s = (hipStream_t)stream;
 #define FX_OUTER(DR_, LPC_, NW_)                                                                                              \
     do {                                                                                                                      \
         const int per_block = NW_ * 64 / LPC_;                                                                                \
         const dim3 grid((VS + per_block - 1) / per_block, H, n_seqs);                                                         \
-        if (vec) gated_outer_kernel<DR_, LPC_, true, NW_><<<grid, NW_ * 64, 0, s>>>(q, ldq, k, ldk, v, ldv, keep, keep_const, take, out, ldo, nq, state, seq_starts, slots, H, G, D, V, VS, q_scale); \
-        else gated_outer_kernel<DR_, LPC_, false, NW_><<<grid, NW_ * 64, 0, s>>>(q, ldq, k, ldk, v, ldv, keep, keep_const, take, out, ldo, nq, state, seq_starts, slots, H, G, D, V, VS, q_scale);    \
+        if (vec) gated_outer_kernel<DR_, LPC_, true, NW_, CHANNEL><<<grid, NW_ * 64, 0, s>>>(q, ldq, k, ldk, v, ldv, keep, keep_const, take, out, ldo, nq, state, seq_starts, slots, H, G, D, V, VS, q_scale, bonus); \
+        else gated_outer_kernel<DR_, LPC_, false, NW_, CHANNEL><<<grid, NW_ * 64, 0, s>>>(q, ldq, k, ldk, v, ldv, keep, keep_const, take, out, ldo, nq, state, seq_starts, slots, H, G, D, V, VS, q_scale, bonus);    \
     } while (0)
     if (D <= 64 && V <= 32) FX_OUTER(4, 16, 2);
     else if (D <= 64) FX_OUTER(4, 16, 4);
     else if (D <= 128) FX_OUTER(4, 32, 4);
     else FX_OUTER(8, 32, 8);
 #undef FX_OUTER
-    FX_CHECK_LAUNCH("gated_outer");
+    FX_CHECK_LAUNCH(who);
     return 0;
+}
+
+FX_API int fx_gated_outer(void* stream, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
+                          const float* keep, int keep_const, const float* take, float* out, long ldo, float* nq, float* state,
+                          const int* seq_starts, const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale) {
+    return launch_gated_outer<false>("gated_outer", stream, q, ldq, k, ldk, v, ldv, keep, keep_const, take, out, ldo, nq, state,
+                                     seq_starts, slots, n_seqs, H, G, D, V, q_scale, nullptr);
+}
+
+FX_API int fx_channel_outer(void* stream, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
+                            const float* keep, const float* bonus, float* out, long ldo, float* state, const int* seq_starts,
+                            const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale) {
+    FX_REQUIRE(bonus, "channel_outer: the current token's bonus is missing");
+    return launch_gated_outer<true>("channel_outer", stream, q, ldq, k, ldk, v, ldv, keep, 0, nullptr, out, ldo, nullptr, state,
+                                    seq_starts, slots, n_seqs, H, G, D, V, q_scale, bonus);
 }
 
 // ---------------------------------------------------------------------------
@@ -888,5 +932,142 @@ FX_API int fx_rglru_scan(void* stream, int out_dtype, const float* a, const floa
     }
 #undef FX_SCAN
     FX_CHECK_LAUNCH("rglru_scan");
+    return 0;
+}
+
+// ---------------------------------------------------------------------------
+// Mixes of every token with the one before it in its sequence, several at once:
+//   out[i, t, c] = x[t, c] + (x'[t, c] - x[t, c]) * mu[i, c],   i < n_mix
+// x' is the sequence's previous row: row t - 1 inside the step's portion, else what was carried from before it
+// (state[slot, c], float32; zeros at a sequence's start).  Afterwards the state holds the portion's last row: the thread
+// that reads a sequence's state writes it too.  Rows are T, the arithmetic is float32.
+// VEC channels to a thread, one block per (stretch of 256 VEC channels, token).
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__device__ __forceinline__ void load_row(const T* p, float (&v)[VEC]) {
+    if constexpr (VEC == 8) {                        // bfloat16, 16 bytes
+        const uint4 a = *(const uint4*)p;
+        const uint32_t w[4] = {a.x, a.y, a.z, a.w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            v[2 * e] = __uint_as_float(w[e] << 16);
+            v[2 * e + 1] = __uint_as_float(w[e] & 0xffff0000u);
+        }
+    } else if constexpr (VEC == 4) {                 // float32, 16 bytes
+        const float4 a = *(const float4*)p;
+        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+    } else {
+        v[0] = to_float(p[0]);
+    }
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void token_shift_kernel(const T* __restrict__ x, long ldx, const float* __restrict__ mu, int n_mix,
+                                                          T* __restrict__ out, float* __restrict__ state,
+                                                          const int* __restrict__ token_seq, const int* __restrict__ seq_starts,
+                                                          const int* __restrict__ slots, int n_tokens, int C) {
+    const int t = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+    if (c >= C) return;                              // (C is a multiple of VEC)
+    const int s = token_seq[t], t0 = seq_starts[s];
+    float cur[VEC], prev[VEC];
+    load_row<T, VEC>(x + (size_t)t * ldx + c, cur);
+    if (t > t0) {
+        load_row<T, VEC>(x + (size_t)(t - 1) * ldx + c, prev);
+    } else {
+        float* carried = state + (size_t)slots[s] * C + c;
+        float last[VEC];
+        load_row<T, VEC>(x + (size_t)(seq_starts[s + 1] - 1) * ldx + c, last);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) prev[e] = carried[e];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) carried[e] = last[e];
+    }
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) prev[e] -= cur[e];
+    for (int i = 0; i < n_mix; ++i) {
+        const float* m = mu + (size_t)i * C + c;
+        T* dst = out + ((size_t)i * n_tokens + t) * C + c;
+        float y[VEC];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) y[e] = fmaf(prev[e], m[e], cur[e]);
+        if constexpr (VEC == 8) *(uint4*)dst = make_uint4(pack_bf16(y[0], y[1]), pack_bf16(y[2], y[3]), pack_bf16(y[4], y[5]), pack_bf16(y[6], y[7]));
+        else if constexpr (VEC == 4) *(float4*)dst = make_float4(y[0], y[1], y[2], y[3]);
+        else from_float(dst, y[0]);
+    }
+}
+
+FX_API int fx_token_shift(void* stream, int dtype, const void* x, long ldx, const float* mu, int n_mix, void* out, float* state,
+                          const int* token_seq, const int* seq_starts, const int* slots, int T, int C) {
+    FX_REQUIRE(T >= 0 && T <= 65535 && C > 0 && n_mix >= 1 && ldx >= C, "token_shift: bad sizes T=%d C=%d mixes=%d", T, C, n_mix);
+    FX_REQUIRE(dtype == FX_F32 || dtype == FX_BF16, "token_shift: unknown dtype %d", dtype);
+    FX_REQUIRE(x != out, "token_shift: the output must not be the input (neighbouring rows are read from it)");
+    if (T == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    const int wide = dtype == FX_BF16 ? 8 : 4;
+    const bool vec = C % wide == 0 && ldx % wide == 0 && (((uintptr_t)x | (uintptr_t)out | (uintptr_t)mu | (uintptr_t)state) % 16) == 0;
+    const int per = 256 * (vec ? wide : 1);
+    const dim3 grid((C + per - 1) / per, T);
+#define FX_SHIFT(T_, VEC_) token_shift_kernel<T_, VEC_><<<grid, 256, 0, s>>>((const T_*)x, ldx, mu, n_mix, (T_*)out, state, token_seq, seq_starts, slots, T, C)
+    if (dtype == FX_F32) {
+        if (vec) FX_SHIFT(float, 4);
+        else FX_SHIFT(float, 1);
+    } else {
+        if (vec) FX_SHIFT(bf16, 8);
+        else FX_SHIFT(bf16, 1);
+    }
+#undef FX_SHIFT
+    FX_CHECK_LAUNCH("token_shift");
+    return 0;
+}
+
+// ---------------------------------------------------------------------------
+// A decay per channel from a low-rank projection, all float32:
+//   out[t, n] = exp(-exp(sum_k tanh(low[t, k]) w2t[k, n] + w0[n])),   k ascending in one accumulator
+// low [T, R] rows are the first half's products; w2t [R, N] is the second half's matrix, transposed, so that
+// neighbouring threads read neighbouring columns.  A thread owns a column, a block 256 columns of TT tokens, whose
+// tanh values lie in LDS, KB of the R at a time.  Grid: (ceil(N / 256), ceil(T / TT)).
+// ---------------------------------------------------------------------------
+template <int TT>
+__global__ __launch_bounds__(256) void lowrank_decay_kernel(const float* __restrict__ low, long ldl, const float* __restrict__ w2t,
+                                                            const float* __restrict__ w0, float* __restrict__ out, int n_tokens, int R, int N) {
+    constexpr int KB = 128;
+    __shared__ __attribute__((aligned(16))) float xs[KB][TT];
+    const int n = blockIdx.x * 256 + threadIdx.x, first = blockIdx.y * TT;
+    float acc[TT];
+#pragma unroll
+    for (int i = 0; i < TT; ++i) acc[i] = 0.f;
+    for (int k0 = 0; k0 < R; k0 += KB) {
+        const int kn = min(KB, R - k0);
+        if (k0) __syncthreads();
+        for (int idx = threadIdx.x; idx < TT * kn; idx += 256) {
+            const int i = idx / kn, k = idx - i * kn, t = first + i;
+            xs[k][i] = t < n_tokens ? tanhf(low[(size_t)t * ldl + k0 + k]) : 0.f;
+        }
+        __syncthreads();
+        if (n < N) {
+            const float* w = w2t + (size_t)k0 * N + n;
+#pragma unroll 8
+            for (int k = 0; k < kn; ++k) {
+                const float wv = w[(size_t)k * N];
+#pragma unroll
+                for (int i = 0; i < TT; ++i) acc[i] = fmaf(xs[k][i], wv, acc[i]);
+            }
+        }
+    }
+    if (n >= N) return;
+    const float base = w0[n];
+#pragma unroll
+    for (int i = 0; i < TT; ++i)
+        if (first + i < n_tokens) out[(size_t)(first + i) * N + n] = expf(-expf(acc[i] + base));
+}
+
+FX_API int fx_lowrank_decay(void* stream, const float* low, long ldl, const float* w2t, const float* w0, float* out, int T, int R, int N) {
+    FX_REQUIRE(T >= 0 && R >= 1 && N >= 1 && ldl >= R, "lowrank_decay: bad sizes T=%d R=%d N=%d", T, R, N);
+    FX_REQUIRE(T <= 65535, "lowrank_decay: %d tokens are more than a launch takes", T);
+    if (T == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    if (T <= 64) lowrank_decay_kernel<1><<<dim3((N + 255) / 256, T), 256, 0, s>>>(low, ldl, w2t, w0, out, T, R, N);
+    else lowrank_decay_kernel<16><<<dim3((N + 255) / 256, (T + 15) / 16), 256, 0, s>>>(low, ldl, w2t, w0, out, T, R, N);
+    FX_CHECK_LAUNCH("lowrank_decay");
     return 0;
 }

@@ -92,6 +92,9 @@ def _register_builtin():
     from ..config.panarax import PanaraxConfig
     from .panarax import build_spec as panarax_spec
     register_architecture(Architecture(PanaraxConfig.architecture, PanaraxConfig.model_type, PanaraxConfig, panarax_spec))
+    from ..config.besulix import BesulixConfig
+    from .besulix import build_spec as besulix_spec
+    register_architecture(Architecture(BesulixConfig.architecture, BesulixConfig.model_type, BesulixConfig, besulix_spec))
 
 
 _register_builtin()

@@ -21,7 +21,7 @@ EPI_STORE, EPI_STORE_F32, EPI_RESID, EPI_GATED = 0, 1, 2, 3
 ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "gelu": 2, "relu": 3, "swiglu_clamped": 4}
 # what a stored product (EPI_STORE) may go through on its way out, the activation of a feed-forward without a
 # gate; SACT_* in csrc/gemm.hip
-STORED_ACTIVATIONS = {None: 0, "relu2": 1, "relu": 2, "silu": 3, "gelu_tanh": 4}
+STORED_ACTIVATIONS = {None: 0, "relu2": 1, "relu": 2, "silu": 3, "gelu_tanh": 4, "softcap": 5}
 GATE_SOFTMAX, GATE_SIGMOID = 0, 1
 ROPE_NEOX, ROPE_INTERLEAVED = 0, 1
 
@@ -60,6 +60,11 @@ def _stream():
 
 _sigs = {
     ("elementwise", "fx_embed"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int],
+    ("elementwise", "fx_embed_rmsnorm"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_int, c_float],
+    ("elementwise", "fx_angle_table"): [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int],
+    ("elementwise", "fx_turned_kv_write"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p,
+                                            c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                                            c_void_p, c_void_p],
     ("elementwise", "fx_layernorm"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float, c_long],
     ("elementwise", "fx_gated_add"): [c_void_p, c_void_p, c_void_p, c_void_p, c_long],
     ("elementwise", "fx_gated_add_layernorm"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
@@ -87,6 +92,11 @@ _sigs = {
     ("recurrent", "fx_gated_outer"): [c_void_p, c_void_p, c_long, c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_void_p,
                                       c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
                                       c_float],
+    ("recurrent", "fx_channel_outer"): [c_void_p, c_void_p, c_long, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p,
+                                        c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float],
+    ("recurrent", "fx_token_shift"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
+                                      c_void_p, c_int, c_int],
+    ("recurrent", "fx_lowrank_decay"): [c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int],
     ("recurrent", "fx_exp_gate_scan"): [c_void_p, c_void_p, c_long, c_void_p, c_long, c_float, c_void_p, c_void_p, c_void_p,
                                         c_void_p, c_void_p, c_void_p, c_int, c_int],
     ("recurrent", "fx_rglru_gates"): [c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_float,
@@ -122,13 +132,13 @@ _sigs = {
     ("attention", "fx_attn_tiles"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p,
                                      c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                                      c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int,
-                                     c_int, c_void_p, c_void_p, c_long, c_float, c_void_p, c_int],
+                                     c_int, c_void_p, c_void_p, c_long, c_float, c_void_p, c_int, c_void_p],
     ("attention", "fx_attn_tile_queries"): [c_int, c_int, c_int],
     ("attention", "fx_attn_decode"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p,
                                       c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                       c_int, c_int, c_int, c_int, c_int, c_float,
                                       c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
-                                      c_int, c_void_p, c_void_p, c_long, c_float, c_void_p, c_int],
+                                      c_int, c_void_p, c_void_p, c_long, c_float, c_void_p, c_int, c_void_p],
     ("moe", "fx_router_select"): [c_void_p, c_void_p, c_long, c_long, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
                                   c_void_p, c_void_p, c_void_p, c_void_p],
     ("moe", "fx_router_select_align"): [c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
@@ -183,6 +193,18 @@ def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor | None = Non
         n_pos = position_table.shape[0]
     _call("elementwise", "fx_embed", _stream(), dtype_code(table.dtype), _p(table), _p(_i32(ids, "ids")), _p(out), T, H, V,
           float(scale), _p(position_table), _p(_i32(positions, "positions")) if position_table is not None else None, n_pos)
+    return out
+
+
+def embed_rmsnorm(table: torch.Tensor, ids: torch.Tensor, weight: torch.Tensor, eps: float, scale: float = 1.0) -> torch.Tensor:
+    """h[t] = x / sqrt(mean(x^2) + eps) * weight, x = table[ids[t]] * scale, as float32."""
+    V, H = table.shape
+    T = ids.numel()
+    if weight.numel() != H or not weight.is_contiguous() or not table.is_contiguous():
+        raise KernelError(f"embed_rmsnorm: a norm weight of {weight.numel()} elements for rows of {H}")
+    out = torch.empty((T, H), dtype=torch.float32, device=table.device)
+    _call("elementwise", "fx_embed_rmsnorm", _stream(), dtype_code(table.dtype), _p(table), _p(_i32(ids, "ids")), _p(out), T, H, V,
+          float(scale), _p(weight), dtype_code(weight.dtype), float(eps))
     return out
 
 
@@ -466,6 +488,49 @@ def span_norm_kv_write(qk, q_out, q_weight, k_weight, eps, positions, token_seq,
           int(n_heads), int(n_kv_heads), int(head_dim), int(block_size))
 
 
+def angle_table(positions, n_tokens: int, inv_freq: torch.Tensor) -> torch.Tensor:
+    """float32 [n_tokens, n, 2]: cosine and sine of positions[t] * inv_freq[m] (a float32 product), for `turned_kv_write`
+    and the attention kernels' `turns`."""
+    if inv_freq.dtype != torch.float32 or not inv_freq.is_contiguous() or inv_freq.numel() < 1 or positions.numel() < n_tokens:
+        raise KernelError("angle_table wants contiguous float32 frequencies and a position per token")
+    out = torch.empty((int(n_tokens), inv_freq.numel(), 2), dtype=torch.float32, device=inv_freq.device)
+    _call("elementwise", "fx_angle_table", _stream(), _p(_i32(positions, "positions")), _p(inv_freq), _p(out), int(n_tokens),
+          inv_freq.numel())
+    return out
+
+
+def turned_kv_write(qkv, q_out, positions, token_seq, block_table, k_pages, v_pages, n_heads: int, n_kv_heads: int, head_dim: int,
+                    v_dim: int, block_size: int, rotary_dim: int = 0, interleaved: bool = False, qk_turns=None, v_turns=None,
+                    temperature=None) -> None:
+    """From the float32 product qkv [T, nh*hd | nkv*hd | nkv*vd]: q, its first `rotary_dim` dimensions rotated by the
+    angles of `qk_turns` (an `angle_table` of rotary_dim / 2 angles a token; pairs (i, i + rotary_dim/2), or (2i, 2i+1)
+    when `interleaved`) and every head multiplied by temperature[head] (float32 [nh] or None), into q_out; k, rotated
+    the same way, into its page; v, with `v_turns` every pair (2m, 2m + 1) of a head turned by angle m, into its
+    transposed page (pages None: nothing is cached)."""
+    T = qkv.shape[0]
+    nh, nkv, hd, vd = int(n_heads), int(n_kv_heads), int(head_dim), int(v_dim)
+    _f32_rows(qkv, "turned_kv_write: qkv", (nh + nkv) * hd + nkv * vd)
+    if q_out.dim() != 2 or q_out.stride(1) != 1 or q_out.shape[0] < T or q_out.shape[1] < nh * hd:
+        raise KernelError(f"turned_kv_write: q_out {tuple(q_out.shape)} for {T} rows of {nh * hd}")
+    if (k_pages is None) != (v_pages is None):
+        raise KernelError("turned_kv_write: key and value pages come together")
+    if k_pages is not None and (tuple(k_pages.shape[1:]) != (nkv, block_size, hd) or tuple(v_pages.shape[1:]) != (nkv, vd, block_size)
+                                or k_pages.dtype != q_out.dtype or v_pages.dtype != q_out.dtype):
+        raise KernelError(f"turned_kv_write: pages {tuple(k_pages.shape)}, {tuple(v_pages.shape)} for {nkv} heads of {hd} / {vd}")
+    if rotary_dim and qk_turns is None:
+        raise KernelError(f"turned_kv_write: {rotary_dim} rotated dimensions need a table of angles")
+    _check_turns(qk_turns, T, int(rotary_dim), "turned_kv_write")
+    _check_turns(v_turns, T, vd, "turned_kv_write")
+    if temperature is not None and (temperature.dtype != torch.float32 or temperature.numel() != nh or not temperature.is_contiguous()):
+        raise KernelError(f"turned_kv_write: temperatures must be {nh} contiguous float32 values")
+    if positions.numel() < T or token_seq.numel() < T:
+        raise KernelError("turned_kv_write: the step's index tensors are shorter than its tokens")
+    _call("elementwise", "fx_turned_kv_write", _stream(), dtype_code(q_out.dtype), _p(qkv), qkv.stride(0), _p(q_out), q_out.stride(0),
+          _p(temperature), _p(_i32(positions, "positions")), _p(_i32(token_seq, "token_seq")), _p(_i32(block_table, "block_table")),
+          block_table.shape[1], _p(k_pages), _p(v_pages), T, nh, nkv, hd, vd, int(block_size), int(rotary_dim),
+          1 if interleaved else 0, _p(qk_turns), _p(v_turns))
+
+
 _constant_rows: dict = {}
 
 
@@ -584,7 +649,7 @@ def gemm(a: torch.Tensor, w: torch.Tensor, *, epilogue: int = EPI_STORE, out: to
     `row_ss` = (ss [M, n] float32, eps): row m of the product is scaled by rsqrt(sum(ss[m]) / K + eps)
     before the bias is added (the rows of `a` are a ScaleLater's; plain stored bfloat16 product, M <= 64).
     `store_activation` (one of STORED_ACTIVATIONS, EPI_STORE or EPI_STORE_F32 without bias): the product goes through
-    it before it is stored, e.g. "relu2" = max(x, 0)^2.
+    it before it is stored, e.g. "relu2" = max(x, 0)^2; "softcap" with `activation_params` = (cap, _): cap tanh(x / cap).
     `activation_params` = (limit, alpha) for "swiglu_clamped": g = min(gate, limit), u = clamp(up, -limit, limit),
     stored g sigmoid(alpha g) (u + 1).
     `pre_scale` (EPI_GATED; float32): gate and up of logical row m are multiplied by pre_scale[m] (or by
@@ -751,7 +816,7 @@ def attention_tile_queries(dtype, head_dim: int, block_size: int) -> int:
 def attention_tiles(q, out, k_pages, v_pages, block_table, positions, item_seq, item_tok, item_n,
                     n_heads, n_kv_heads, head_dim, block_size, window, scale, tile_q: int = 64, mask_chunk: int = 0,
                     v_dim: int | None = None, keep_first: int = 0, sinks=None, gate=None, softcap: float = 0.0,
-                    slopes=None, gate_per_head: bool = False) -> None:
+                    slopes=None, gate_per_head: bool = False, turns=None) -> None:
     """Blocks of queries: item i is item_n[i] <= tile_q consecutive tokens of sequence item_seq[i] from token
     item_tok[i] on; tile_q is 64 or attention_tile_queries(...).  `mask_chunk` > 0: the chunked mask (a query sees
     the keys of its own chunk of that many positions) instead of a window.  `v_dim`: size of a value head where it
@@ -759,16 +824,24 @@ def attention_tiles(q, out, k_pages, v_pages, block_table, positions, item_seq, 
     sequence stay visible to every later query.  `sinks` (float32 [n_heads]): a logit per head that joins the
     softmax's denominator and has no value.  `gate` (shape and type of `out`): the output is multiplied by sigmoid(gate).
     `softcap` > 0: a scaled score s becomes softcap * tanh(s / softcap).  `slopes` (float32 [n_heads]): the score of
-    key t for the query at position p then loses slopes[h] * (p - t)."""
+    key t for the query at position p then loses slopes[h] * (p - t).  `turns` (an `angle_table` of v_dim / 2 angles a
+    token): the output pair (2m, 2m + 1) of every head is turned back by the token's angle m, before the gate."""
     _check_attention_shapes(q, out, k_pages, v_pages, n_heads, n_kv_heads, head_dim, int(v_dim or head_dim), block_size)
     _check_attention_extras(out, n_heads, 1 if gate_per_head else int(v_dim or head_dim), window, keep_first, sinks, gate, softcap, slopes)
+    _check_turns(turns, q.shape[0], int(v_dim or head_dim), "attention")
     _call("attention", "fx_attn_tiles", _stream(), dtype_code(q.dtype), _p(q), q.stride(0), _p(out), out.stride(0),
           _p(k_pages), _p(v_pages), _p(_i32(block_table, "block_table")), block_table.shape[1],
           _p(_i32(positions, "positions")), _p(_i32(item_seq, "item_seq")), _p(_i32(item_tok, "item_tok")),
           _p(_i32(item_n, "item_n")), item_seq.numel(), n_heads, n_kv_heads, head_dim, block_size,
           int(window or 0), float(scale), int(tile_q), int(v_dim or head_dim), int(mask_chunk or 0),
           int(keep_first or 0), _p(sinks), _p(gate), gate.stride(0) if gate is not None else 0, float(softcap or 0.0),
-          _p(slopes), 1 if gate_per_head else 0)
+          _p(slopes), 1 if gate_per_head else 0, _p(turns))
+
+
+def _check_turns(turns, n_tokens: int, dims: int, what: str) -> None:
+    if turns is not None and (dims % 2 or turns.dtype != torch.float32 or not turns.is_contiguous() or turns.dim() != 3
+                              or turns.shape[0] < n_tokens or tuple(turns.shape[1:]) != (dims // 2, 2)):
+        raise KernelError(f"{what}: a table of angles {tuple(turns.shape)} for {n_tokens} tokens of {dims} turned dimensions")
 
 
 def _check_attention_extras(out, n_heads, v_dim, window, keep_first, sinks, gate, softcap=0.0, slopes=None) -> None:
@@ -825,7 +898,7 @@ def decode_attention_chunk(n_items: int, n_heads: int, n_kv_heads: int, max_kv_l
 def attention_decode(q, out, k_pages, v_pages, block_table, positions, item_seq, item_tok,
                      n_heads, n_kv_heads, head_dim, block_size, window, scale, max_kv_len, chunk=None,
                      waves=0, mask_chunk: int = 0, v_dim: int | None = None, keep_first: int = 0, sinks=None,
-                     gate=None, softcap: float = 0.0, slopes=None, gate_per_head: bool = False) -> None:
+                     gate=None, softcap: float = 0.0, slopes=None, gate_per_head: bool = False, turns=None) -> None:
     """Single queries.  The keys go to ceil(max_kv_len / chunk) blocks whose results are merged in ascending
     order.  float32 cuts them at multiples of `chunk`, 256 by default (so that a result does not depend on the
     batch); bfloat16, whose blocks of up to eight waves share a chunk, cuts every sequence's own range of keys (from
@@ -835,6 +908,7 @@ def attention_decode(q, out, k_pages, v_pages, block_table, positions, item_seq,
     v_dim = int(v_dim or head_dim)
     _check_attention_shapes(q, out, k_pages, v_pages, n_heads, n_kv_heads, head_dim, v_dim, block_size)
     _check_attention_extras(out, n_heads, 1 if gate_per_head else v_dim, window, keep_first, sinks, gate, softcap, slopes)
+    _check_turns(turns, q.shape[0], v_dim, "attention")
     if chunk is None:
         chunk = 256
         if q.dtype == torch.bfloat16:
@@ -848,7 +922,7 @@ def attention_decode(q, out, k_pages, v_pages, block_table, positions, item_seq,
           n_heads, n_kv_heads, head_dim, block_size, int(window or 0), float(scale),
           _p(part_o), _p(part_ml), splits, chunk, int(waves), v_dim, int(mask_chunk or 0),
           int(keep_first or 0), _p(sinks), _p(gate), gate.stride(0) if gate is not None else 0, float(softcap or 0.0),
-          _p(slopes), 1 if gate_per_head else 0)
+          _p(slopes), 1 if gate_per_head else 0, _p(turns))
 
 
 def router_select(logits, n_experts, top_k, renorm, gating=GATE_SOFTMAX, has_gate=False, selection_bias=None,
@@ -1179,6 +1253,64 @@ def gated_outer(q, k, v, keep, take, state, seq_starts, slot_ids, n_seqs: int, n
           1 if keep_const else 0, _p(take), _p(out), out.stride(0), _p(nq), _p(state), _p(_i32(seq_starts, "seq_starts")),
           _p(_i32(slot_ids, "slot_ids")), int(n_seqs), H, G, D, V, float(q_scale))
     return (out, nq) if normalizer else out
+
+
+def channel_outer(q, k, v, keep, bonus, state, seq_starts, slot_ids, n_seqs: int, n_heads: int, key_dim: int, v_dim: int,
+                  q_scale: float = 1.0) -> torch.Tensor:
+    """A matrix memory with one forgetting factor per key channel and a bonus for the current token, over each sequence's
+    tokens in order, from and into state[slot] (float32 [slots, H, V, D], transposed as in `gated_outer`):
+        o_t = q_scale (S + diag(bonus) k_t v_t^T)^T q_t;   S <- diag(keep_t) S + k_t v_t^T
+    q, k [T, H*D], v [T, H*V] float32 rows; keep float32 contiguous [T, H*D]; bonus float32 [H, D].  Returns o [T, H*V]."""
+    T = q.shape[0]
+    H, D, V = int(n_heads), int(key_dim), int(v_dim)
+    _f32_rows(q, "channel_outer: q", H * D), _f32_rows(k, "channel_outer: k", H * D), _f32_rows(v, "channel_outer: v", H * V)
+    if keep.dtype != torch.float32 or not keep.is_contiguous() or tuple(keep.shape) != (T, H * D) or k.shape[0] != T or v.shape[0] != T:
+        raise KernelError(f"channel_outer: forgetting factors {tuple(keep.shape)} for {T} tokens of {H} heads of {D}")
+    if bonus.dtype != torch.float32 or not bonus.is_contiguous() or bonus.numel() != H * D:
+        raise KernelError(f"channel_outer: a bonus of {bonus.numel()} elements for {H} heads of {D}")
+    if state.dtype != torch.float32 or not state.is_contiguous() or tuple(state.shape[1:]) != (H, V, D):
+        raise KernelError(f"channel_outer: state {tuple(state.shape)} for [slots, {H}, {V}, {D}]")
+    if seq_starts.numel() < n_seqs + 1 or slot_ids.numel() < n_seqs:
+        raise KernelError("channel_outer: the step's index tensors are shorter than its sequences")
+    out = torch.empty((T, H * V), dtype=torch.float32, device=q.device)
+    _call("recurrent", "fx_channel_outer", _stream(), _p(q), q.stride(0), _p(k), k.stride(0), _p(v), v.stride(0), _p(keep), _p(bonus),
+          _p(out), out.stride(0), _p(state), _p(_i32(seq_starts, "seq_starts")), _p(_i32(slot_ids, "slot_ids")), int(n_seqs),
+          H, H, D, V, float(q_scale))
+    return out
+
+
+def token_shift(x, mu, state, token_seq, seq_starts, slot_ids) -> torch.Tensor:
+    """out[i, t] = x[t] + (x'[t] - x[t]) * mu[i], x'[t] the row before t in its sequence: row t - 1 of the step, or, for a
+    portion's first row, what state[slot] (float32 [slots, C]) carried; afterwards the state holds the portion's last row.
+    x [T, C] rows of either type, mu float32 [n, C]; returns [n, T, C] of x's type."""
+    T, C = x.shape
+    if x.stride(1) != 1 or mu.dtype != torch.float32 or mu.dim() != 2 or mu.shape[1] != C or not mu.is_contiguous():
+        raise KernelError(f"token_shift: mixes {tuple(mu.shape)} ({mu.dtype}) for rows of {C}")
+    if state.dtype != torch.float32 or not state.is_contiguous() or tuple(state.shape[1:]) != (C,):
+        raise KernelError(f"token_shift: state {tuple(state.shape)} for [slots, {C}]")
+    if token_seq.numel() < T:
+        raise KernelError("token_shift: the step's index tensors are shorter than its tokens")
+    n = mu.shape[0]
+    out = torch.empty((n, T, C), dtype=x.dtype, device=x.device)
+    _call("recurrent", "fx_token_shift", _stream(), dtype_code(x.dtype), _p(x), x.stride(0), _p(mu), n, _p(out), _p(state),
+          _p(_i32(token_seq, "token_seq")), _p(_i32(seq_starts, "seq_starts")), _p(_i32(slot_ids, "slot_ids")), T, C)
+    return out
+
+
+def lowrank_decay(low, w2t, w0) -> torch.Tensor:
+    """exp(-exp(tanh(low) w2t + w0)), float32 [T, N]: low float32 rows [T, R], w2t float32 [R, N] (the matrix transposed),
+    w0 float32 [N]."""
+    T = low.shape[0]
+    R, N = w2t.shape
+    _f32_rows(low, "lowrank_decay: low", R)
+    for t in (w2t, w0):
+        if t.dtype != torch.float32 or not t.is_contiguous():
+            raise KernelError("lowrank_decay: weights are contiguous float32")
+    if w0.numel() != N:
+        raise KernelError(f"lowrank_decay: {w0.numel()} offsets for {N} channels")
+    out = torch.empty((T, N), dtype=torch.float32, device=low.device)
+    _call("recurrent", "fx_lowrank_decay", _stream(), _p(low), low.stride(0), _p(w2t), _p(w0), _p(out), T, R, N)
+    return out
 
 
 def exp_gate_scan(x_in, x_forget, cap: float, state, seq_starts, slot_ids, n_seqs: int, n_heads: int):

@@ -64,7 +64,7 @@ class PagedAttention(Mixer):
     takes_post_norm = True     # forward(..., post_norm=(weight, eps)) norms the output rows before they join the stream
     TENSORS = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
                "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias",
-               "q_norm": "q_norm.", "k_norm": "k_norm.", "sink": "sinks", "gate": "gate_proj.weight"}
+               "q_norm": "q_norm.", "k_norm": "k_norm.", "sink": "sinks", "gate": "gate_proj.weight", "temperature": "temperature"}
 
     def __init__(self, hidden_size: int, n_heads: int, n_kv_heads: int, head_dim: int, bias: bool,
                  position: PartSpec, window: int | None = None, scale: float | None = None,
@@ -72,7 +72,8 @@ class PagedAttention(Mixer):
                  names: dict | None = None, keep_first: int = 0, sink: bool = False, out_gate: bool = False,
                  own_kv: bool = True, retain: tuple | None = None, softcap: float | None = None,
                  distance_slopes=None, values_from_keys: bool = False, qk_norm_span: str = "head",
-                 q_temperature: tuple | None = None, unit_values: float | None = None):
+                 q_temperature: tuple | None = None, unit_values: float | None = None, head_temperature: bool = False,
+                 value_rotation: float | None = None):
         """`qk_norm`: kind and arguments of a norm over head_dim; two of them are built, with tensors under
         `q_norm.` and `k_norm.`, and applied to every head of q and of k before the rotation.
         `v_dim`: size of a value head where it differs from head_dim (the size of a query and key head).
@@ -86,6 +87,11 @@ class PagedAttention(Mixer):
         projection (W_g: [n_heads * v_dim, hidden]); "head": one gate per head, W_g: [n_heads, hidden].
         `q_temperature` = (coef, every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1),
         which is how positions enter the scores of such a mixer (it rotates nothing).
+        `head_temperature`: a learned number per head ([n_heads]) multiplies that head's scores (not its sink).
+        `value_rotation` (a base): every value head is turned by its key's position over all of its v_dim dimensions, pair
+        m by pos * base^(-2m / v_dim), pairs laid out as the key rotation's (halves of the head, or neighbours), and cached
+        so; every head's output is turned back by the query's position.  What a key hands to a query then depends on how
+        far apart the two are.
         `unit_values` (an eps): every value head is divided by its root mean square over v_dim (eps inside the root,
         no weight) and cached so.
         `own_kv` False: the mixer has no key and value projections and writes no cache; its schedule entry reads
@@ -123,6 +129,15 @@ class PagedAttention(Mixer):
         self.prepares = self.q_temperature is not None or self.unit_values is not None
         if self.prepares and (bias or qk_norm is not None or values_from_keys or not own_kv):
             raise ValueError("a query temperature and unit values go with projections of q, k and v without biases and head norms")
+        # temperatures per head or turned values: float32 arithmetic on the product's rows in the launch that writes the
+        # cache, from tables of angles that the step's layers share
+        self.head_temperature = bool(head_temperature)
+        self.value_rotation = float(value_rotation) if value_rotation is not None else None
+        self.turns = self.head_temperature or self.value_rotation is not None
+        if self.turns and (self.prepares or qk_norm is not None or values_from_keys or not own_kv or out_gate):
+            raise ValueError("head temperatures and turned values go with plain projections of q, k and v")
+        if self.value_rotation is not None and not self.value_rotation > 0:
+            raise ValueError(f"the base of the values' rotation must be positive, got {value_rotation}")
         if self.chunk and (retain is not None or keep_first):
             raise ValueError("kept first keys and a retention of their own go with a window, not with a chunked mask")
         # (None, 0): every key is kept; (W, F): the last W and the first F
@@ -131,6 +146,8 @@ class PagedAttention(Mixer):
             raise ValueError(f"a cache that keeps the last {self.retain[0]} and the first {self.retain[1]} keys does not hold "
                              f"what a window of {self.window} with {self.keep_first} kept keys sees")
         self.v_dim = int(v_dim) if v_dim else head_dim
+        if self.value_rotation is not None and self.v_dim % 2:
+            raise ValueError(f"turned values come in pairs: v_dim {self.v_dim} must be even")
         self.softcap = float(softcap) if softcap else 0.0
         if not 0.0 <= self.softcap < math.inf:
             raise ValueError(f"a cap of {softcap} on the scores")
@@ -162,7 +179,7 @@ class PagedAttention(Mixer):
             self.kvw = self.vw = 0       # (no rows of k and v in the mixer's matrix)
         if self.values_from_keys:
             self.vw = 0                  # (no rows of v: the key rows are the values)
-        self.qkv = self.o_proj = self.sinks = self.slopes = None
+        self.qkv = self.o_proj = self.sinks = self.slopes = self.temperature = self.value_frequencies = None
         self.q_norm = self.k_norm = None
         if qk_norm is not None and self.span_norms:
             self.q_norm = NORMS.build(PartSpec(qk_norm.kind, dict(qk_norm.args, size=self.qw)))
@@ -173,6 +190,8 @@ class PagedAttention(Mixer):
             self.q_norm, self.k_norm = (NORMS.build(PartSpec(qk_norm.kind, dict(qk_norm.args))) for _ in range(2))
         if self.prepares and (self.position.rotary() is None or self.position.rotary().rotary_dim):
             raise ValueError("a query temperature and unit values go with a mixer that rotates nothing")
+        if self.turns and (self.position.rotary() is None or self.position.rotary().freq_factors is not None):
+            raise ValueError("head temperatures and turned values go with a rotation given by its frequencies")
         if (self.position.rotary() or Rotary(0, 1.0)).magnitude != 1.0:
             raise ValueError("this mixer's rotation kernels turn and do not stretch: a rotation's magnitude must be 1")
         if bias and out_gate:
@@ -194,6 +213,8 @@ class PagedAttention(Mixer):
                           n["v_bias"]: ParamSpec((self.vw,))})
         if self.has_sink:
             specs[n["sink"]] = ParamSpec((self.n_heads,))
+        if self.head_temperature:
+            specs[n["temperature"]] = ParamSpec((self.n_heads,), init="ones")
         if self.out_gate:
             specs[n["gate"]] = ParamSpec((self.n_heads if self.gate_per_head else self.ow, H))
         return specs
@@ -208,12 +229,50 @@ class PagedAttention(Mixer):
         b = None
         if self.bias:
             b = torch.cat(same_dtype([fetch(n["q_bias"]), fetch(n["k_bias"]), fetch(n["v_bias"])]), dim=0)
+        o = fetch(n["o"])
+        if self.value_rotation is not None:
+            # pairs of value channels lie side by side in the pages: pairs that are halves of a head are brought together
+            # by the order of W_v's rows, and W_o reads its columns in that order
+            order = self.value_pair_order()
+            cut = self.qw + self.kvw
+            v_rows = torch.cat([order + g * self.v_dim for g in range(self.n_kv_heads)]).to(w.device)
+            w = torch.cat([w[:cut], w[cut:][v_rows]], dim=0)
+            if b is not None:
+                b = torch.cat([b[:cut], b[cut:][v_rows]], dim=0)
+            o = o[:, torch.cat([order + h * self.v_dim for h in range(self.n_heads)]).to(w.device)]
+            self.value_frequencies = ops.rotary_frequencies(w.device, self.v_dim, self.value_rotation)
         self.qkv = Linear(w, b)
-        self.o_proj = Linear(fetch(n["o"]))
+        self.o_proj = Linear(o)
+        if self.head_temperature:
+            self.temperature = fetch(n["temperature"]).float().contiguous()
         if self.has_sink:
             self.sinks = fetch(n["sink"]).float().contiguous()
         if self.distance_slopes is not None:
             self.slopes = torch.tensor(self.distance_slopes, dtype=torch.float64).to(torch.float32).to(w.device)
+
+    def value_pair_order(self) -> torch.Tensor:
+        """Element i of a value head as the pages hold it is element order[i] of the head as the checkpoint has it."""
+        if self.position.rotary().interleaved:
+            return torch.arange(self.v_dim)
+        return torch.arange(self.v_dim).view(2, self.v_dim // 2).t().reshape(-1)
+
+    def turned_heads_and_cache(self, x, ctx, table, cache, rot):
+        """q [T, qw], rotated and multiplied by the heads' temperatures, with k (rotated) and v (turned, where values are)
+        in their pages; one launch behind a float32 product.  Also the table of the values' angles, or None."""
+        rows = matmul(x, self.qkv.weight, bias=self.qkv.bias, epilogue=ops.EPI_STORE_F32)
+        q = torch.empty((ctx.n_tokens, self.qw), dtype=ctx.act_dtype, device=rows.device)
+        debug.region("rope + cache write")
+        qk_turns = v_turns = None
+        if rot.rotary_dim:
+            freq = ops.rotary_frequencies(rows.device, rot.rotary_dim, rot.theta, rot.frequencies)
+            qk_turns = ctx.memo(("angles", freq.data_ptr()), lambda: ops.angle_table(ctx.positions, ctx.n_tokens, freq))
+        if self.value_rotation is not None:
+            v_turns = ctx.memo(("angles", self.value_frequencies.data_ptr()),
+                               lambda: ops.angle_table(ctx.positions, ctx.n_tokens, self.value_frequencies))
+        ops.turned_kv_write(rows, q, ctx.positions, ctx.token_seq, table, cache.pages["k"] if cache.writes else None,
+                            cache.pages["v"] if cache.writes else None, self.n_heads, self.n_kv_heads, self.head_dim, self.v_dim,
+                            cache.block_size, rot.rotary_dim, rot.interleaved, qk_turns, v_turns, self.temperature)
+        return q, v_turns
 
     def normed_spans_and_cache(self, x, ctx, table, cache):
         """As `normed_heads_and_cache` for norms over the whole projection: q [T, qw] normed over all its columns, the
@@ -254,7 +313,7 @@ class PagedAttention(Mixer):
         # (heads that are normed again take their q and k from a float32 product; the norm inside two products, one
         # of them stored in float32, was measured and is behind the norm kernel: every block norms all rows)
         if (ctx.act_dtype != torch.bfloat16 or rms is None or residual.shape[0] > 16 or self.q_norm is not None
-                or self.prepares or not self.own_kv or not ops.can_fuse_norm(residual, self.qkv.weight, residual.shape[0])):
+                or self.prepares or self.turns or not self.own_kv or not ops.can_fuse_norm(residual, self.qkv.weight, residual.shape[0])):
             return False
         debug.region("qkv")
         qkv = ops.gemm(residual, self.qkv.weight, bias=self.qkv.bias, norm=rms)
@@ -264,7 +323,7 @@ class PagedAttention(Mixer):
     def takes_scale_later(self, act_dtype) -> bool:
         """Whether forward takes an ops.ScaleLater as x (the block before then leaves its rows that way)."""
         w = self.qkv.weight
-        return (self.q_norm is None and not self.prepares and self.own_kv and act_dtype == torch.bfloat16 and w.dtype == torch.bfloat16
+        return (self.q_norm is None and not self.prepares and not self.turns and self.own_kv and act_dtype == torch.bfloat16 and w.dtype == torch.bfloat16
                 and w.shape[1] % 8 == 0 and w.data_ptr() % 16 == 0)
 
     def tile_queries(self, ctx, dtype, block_size: int) -> int:
@@ -353,7 +412,8 @@ class PagedAttention(Mixer):
         k_pages, v_pages = cache.pages["k"], cache.pages["v"]
         rot = self.position.rotary()
         debug.region("qkv")
-        fused = (qkv is None and self.q_norm is None and rot is not None and rot.frequencies is None and not self.prepares
+        v_turns = None
+        fused = (qkv is None and self.q_norm is None and rot is not None and rot.frequencies is None and not self.prepares and not self.turns
                  and self.v_dim == self.head_dim and self.own_kv and not self.out_gate
                  and ops.can_qkv_rope(x, self.qkv.weight, ctx.n_tokens, self.head_dim, rot.rotary_dim, rot.interleaved))
         if fused:
@@ -366,7 +426,10 @@ class PagedAttention(Mixer):
         else:
             gate = None
             wrote = False
-            if self.prepares:
+            if self.turns:
+                q, v_turns = self.turned_heads_and_cache(x, ctx, table, cache, rot)
+                qkv, k, v, wrote = q, None, None, True
+            elif self.prepares:
                 # one float32 product, then one launch: q times its position's temperature, the gate's columns behind
                 # it, k into its page, v (of unit size) into its page
                 n_gate = (self.n_heads if self.gate_per_head else self.ow) if self.out_gate else 0
@@ -422,7 +485,7 @@ class PagedAttention(Mixer):
         # (the gate multiplies the heads' outputs as the attention kernels write them)
         mask = dict(mask_chunk=self.chunk or 0, v_dim=self.v_dim, keep_first=self.keep_first, sinks=self.sinks,
                     gate=None if fused else gate, softcap=self.softcap, slopes=self.slopes,
-                    gate_per_head=self.gate_per_head and gate is not None)
+                    gate_per_head=self.gate_per_head and gate is not None, turns=v_turns)
         if items["n_tiles"]:
             ops.attention_tiles(q, out, k_pages, v_pages, table, ctx.positions,
                                 items["tile_seq"], items["tile_tok"], items["tile_n"], *common, tile_q=tile_q, **mask)

@@ -15,12 +15,15 @@ class GatedMLP(FeedForward):
     kernel_libraries = ("gemm",)
     TENSORS = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
 
-    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu", names: dict | None = None):
-        """`names`: what the checkpoint calls the three matrices, where that differs from `TENSORS`."""
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu", names: dict | None = None,
+                 activation_params: tuple = (0.0, 0.0)):
+        """`names`: what the checkpoint calls the three matrices, where that differs from `TENSORS`.
+        `activation_params`: the numbers of an activation that has some (`ops.gemm`)."""
         if activation not in ops.ACTIVATIONS:
             raise ValueError(f"activation '{activation}' is not one of {sorted(ops.ACTIVATIONS)}")
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.activation = activation
+        self.activation_params = tuple(float(p) for p in activation_params)
         self.names = dict(self.TENSORS, **(names or {}))
         self.gate_up = self.down = None
 
@@ -35,13 +38,16 @@ class GatedMLP(FeedForward):
 
     def output(self, x):
         """The feed-forward's output as float32 [T, H], added to nothing."""
-        return self.down(self.gate_up(x, epilogue=ops.EPI_GATED, activation=self.activation), epilogue=ops.EPI_STORE_F32)
+        return self.down(self._act(x), epilogue=ops.EPI_STORE_F32)
+
+    def _act(self, x):
+        return self.gate_up(x, epilogue=ops.EPI_GATED, activation=self.activation, activation_params=self.activation_params)
 
     takes_fresh = True       # forward(..., fresh=True): `residual` holds nothing yet, the output is stored into it
 
     def forward(self, x, ctx, residual, row_scale=None, fresh: bool = False) -> None:
         debug.region("mlp gate/up")
-        act = self.gate_up(x, epilogue=ops.EPI_GATED, activation=self.activation)
+        act = self._act(x)
         debug.region("mlp down")
         if fresh and row_scale is None:
             self.down(act, epilogue=ops.EPI_STORE_F32, out=residual)
