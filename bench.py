@@ -6,7 +6,8 @@
     python bench.py --kernel-table decode_b1|decode_b8|decode_b16|..|decode_b64|prefill_128|prefill_512|prefill_2048|prefill_4096 [--out FILE]
                                                                  per-kernel times under rocprofv3 (a child process)
     python bench.py --compare-designs [--design TEXT] [--design-size 1k|2k]
-                                                                 four layers of each other design (Rafilix, Kovalorn, Fokinex, Panarax)
+                                                                 four layers of each other design (Rafilix, Kovalorn, Fokinex, Panarax,
+                                                                 Besulix)
                                                                  beside the closest models at equal sizes: prefill and decode
 
 Model: the layer sizes of Qwen1.5-MoE-A2.7B with seeded random bf16 weights
@@ -408,7 +409,7 @@ def run_workload(name: str, args) -> int:
     return 0
 
 
-# ---- Rafilix, Kovalorn, Fokinex and Panarax beside the closest existing model, at equal layer sizes ----------------------------------
+# ---- Rafilix, Kovalorn, Fokinex, Panarax and Besulix beside the closest existing model, at equal layer sizes ----------------------------------
 # Layer sizes that resemble a real model's; every model is four layers of random weights.  The Rafilix layers are
 # measured by kind (all attention, all recurrent) and in the design's usual mixture, the Qwen2-MoE layers have the
 # same width, heads, experts and expert width and no shared expert (Rafilix has none).
@@ -500,9 +501,27 @@ def design_configs(s: dict) -> dict:
         layers = [{"type": kind, "mixer": mixers[kind], "mlp": experts if i in sparse else dense} for i, kind in enumerate(kinds)]
         return {"architecture": "Panarax", "vocab": s["vocab"], "width": s["width"], "max_positions": 16384, "norm": {"eps": 1e-5},
                 "canon": {"taps": 4}, "layers": layers}
+    # Besulix: chunked attention with turned values beside a time-mixing recurrence (heads of 64), or a matrix memory,
+    # with dense feed-forwards that clamp gate and up; in the mixed variant the memory layers have no feed-forward.
+    # Beside it (above): Panarax's and Fokinex's side-by-side layers and Kovalorn's attention with the same dense
+    # feed-forward, Rafilix's delta-rule layers.
+    def besulix(kinds, bare=()):
+        H, D = s["heads"], s["dim"]
+        mixers = {
+            "parallel": {"left": {"heads": H, "kv_heads": s["kv_heads"], "dim": D, "vdim": D, "scale": D ** -0.5,
+                                  "rot": {"base": 500000.0, "dims": D // 2}, "mask": {"size": 8192}},
+                         "right": {"heads": s["width"] // 64, "dim": 64, "decay_rank": 64}, "left_scale": 0.7, "right_scale": 0.7},
+            "mlstm": {"heads": H, "dim": D, "vdim": D, "gate_cap": 15.0},
+        }
+        dense = {"kind": "dense", "ff": s["dense_ff"], "limit": 7.0}
+        return {"architecture": "Besulix", "vocab": s["vocab"], "width": s["width"], "max_positions": 16384, "norm": {"eps": 1e-5},
+                "logit_softcap": 30.0, "layers": [{"type": kind, "mixer": mixers[kind], "mlp": None if i in bare else dense}
+                                                  for i, kind in enumerate(kinds)]}
     more = {"panarax lightning": panarax(["lightning"] * 4), "panarax lru": panarax(["rglru"] * 4),
             "panarax side by side": panarax(["parallel"] * 4), "panarax experts": panarax(["lightning"] * 4, sparse=(0, 1, 2, 3)),
             "panarax mixed": panarax(["lightning", "rglru", "parallel", "lightning"], sparse=(1, 3)),
+            "besulix side by side": besulix(["parallel"] * 4), "besulix memory": besulix(["mlstm"] * 4),
+            "besulix mixed": besulix(["parallel", "mlstm", "parallel", "mlstm"], bare=(1, 3)),
             "kovalorn dense": kovalorn_dense(), "fokinex latent": fokinex(["latent"] * 4),
             "fokinex side by side": fokinex(["parallel"] * 4),
             "fokinex mixed": fokinex(["latent", "latent", "reader", "parallel"])}

@@ -64,6 +64,24 @@ __global__ __launch_bounds__(256) void embed_rmsnorm_kernel(const W* __restrict_
     }
     const W* row = table + (size_t)id * H;
     float ss = 0.f;
+    if (H <= 256 * 16) {           // the row stays in registers; the weights are fetched meanwhile
+        float xv[16], wv[16];
+        load_strided_typed<W, 16, 256>(row, threadIdx.x, H, xv);
+        load_strided_as_float<16, 256>(w, w_dtype, threadIdx.x, H, wv);
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            xv[i] *= scale;
+            ss = fmaf(xv[i], xv[i], ss);
+        }
+        ss = block_sum<4>(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)H + eps);
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int c = threadIdx.x + i * 256;
+            if (c < H) h[(size_t)t * H + c] = xv[i] * inv * wv[i];
+        }
+        return;
+    }
     for (int c = threadIdx.x; c < H; c += 256) {
         const float x = to_float(row[c]) * scale;
         ss = fmaf(x, x, ss);

@@ -1479,7 +1479,11 @@ FX_API int fx_gemm(void* stream, int dtype, int epi, const void* A, long lda, co
     // 11 us up to 128 rows and 18 us up to 256 against 20-24 us; 3,584 x 3,584: 26-30 us up to 128 rows against 31-39;
     // with 48 tiles, the q/k/v product, the tiled kernel is ahead)
     const bool few_tiles = !expert_offsets && !pair_ids && M > 64 && M <= 256 && (long)ceil_div(N, 128) * ceil_div(M, 128) <= 32 && !g_wide_force;
-    const long plain_limit = g_plain_rows > 0 ? g_plain_rows : (few_tiles ? 256 : 64);
+    // More rows against very few weight rows (a low-rank projection, a router): tiles of 128 rows leave most CUs idle
+    // through the whole chain of K steps, the product for few rows covers them (2,048 rows of K = 2,048 against 64 weight
+    // rows: 9 against 24 us, against 256: 18 against 25 us; against 512 it falls behind)
+    const bool narrow = !expert_offsets && !pair_ids && M > 256 && (long)M * N <= 524288 && !g_wide_force;
+    const long plain_limit = g_plain_rows > 0 ? g_plain_rows : (few_tiles ? 256 : (narrow ? M : 64));
     const long few_limit = expert_offsets ? (wide_ok ? g_few_rows : 64) : plain_limit;
     if (g.vec_ok && (per_group <= few_limit || pair_ids) && !many_columns) {
         int mt = pair_ids ? 1 : (per_group <= 16 ? 1 : (per_group <= 32 ? 2 : 4));

@@ -550,59 +550,142 @@ FX_API int fx_gated_head_norm(void* stream, int out_dtype, const float* o, long 
 // decay; the matrix memory of an LSTM with exponential gates):
 //   S <- keep_t S + take_t k_t v_t^T;   o_t = q_scale S^T q_t           S: [D, V] per head, float32
 // keep [T, H] (or, with keep_const, [H]: the same factor at every token) and take [T, H] (null: 1) are float32.
-// With `normalizer`, the state has one more column, n <- keep_t n + take_t k_t, and nq[t, h] = q_scale n_t . q_t
+// With `nq` (a normaliser), the state has one more column, n <- keep_t n + take_t k_t, and nq[t, h] = q_scale n_t . q_t
 // leaves beside o: it is column V of a state [slot][head][V + 1][D], computed as a column whose value is always 1.
-// Lanes, columns, the state's transposed layout, the groups of P tokens that a block of waves brings into LDS a
-// group ahead: as in the delta rule's kernel above; a token's work is one pass over the lane's rows (S updated,
-// then its part of S^T q) and one sum over the lanes of a column.
 // CHANNEL: one forgetting factor per key channel instead, and a read-out that comes before the update, with a bonus
 // u [H, D] that the current token alone gets:
 //   o_t = q_scale (S + diag(u) k_t v_t^T)^T q_t;   S <- diag(keep_t) S + k_t v_t^T            keep: [T, H, D]
 // (the factors travel through LDS beside k and q; no writing factors, no normaliser).
-// Grid: (ceil((V + normalizer) / (NW 64 / LPC)), heads, sequences).
+// Lanes, columns, the state's transposed layout, the groups of P tokens that a block of waves brings into LDS a
+// group ahead: as in the delta rule's kernel above; a token's work is one pass over the lane's rows (S updated, and
+// its part of S^T q) and one sum over the lanes of a column.
+//
+// A long portion is a long chain of tokens on few waves, so it may be cut into `segs` segments that run at once: PASS 1
+// takes every segment but the last from zero (the first from the carried state) to its local state, with the product
+// of its forgetting factors; PASS 2 puts a segment's start together from the segments before it,
+//   S_g = K_(g-1) S_(g-1) + L_(g-1),   K a segment's product of factors, L its local state,
+// and runs it with its outputs.  Twice the updates, a `segs`-th of the chain.  PASS 0 is the one-launch form.
+// `part` [sequence][segs][H][VS][D]: the carried state, then the local states; `prod` [sequence][segs][H][D or 1].
+// Grid: (ceil(VS / (NW 64 / LPC)), heads, sequences x (1, segs - 1 or segs)).
 // ---------------------------------------------------------------------------
-template <int DR, int LPC, bool VEC, int NW, bool CHANNEL>
-__global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __restrict__ q, long ldq, const float* __restrict__ k, long ldk,
-                                                              const float* __restrict__ v, long ldv, const float* __restrict__ keep,
-                                                              int keep_const, const float* __restrict__ take, float* __restrict__ out,
-                                                              long ldo, float* __restrict__ nq, float* __restrict__ state,
-                                                              const int* __restrict__ seq_starts, const int* __restrict__ slots,
-                                                              int H, int G, int D, int V, int VS, float q_scale, const float* __restrict__ bonus) {
+struct OuterArgs {
+    const float* q;
+    const float* k;
+    const float* v;
+    long ldq, ldk, ldv, ldo;
+    const float* keep;
+    const float* take;
+    const float* bonus;
+    float* out;
+    float* nq;
+    float* state;
+    const int* seq_starts;
+    const int* slots;
+    float* part;
+    float* prod;
+    int keep_const, segs, H, G, D, V, VS;
+    float q_scale;
+};
+#define OUTER_GROUP 8            // tokens that travel together
+#define OUTER_MIN_SEGMENT 64     // the fewest tokens of a segment that is not a sequence's last
+__host__ __device__ __forceinline__ int outer_segment(int n, int segs) {      // tokens of a segment of an n-token portion
+    const int per = ((n + segs - 1) / segs + OUTER_GROUP - 1) / OUTER_GROUP * OUTER_GROUP;
+    return per > OUTER_MIN_SEGMENT ? per : OUTER_MIN_SEGMENT;
+}
+
+template <int DR, int LPC, bool VEC, int NW, bool CHANNEL, int PASS>
+__global__ __launch_bounds__(NW * 64) void gated_outer_kernel(OuterArgs a) {
     constexpr int DP = LPC * DR;                     // rows as a wave holds them
     constexpr int W = VEC ? 4 : 1;                   // floats per load
-    constexpr int P = 8;                             // tokens that travel together
+    constexpr int P = OUTER_GROUP;
     constexpr int NT = NW * 64;
-    constexpr int OPS = CHANNEL ? 3 : 2;
-    constexpr int PIECES = OPS * DP / W;             // loads that bring one token's (k | q), or (k | q | keep)
+    constexpr int OPS = (PASS == 1 ? 1 : 2) + (CHANNEL ? 1 : 0);      // k (, q) (, keep)
+    constexpr int PIECES = OPS * DP / W;             // loads that bring one token's operands
     constexpr int NL = (P * PIECES + NT - 1) / NT;   // loads a thread makes per group
     constexpr int COLS = 64 / LPC;
     static_assert(DR % 4 == 0, "a lane's rows are read from LDS in 16-byte pieces");
-    __shared__ __attribute__((aligned(16))) float kq[2][P][OPS][DP];      // two groups of P tokens x (k, q (, keep))
+    __shared__ __attribute__((aligned(16))) float kq[2][P][OPS][DP];      // two groups of P tokens
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int r = lane % LPC, j = (blockIdx.x * NW + wave) * COLS + lane / LPC;
-    const int h = blockIdx.y, s = blockIdx.z, g = h / (H / G);
-    const int t0 = seq_starts[s], t1 = seq_starts[s + 1];
+    const int H = a.H, D = a.D, V = a.V, VS = a.VS;  // VS = V (+ 1: the normaliser's column, whose value is 1)
+    const int runs = PASS == 0 ? 1 : (PASS == 1 ? a.segs - 1 : a.segs);
+    const int h = blockIdx.y, s = blockIdx.z / runs, seg = blockIdx.z - s * runs, g = h / (H / a.G);
+    int t0 = a.seq_starts[s], t1 = a.seq_starts[s + 1];
+    const int t_end = t1;
+    if constexpr (PASS != 0) {
+        const int per = outer_segment(t1 - t0, a.segs);
+        t0 += seg * per;
+        t1 = min(t0 + per, t_end);
+        if (PASS == 1 && t1 >= t_end) return;        // the last segment's local state is nobody's start
+    }
     if (t1 <= t0) return;                            // (the same in every thread of the block)
-    const bool col = j < VS, ones = j == V;          // VS = V (+ 1: the normaliser's column, whose value is 1)
-    float* S_g = state + (((size_t)slots[s] * H + h) * VS + (col ? j : 0)) * D + r * DR;
-    float S[DR];
+    const bool col = j < VS, ones = j == V;
+    auto load_rows = [&](const float* p, float (&x)[DR]) {      // this lane's rows of a [D] column; zeros past D
 #pragma unroll
-    for (int i = 0; i < DR; i += 4) {
-        if constexpr (VEC) {
-            const bool in = col && r * DR + i < D;      // (D % 4 == 0: a piece is inside or outside as a whole)
-            const float4 x = in ? *(const float4*)(S_g + i) : make_float4(0.f, 0.f, 0.f, 0.f);
-            S[i] = x.x; S[i + 1] = x.y; S[i + 2] = x.z; S[i + 3] = x.w;
+        for (int i = 0; i < DR; i += 4) {
+            if constexpr (VEC) {
+                const bool in = col && r * DR + i < D;      // (D % 4 == 0: a piece is inside or outside as a whole)
+                const float4 y = in ? *(const float4*)(p + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+                x[i] = y.x; x[i + 1] = y.y; x[i + 2] = y.z; x[i + 3] = y.w;
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[i + e] = (col && r * DR + i + e < D) ? p[i + e] : 0.f;
+            }
+        }
+    };
+    auto store_rows = [&](float* p, const float (&x)[DR]) {
+#pragma unroll
+        for (int i = 0; i < DR; i += 4) {
+            if constexpr (VEC) {
+                if (col && r * DR + i < D) *(float4*)(p + i) = make_float4(x[i], x[i + 1], x[i + 2], x[i + 3]);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (col && r * DR + i + e < D) p[i + e] = x[i + e];
+            }
+        }
+    };
+    const size_t at = ((size_t)h * VS + (col ? j : 0)) * D + r * DR;        // this lane's rows inside one sequence's state
+    const size_t one = (size_t)H * VS * D;
+    float* S_g = a.state + (size_t)a.slots[s] * one + at;
+    float* part = PASS == 0 ? nullptr : a.part + (size_t)s * a.segs * one + at;
+    const int pw = CHANNEL ? D : 1;
+    float* prod = PASS == 0 ? nullptr : a.prod + ((size_t)s * a.segs * H + h) * pw;      // + segment * H * pw
+    float S[DR];
+    if constexpr (PASS == 0) {
+        load_rows(S_g, S);
+    } else if constexpr (PASS == 1) {
+        if (seg == 0) {
+            load_rows(S_g, S);
+            store_rows(part, S);                     // (the state itself is overwritten by the last segment of pass 2)
         } else {
 #pragma unroll
-            for (int e = 0; e < 4; ++e) S[i + e] = (col && r * DR + i + e < D) ? S_g[i + e] : 0.f;
+            for (int i = 0; i < DR; ++i) S[i] = 0.f;
+        }
+    } else {
+        if (seg == 0) {
+            load_rows(t1 == t_end ? S_g : part, S);
+        } else {
+            load_rows(part + one, S);
+            for (int e = 1; e < seg; ++e) {
+                float L[DR];
+                load_rows(part + (size_t)(e + 1) * one, L);
+                const float* K = prod + (size_t)e * H * pw;
+#pragma unroll
+                for (int i = 0; i < DR; ++i) S[i] = fmaf(CHANNEL ? (r * DR + i < D ? K[CHANNEL ? r * DR + i : 0] : 0.f) : K[0], S[i], L[i]);
+            }
         }
     }
-    float u[CHANNEL ? DR : 1];
-    if constexpr (CHANNEL) {
+    float u[CHANNEL && PASS != 1 ? DR : 1], K[CHANNEL && PASS == 1 ? DR : 1];
+    if constexpr (CHANNEL && PASS != 1) {
 #pragma unroll
-        for (int i = 0; i < DR; ++i) u[i] = r * DR + i < D ? bonus[(size_t)h * D + r * DR + i] : 0.f;
+        for (int i = 0; i < DR; ++i) u[i] = r * DR + i < D ? a.bonus[(size_t)h * D + r * DR + i] : 0.f;
     }
-    const float keep_fixed = keep_const ? keep[h] : 0.f;
+    if constexpr (PASS == 1) {
+#pragma unroll
+        for (int i = 0; i < (CHANNEL ? DR : 1); ++i) K[i] = 1.f;
+    }
+    const float keep_fixed = a.keep_const ? a.keep[h] : 0.f;
     float nxt[NL][W], v_nxt[P], a_nxt[P], b_nxt[P];
     auto fetch = [&](int first) {
 #pragma unroll
@@ -610,8 +693,9 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
             const int idx = n * NT + tid, p = idx / PIECES, e = (idx - p * PIECES) * W, which = e / DP, row = e - which * DP;
             const int t = first + p;
             const bool ok = idx < P * PIECES && t < t1 && row < D;
-            const float* src = which == 0 ? k + (size_t)t * ldk + (size_t)g * D : q + (size_t)t * ldq + (size_t)g * D;
-            if constexpr (CHANNEL) src = which == 2 ? keep + ((size_t)t * H + h) * D : src;
+            const float* src = a.k + (size_t)t * a.ldk + (size_t)g * D;
+            if constexpr (PASS != 1) src = which == 1 ? a.q + (size_t)t * a.ldq + (size_t)g * D : src;
+            if constexpr (CHANNEL) src = which == OPS - 1 ? a.keep + ((size_t)t * H + h) * D : src;
             if constexpr (VEC) {
                 const float4 x = ok ? *(const float4*)(src + row) : make_float4(0.f, 0.f, 0.f, 0.f);
                 nxt[n][0] = x.x; nxt[n][W - 3] = x.y; nxt[n][W - 2] = x.z; nxt[n][W - 1] = x.w;
@@ -622,13 +706,13 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
 #pragma unroll
         for (int p = 0; p < P; ++p) {
             const bool live = first + p < t1;
-            v_nxt[p] = (live && col) ? (ones ? 1.0f : v[(size_t)(first + p) * ldv + (size_t)h * V + j]) : 0.f;
+            v_nxt[p] = (live && col) ? (ones ? 1.0f : a.v[(size_t)(first + p) * a.ldv + (size_t)h * V + j]) : 0.f;
             if constexpr (CHANNEL) {
                 a_nxt[p] = 1.f;
                 b_nxt[p] = 1.f;
             } else {
-                a_nxt[p] = live ? (keep_const ? keep_fixed : keep[(size_t)(first + p) * H + h]) : 1.f;
-                b_nxt[p] = live ? (take ? take[(size_t)(first + p) * H + h] : 1.f) : 0.f;
+                a_nxt[p] = live ? (a.keep_const ? keep_fixed : a.keep[(size_t)(first + p) * H + h]) : 1.f;
+                b_nxt[p] = live ? (a.take ? a.take[(size_t)(first + p) * H + h] : 1.f) : 0.f;
             }
         }
     };
@@ -656,33 +740,40 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
         const bool more = first + P < t1;
         if (more) fetch(first + P);                  // the next group's operands leave now and are staged after this group's work
         auto token = [&](int p, int t) {
-            const float* kk = &kq[cur][p][0][r * DR];
-            const float* qq = &kq[cur][p][1][r * DR];
             float sq = 0.f;
 #pragma unroll
             for (int i = 0; i < DR; i += 4) {
-                const float4 k4 = *(const float4*)(kk + i), q4 = *(const float4*)(qq + i);
-                const float ka[4] = {k4.x, k4.y, k4.z, k4.w}, qa[4] = {q4.x, q4.y, q4.z, q4.w};
+                const float4 k4 = *(const float4*)(&kq[cur][p][0][r * DR] + i);
+                const float ka[4] = {k4.x, k4.y, k4.z, k4.w};
+                float qa[4] = {0.f, 0.f, 0.f, 0.f}, da[4] = {1.f, 1.f, 1.f, 1.f};
+                if constexpr (PASS != 1) {
+                    const float4 q4 = *(const float4*)(&kq[cur][p][OPS > 1 ? 1 : 0][r * DR] + i);
+                    qa[0] = q4.x; qa[1] = q4.y; qa[2] = q4.z; qa[3] = q4.w;
+                }
                 if constexpr (CHANNEL) {
                     const float4 d4 = *(const float4*)(&kq[cur][p][OPS - 1][r * DR] + i);
-                    const float da[4] = {d4.x, d4.y, d4.z, d4.w};
+                    da[0] = d4.x; da[1] = d4.y; da[2] = d4.z; da[3] = d4.w;
+                }
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        sq = fmaf(fmaf(u[i + e] * ka[e], bv_cur[p], S[i + e]), qa[e], sq);
+                for (int e = 0; e < 4; ++e) {
+                    if constexpr (CHANNEL) {
+                        if constexpr (PASS != 1) sq = fmaf(fmaf(u[i + e] * ka[e], bv_cur[p], S[i + e]), qa[e], sq);
+                        else K[i + e] *= da[e];
                         S[i + e] = fmaf(ka[e], bv_cur[p], S[i + e] * da[e]);
-                    }
-                } else {
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) {
+                    } else {
                         S[i + e] = fmaf(ka[e], bv_cur[p], S[i + e] * a_cur[p]);
-                        sq = fmaf(S[i + e], qa[e], sq);
+                        if constexpr (PASS != 1) sq = fmaf(S[i + e], qa[e], sq);
                     }
                 }
             }
-            sq = column_sum<LPC>(sq) * q_scale;
-            if (col && r == 0) {
-                if (ones) nq[(size_t)t * H + h] = sq;
-                else out[(size_t)t * ldo + (size_t)h * V + j] = sq;
+            if constexpr (PASS == 1) {
+                if constexpr (!CHANNEL) K[0] *= a_cur[p];
+            } else {
+                sq = column_sum<LPC>(sq) * a.q_scale;
+                if (col && r == 0) {
+                    if (ones) a.nq[(size_t)t * H + h] = sq;
+                    else a.out[(size_t)t * a.ldo + (size_t)h * V + j] = sq;
+                }
             }
         };
         if (first + P <= t1) {
@@ -696,61 +787,100 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(const float* __res
         if (more) stage(cur ^ 1);                    // (the buffer that every wave left before the last barrier)
         __syncthreads();
     }
+    if constexpr (PASS == 1) {
+        store_rows(part + (size_t)(seg + 1) * one, S);
+        if (blockIdx.x == 0 && wave == 0 && lane < (CHANNEL ? LPC : 1)) {      // (every column's lanes hold the same products)
+            float* K_g = prod + (size_t)seg * H * pw;
+            if constexpr (CHANNEL) {
 #pragma unroll
-    for (int i = 0; i < DR; i += 4) {
-        if constexpr (VEC) {
-            if (col && r * DR + i < D) *(float4*)(S_g + i) = make_float4(S[i], S[i + 1], S[i + 2], S[i + 3]);
-        } else {
-#pragma unroll
-            for (int e = 0; e < 4; ++e)
-                if (col && r * DR + i + e < D) S_g[i + e] = S[i + e];
+                for (int i = 0; i < DR; ++i)
+                    if (r * DR + i < D) K_g[r * DR + i] = K[i];
+            } else {
+                K_g[0] = K[0];
+            }
         }
+    } else if (t1 == t_end) {
+        store_rows(S_g, S);
     }
 }
 
+// columns of a state per block, by the sizes alone (as FX_OUTER dispatches)
+static int outer_columns(int D, int V) { return D <= 64 ? (V <= 32 ? 2 * 4 : 4 * 4) : (D <= 128 ? 4 * 2 : 8 * 2); }
+
+// Into how many segments portions of up to `longest` tokens are cut (1: one launch): enough for about four waves a
+// SIMD, none shorter than 128 tokens.
+FX_API int fx_outer_segments(int n_seqs, int H, int D, int V, int normalizer, int longest) {
+    if (n_seqs <= 0 || H <= 0 || D <= 0 || V <= 0 || longest < 256) return 1;
+    const long blocks = (long)ceil_div(V + (normalizer ? 1 : 0), outer_columns(D, V)) * H * n_seqs;
+    const long waves = blocks * (D <= 64 ? (V <= 32 ? 2 : 4) : (D <= 128 ? 4 : 8));
+    long segs = 16L * fx_compute_units() / waves;
+    if (segs > longest / 128) segs = longest / 128;
+    if (segs > 16) segs = 16;
+    return segs < 2 ? 1 : (int)segs;
+}
+
 template <bool CHANNEL>
-static int launch_gated_outer(const char* who, void* stream, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
-                              const float* keep, int keep_const, const float* take, float* out, long ldo, float* nq, float* state,
-                              const int* seq_starts, const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale,
-                              const float* bonus) {
-    FX_REQUIRE(n_seqs >= 0 && H > 0 && G > 0 && H % G == 0, "%s: bad sizes sequences=%d H=%d G=%d", who, n_seqs, H, G);
-    FX_REQUIRE(D >= 1 && D <= 256 && V >= 1, "%s: key size %d (up to 256) and value size %d", who, D, V);
-    FX_REQUIRE(ldq >= (long)G * D && ldk >= (long)G * D && ldv >= (long)H * V && ldo >= (long)H * V, "%s: rows too short for %d heads", who, H);
-    FX_REQUIRE(n_seqs <= 65535 && H <= 65535, "%s: %d sequences of %d heads are more than a launch takes", who, n_seqs, H);
-    FX_REQUIRE(keep, "%s: the forgetting factors are missing", who);
+static int launch_gated_outer(const char* who, hipStream_t s, const OuterArgs& a, int n_seqs) {
+    FX_REQUIRE(n_seqs >= 0 && a.H > 0 && a.G > 0 && a.H % a.G == 0, "%s: bad sizes sequences=%d H=%d G=%d", who, n_seqs, a.H, a.G);
+    FX_REQUIRE(a.D >= 1 && a.D <= 256 && a.V >= 1, "%s: key size %d (up to 256) and value size %d", who, a.D, a.V);
+    FX_REQUIRE(a.ldq >= (long)a.G * a.D && a.ldk >= (long)a.G * a.D && a.ldv >= (long)a.H * a.V && a.ldo >= (long)a.H * a.V,
+               "%s: rows too short for %d heads", who, a.H);
+    FX_REQUIRE(a.segs >= 1 && a.segs <= 64 && (a.segs == 1 || (a.part && a.prod)), "%s: %d segments (up to 64) need room for their states", who, a.segs);
+    FX_REQUIRE((long)n_seqs * a.segs <= 65535 && a.H <= 65535, "%s: %d sequences of %d heads are more than a launch takes", who, n_seqs, a.H);
+    FX_REQUIRE(a.keep, "%s: the forgetting factors are missing", who);
     if (n_seqs == 0) return 0;
-    const int VS = V + (nq ? 1 : 0);
-    const bool vec = D % 4 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && (((uintptr_t)state | (uintptr_t)q | (uintptr_t)k | (CHANNEL ? (uintptr_t)keep : 0)) % 16) == 0;
-    hipStream_t s = (hipStream_t)stream;
-#define FX_OUTER(DR_, LPC_, NW_)                                                                                              \
+    const bool vec = a.D % 4 == 0 && a.ldq % 4 == 0 && a.ldk % 4 == 0 &&
+                     (((uintptr_t)a.state | (uintptr_t)a.q | (uintptr_t)a.k | (uintptr_t)a.part | (CHANNEL ? (uintptr_t)a.keep : 0)) % 16) == 0;
+#define FX_OUTER_PASS(DR_, LPC_, NW_, PASS_, RUNS_)                                                                           \
     do {                                                                                                                      \
         const int per_block = NW_ * 64 / LPC_;                                                                                \
-        const dim3 grid((VS + per_block - 1) / per_block, H, n_seqs);                                                         \
-        if (vec) gated_outer_kernel<DR_, LPC_, true, NW_, CHANNEL><<<grid, NW_ * 64, 0, s>>>(q, ldq, k, ldk, v, ldv, keep, keep_const, take, out, ldo, nq, state, seq_starts, slots, H, G, D, V, VS, q_scale, bonus); \
-        else gated_outer_kernel<DR_, LPC_, false, NW_, CHANNEL><<<grid, NW_ * 64, 0, s>>>(q, ldq, k, ldk, v, ldv, keep, keep_const, take, out, ldo, nq, state, seq_starts, slots, H, G, D, V, VS, q_scale, bonus);    \
+        const dim3 grid((a.VS + per_block - 1) / per_block, a.H, n_seqs * (RUNS_));                                           \
+        if (vec) gated_outer_kernel<DR_, LPC_, true, NW_, CHANNEL, PASS_><<<grid, NW_ * 64, 0, s>>>(a);                       \
+        else gated_outer_kernel<DR_, LPC_, false, NW_, CHANNEL, PASS_><<<grid, NW_ * 64, 0, s>>>(a);                          \
     } while (0)
-    if (D <= 64 && V <= 32) FX_OUTER(4, 16, 2);
-    else if (D <= 64) FX_OUTER(4, 16, 4);
-    else if (D <= 128) FX_OUTER(4, 32, 4);
+#define FX_OUTER(DR_, LPC_, NW_)                                    \
+    do {                                                            \
+        if (a.segs == 1) FX_OUTER_PASS(DR_, LPC_, NW_, 0, 1);       \
+        else {                                                      \
+            FX_OUTER_PASS(DR_, LPC_, NW_, 1, a.segs - 1);           \
+            FX_OUTER_PASS(DR_, LPC_, NW_, 2, a.segs);               \
+        }                                                           \
+    } while (0)
+    if (a.D <= 64 && a.V <= 32) FX_OUTER(4, 16, 2);
+    else if (a.D <= 64) FX_OUTER(4, 16, 4);
+    else if (a.D <= 128) FX_OUTER(4, 32, 4);
     else FX_OUTER(8, 32, 8);
 #undef FX_OUTER
+#undef FX_OUTER_PASS
     FX_CHECK_LAUNCH(who);
     return 0;
 }
 
+// `segs` > 1: portions are cut (see above); `part` and `prod` are then float32 [n_seqs, segs, H, V (+ 1), D] and
+// [n_seqs, segs, H] (channel_outer: [n_seqs, segs, H, D]) that the call may overwrite.
 FX_API int fx_gated_outer(void* stream, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
                           const float* keep, int keep_const, const float* take, float* out, long ldo, float* nq, float* state,
-                          const int* seq_starts, const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale) {
-    return launch_gated_outer<false>("gated_outer", stream, q, ldq, k, ldk, v, ldv, keep, keep_const, take, out, ldo, nq, state,
-                                     seq_starts, slots, n_seqs, H, G, D, V, q_scale, nullptr);
+                          const int* seq_starts, const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale,
+                          int segs, float* part, float* prod) {
+    OuterArgs a = {};
+    a.q = q; a.ldq = ldq; a.k = k; a.ldk = ldk; a.v = v; a.ldv = ldv; a.keep = keep; a.keep_const = keep_const; a.take = take;
+    a.out = out; a.ldo = ldo; a.nq = nq; a.state = state; a.seq_starts = seq_starts; a.slots = slots;
+    a.H = H; a.G = G; a.D = D; a.V = V; a.VS = V + (nq ? 1 : 0); a.q_scale = q_scale;
+    a.segs = segs; a.part = part; a.prod = prod;
+    return launch_gated_outer<false>("gated_outer", (hipStream_t)stream, a, n_seqs);
 }
 
 FX_API int fx_channel_outer(void* stream, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
                             const float* keep, const float* bonus, float* out, long ldo, float* state, const int* seq_starts,
-                            const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale) {
+                            const int* slots, int n_seqs, int H, int G, int D, int V, float q_scale, int segs, float* part,
+                            float* prod) {
     FX_REQUIRE(bonus, "channel_outer: the current token's bonus is missing");
-    return launch_gated_outer<true>("channel_outer", stream, q, ldq, k, ldk, v, ldv, keep, 0, nullptr, out, ldo, nullptr, state,
-                                    seq_starts, slots, n_seqs, H, G, D, V, q_scale, bonus);
+    OuterArgs a = {};
+    a.q = q; a.ldq = ldq; a.k = k; a.ldk = ldk; a.v = v; a.ldv = ldv; a.keep = keep; a.bonus = bonus;
+    a.out = out; a.ldo = ldo; a.state = state; a.seq_starts = seq_starts; a.slots = slots;
+    a.H = H; a.G = G; a.D = D; a.V = V; a.VS = V; a.q_scale = q_scale;
+    a.segs = segs; a.part = part; a.prod = prod;
+    return launch_gated_outer<true>("channel_outer", (hipStream_t)stream, a, n_seqs);
 }
 
 // ---------------------------------------------------------------------------
@@ -760,35 +890,52 @@ FX_API int fx_channel_outer(void* stream, const float* q, long ldq, const float*
 //   m_t = max(f + m_(t-1), i);  keep_t = exp(f + m_(t-1) - m_t);  take_t = exp(i - m_t)
 // m is carried in state[slot, h] (zero at a sequence's start).  Outputs keep, take, m: float32 [T, H].
 // The running maximum is a scan: token t maps m to max(m + f_t, i_t), and two such maps in a row are one of the same
-// form, (f_a + f_b, max(i_a + f_b, i_b)); a wave takes 64 tokens at a time, a lane each, and combines them in six
-// rounds.  One wave per (sequence, head).
+// form, (f_a + f_b, max(i_a + f_b, i_b)); a wave takes 64 tokens, a lane each, and combines them in six rounds.  The
+// NW waves of a block take the next NW chunks of 64 tokens at once; a wave's start is the carried maximum through the
+// maps of the chunks before its own, one by one, which is what a single wave going through them does (the same bits
+// whatever NW).  One block per (sequence, head).
 // ---------------------------------------------------------------------------
 __device__ __forceinline__ float log_sigmoid_f(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
 
-__global__ __launch_bounds__(64) void exp_gate_scan_kernel(const float* __restrict__ xi, long ldi, const float* __restrict__ xf, long ldf,
-                                                           float cap, float* __restrict__ keep, float* __restrict__ take,
-                                                           float* __restrict__ m_out, float* __restrict__ state,
-                                                           const int* __restrict__ seq_starts, const int* __restrict__ slots, int H) {
-    const int h = blockIdx.x, s = blockIdx.y, lane = threadIdx.x;
+template <int NW>
+__global__ __launch_bounds__(NW * 64) void exp_gate_scan_kernel(const float* __restrict__ xi, long ldi, const float* __restrict__ xf, long ldf,
+                                                                float cap, float* __restrict__ keep, float* __restrict__ take,
+                                                                float* __restrict__ m_out, float* __restrict__ state,
+                                                                const int* __restrict__ seq_starts, const int* __restrict__ slots, int H) {
+    __shared__ float F_of[2][NW], I_of[2][NW];
+    const int h = blockIdx.x, s = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int t0 = seq_starts[s], t1 = seq_starts[s + 1];
     if (t1 <= t0) return;
     float* carried = state + (size_t)slots[s] * H + h;
-    float m_prev = *carried;
-    for (int base = t0; base < t1; base += 64) {
-        const int t = base + lane;
+    float m_start = *carried;                        // before the group's first chunk
+    for (int base = t0, cur = 0; base < t1; base += NW * 64, cur ^= 1) {
+        const int t = base + wave * 64 + lane;
         const bool live = t < t1;
-        float gi = -INFINITY, gf = 0.f;
+        float gi = -INFINITY, gf = 0.f;              // (past the end: the map that changes nothing)
         if (live) {
             gi = cap * tanhf(xi[(size_t)t * ldi + h] / cap);
             gf = log_sigmoid_f(cap * tanhf(xf[(size_t)t * ldf + h] / cap));
         }
-        float F = gf, I = gi;                       // the map of this lane's token; then of all tokens up to it
+        float F = gf, I = gi;                       // the map of this lane's token; then of the chunk's tokens up to it
 #pragma unroll
         for (int d = 1; d < 64; d <<= 1) {
             const float Fp = __shfl_up(F, d), Ip = __shfl_up(I, d);
             if (lane >= d) {
                 I = fmaxf(Ip + F, I);
                 F = Fp + F;
+            }
+        }
+        float m_prev = m_start;
+        if constexpr (NW > 1) {
+            if (lane == 63) {
+                F_of[cur][wave] = F;
+                I_of[cur][wave] = I;
+            }
+            __syncthreads();                         // (the other of the two buffers is written before the next barrier)
+#pragma unroll
+            for (int w = 0; w < NW; ++w) {
+                if (w == wave) m_prev = m_start;
+                m_start = fmaxf(m_start + F_of[cur][w], I_of[cur][w]);
             }
         }
         const float m_t = fmaxf(m_prev + F, I);
@@ -799,17 +946,20 @@ __global__ __launch_bounds__(64) void exp_gate_scan_kernel(const float* __restri
             take[(size_t)t * H + h] = expf(gi - m_t);
             m_out[(size_t)t * H + h] = m_t;
         }
-        m_prev = __shfl(m_t, min(63, t1 - 1 - base));
+        if constexpr (NW == 1) m_start = __shfl(m_t, 63);
     }
-    if (lane == 0) *carried = m_prev;
+    if (threadIdx.x == 0) *carried = m_start;
 }
 
 FX_API int fx_exp_gate_scan(void* stream, const float* xi, long ldi, const float* xf, long ldf, float cap, float* keep,
-                            float* take, float* m_out, float* state, const int* seq_starts, const int* slots, int n_seqs, int H) {
+                            float* take, float* m_out, float* state, const int* seq_starts, const int* slots, int n_seqs, int H,
+                            int longest) {
     FX_REQUIRE(n_seqs >= 0 && n_seqs <= 65535 && H > 0 && ldi >= H && ldf >= H, "exp_gate_scan: bad sizes sequences=%d H=%d", n_seqs, H);
     FX_REQUIRE(cap > 0.f, "exp_gate_scan: a cap of %g", (double)cap);
     if (n_seqs == 0) return 0;
-    exp_gate_scan_kernel<<<dim3(H, n_seqs), 64, 0, (hipStream_t)stream>>>(xi, ldi, xf, ldf, cap, keep, take, m_out, state, seq_starts, slots, H);
+    // (`longest`: the most tokens any sequence brings; it picks how many waves a block has, nothing else)
+    if (longest > 64) exp_gate_scan_kernel<16><<<dim3(H, n_seqs), 1024, 0, (hipStream_t)stream>>>(xi, ldi, xf, ldf, cap, keep, take, m_out, state, seq_starts, slots, H);
+    else exp_gate_scan_kernel<1><<<dim3(H, n_seqs), 64, 0, (hipStream_t)stream>>>(xi, ldi, xf, ldf, cap, keep, take, m_out, state, seq_starts, slots, H);
     FX_CHECK_LAUNCH("exp_gate_scan");
     return 0;
 }
@@ -1024,18 +1174,20 @@ FX_API int fx_token_shift(void* stream, int dtype, const void* x, long ldx, cons
 // A decay per channel from a low-rank projection, all float32:
 //   out[t, n] = exp(-exp(sum_k tanh(low[t, k]) w2t[k, n] + w0[n])),   k ascending in one accumulator
 // low [T, R] rows are the first half's products; w2t [R, N] is the second half's matrix, transposed, so that
-// neighbouring threads read neighbouring columns.  A thread owns a column, a block 256 columns of TT tokens, whose
-// tanh values lie in LDS, KB of the R at a time.  Grid: (ceil(N / 256), ceil(T / TT)).
+// neighbouring threads read neighbouring columns.  A thread owns C columns of TT tokens (C float32 products share one
+// read of the tokens' tanh values, which lie in LDS, KB of the R at a time).  Grid: (ceil(N / (256 C)), ceil(T / TT)).
 // ---------------------------------------------------------------------------
-template <int TT>
+template <int TT, int C>
 __global__ __launch_bounds__(256) void lowrank_decay_kernel(const float* __restrict__ low, long ldl, const float* __restrict__ w2t,
                                                             const float* __restrict__ w0, float* __restrict__ out, int n_tokens, int R, int N) {
     constexpr int KB = 128;
     __shared__ __attribute__((aligned(16))) float xs[KB][TT];
-    const int n = blockIdx.x * 256 + threadIdx.x, first = blockIdx.y * TT;
-    float acc[TT];
+    const int n = (blockIdx.x * 256 + threadIdx.x) * C, first = blockIdx.y * TT;      // (N is a multiple of C)
+    float acc[TT][C];
 #pragma unroll
-    for (int i = 0; i < TT; ++i) acc[i] = 0.f;
+    for (int i = 0; i < TT; ++i)
+#pragma unroll
+        for (int c = 0; c < C; ++c) acc[i][c] = 0.f;
     for (int k0 = 0; k0 < R; k0 += KB) {
         const int kn = min(KB, R - k0);
         if (k0) __syncthreads();
@@ -1048,17 +1200,34 @@ __global__ __launch_bounds__(256) void lowrank_decay_kernel(const float* __restr
             const float* w = w2t + (size_t)k0 * N + n;
 #pragma unroll 8
             for (int k = 0; k < kn; ++k) {
-                const float wv = w[(size_t)k * N];
+                float wv[C];
+                if constexpr (C == 4) {
+                    const float4 w4 = *(const float4*)(w + (size_t)k * N);
+                    wv[0] = w4.x; wv[1] = w4.y; wv[2] = w4.z; wv[3] = w4.w;
+                } else {
+                    wv[0] = w[(size_t)k * N];
+                }
 #pragma unroll
-                for (int i = 0; i < TT; ++i) acc[i] = fmaf(xs[k][i], wv, acc[i]);
+                for (int i = 0; i < TT; ++i)
+#pragma unroll
+                    for (int c = 0; c < C; ++c) acc[i][c] = fmaf(xs[k][i], wv[c], acc[i][c]);
             }
         }
     }
     if (n >= N) return;
-    const float base = w0[n];
+    float base[C];
 #pragma unroll
-    for (int i = 0; i < TT; ++i)
-        if (first + i < n_tokens) out[(size_t)(first + i) * N + n] = expf(-expf(acc[i] + base));
+    for (int c = 0; c < C; ++c) base[c] = w0[n + c];
+#pragma unroll
+    for (int i = 0; i < TT; ++i) {
+        if (first + i >= n_tokens) break;
+        float y[C];
+#pragma unroll
+        for (int c = 0; c < C; ++c) y[c] = expf(-expf(acc[i][c] + base[c]));
+        float* dst = out + (size_t)(first + i) * N + n;
+        if constexpr (C == 4) *(float4*)dst = make_float4(y[0], y[1], y[2], y[3]);
+        else *dst = y[0];
+    }
 }
 
 FX_API int fx_lowrank_decay(void* stream, const float* low, long ldl, const float* w2t, const float* w0, float* out, int T, int R, int N) {
@@ -1066,8 +1235,10 @@ FX_API int fx_lowrank_decay(void* stream, const float* low, long ldl, const floa
     FX_REQUIRE(T <= 65535, "lowrank_decay: %d tokens are more than a launch takes", T);
     if (T == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    if (T <= 64) lowrank_decay_kernel<1><<<dim3((N + 255) / 256, T), 256, 0, s>>>(low, ldl, w2t, w0, out, T, R, N);
-    else lowrank_decay_kernel<16><<<dim3((N + 255) / 256, (T + 15) / 16), 256, 0, s>>>(low, ldl, w2t, w0, out, T, R, N);
+    const bool vec = N % 4 == 0 && (((uintptr_t)w2t | (uintptr_t)out) % 16) == 0;
+    if (T <= 64) lowrank_decay_kernel<1, 1><<<dim3((N + 255) / 256, T), 256, 0, s>>>(low, ldl, w2t, w0, out, T, R, N);
+    else if (vec) lowrank_decay_kernel<8, 4><<<dim3((N + 1023) / 1024, (T + 7) / 8), 256, 0, s>>>(low, ldl, w2t, w0, out, T, R, N);
+    else lowrank_decay_kernel<8, 1><<<dim3((N + 255) / 256, (T + 7) / 8), 256, 0, s>>>(low, ldl, w2t, w0, out, T, R, N);
     FX_CHECK_LAUNCH("lowrank_decay");
     return 0;
 }

@@ -91,14 +91,16 @@ _sigs = {
                                      c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_int],
     ("recurrent", "fx_gated_outer"): [c_void_p, c_void_p, c_long, c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_void_p,
                                       c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
-                                      c_float],
+                                      c_float, c_int, c_void_p, c_void_p],
+    ("recurrent", "fx_outer_segments"): [c_int, c_int, c_int, c_int, c_int, c_int],
     ("recurrent", "fx_channel_outer"): [c_void_p, c_void_p, c_long, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p,
-                                        c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float],
+                                        c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float,
+                                        c_int, c_void_p, c_void_p],
     ("recurrent", "fx_token_shift"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                                       c_void_p, c_int, c_int],
     ("recurrent", "fx_lowrank_decay"): [c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int],
     ("recurrent", "fx_exp_gate_scan"): [c_void_p, c_void_p, c_long, c_void_p, c_long, c_float, c_void_p, c_void_p, c_void_p,
-                                        c_void_p, c_void_p, c_void_p, c_int, c_int],
+                                        c_void_p, c_void_p, c_void_p, c_int, c_int, c_int],
     ("recurrent", "fx_rglru_gates"): [c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_float,
                                       c_void_p, c_void_p, c_int, c_int, c_int],
     ("recurrent", "fx_rglru_scan"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p,
@@ -1226,13 +1228,14 @@ def small_rows_parts(x, wt):
 
 
 def gated_outer(q, k, v, keep, take, state, seq_starts, slot_ids, n_seqs: int, n_heads: int, n_kv_heads: int, key_dim: int,
-                v_dim: int, q_scale: float = 1.0, normalizer: bool = False):
+                v_dim: int, q_scale: float = 1.0, normalizer: bool = False, longest: int = 1, segments: int | None = None):
     """A matrix memory with one forgetting and one writing factor per head and token, over each sequence's tokens in
     order, from and into state[slot]:  S <- keep_t S + take_t k_t v_t^T;  o_t = q_scale S^T q_t.  q, k: float32 rows
     [T, G*D]; v [T, H*V]; `keep` float32 [T, H], or [H] (the same factors at every token); `take` float32 [T, H] or
     None (1).  The state is float32 [slots, H, V, D] (transposed).  With `normalizer` it is [slots, H, V + 1, D]: its
     last column is n <- keep_t n + take_t k_t, and the call also returns nq [T, H] = q_scale n_t . q_t.
-    Returns o float32 [T, H*V], or (o, nq)."""
+    `longest`: the most tokens any sequence brings; long portions are cut into segments that run at once (`segments`:
+    into so many).  Returns o float32 [T, H*V], or (o, nq)."""
     T = q.shape[0]
     H, G, D, V = int(n_heads), int(n_kv_heads), int(key_dim), int(v_dim)
     _f32_rows(q, "gated_outer: q", G * D), _f32_rows(k, "gated_outer: k", G * D), _f32_rows(v, "gated_outer: v", H * V)
@@ -1249,18 +1252,33 @@ def gated_outer(q, k, v, keep, take, state, seq_starts, slot_ids, n_seqs: int, n
         raise KernelError("gated_outer: the step's index tensors are shorter than its sequences")
     out = torch.empty((T, H * V), dtype=torch.float32, device=q.device)
     nq = torch.empty((T, H), dtype=torch.float32, device=q.device) if normalizer else None
+    segs, part, prod = _segment_room(q.device, n_seqs, H, D, V, normalizer, longest, segments, 1)
     _call("recurrent", "fx_gated_outer", _stream(), _p(q), q.stride(0), _p(k), k.stride(0), _p(v), v.stride(0), _p(keep),
           1 if keep_const else 0, _p(take), _p(out), out.stride(0), _p(nq), _p(state), _p(_i32(seq_starts, "seq_starts")),
-          _p(_i32(slot_ids, "slot_ids")), int(n_seqs), H, G, D, V, float(q_scale))
+          _p(_i32(slot_ids, "slot_ids")), int(n_seqs), H, G, D, V, float(q_scale), segs, _p(part), _p(prod))
     return (out, nq) if normalizer else out
 
 
+def _segment_room(device, n_seqs: int, H: int, D: int, V: int, normalizer: bool, longest: int, segments, factors: int):
+    """(segments, room for their states, room for their products of factors) of an outer-product recurrence."""
+    if segments is None:
+        f, _ = _fn("recurrent", "fx_outer_segments")
+        segments = int(f(int(n_seqs), H, D, V, 1 if normalizer else 0, int(longest)))
+    if segments == 1:
+        return 1, None, None
+    VS = V + (1 if normalizer else 0)
+    part = torch.empty((n_seqs, segments, H, VS, D), dtype=torch.float32, device=device)
+    prod = torch.empty((n_seqs, segments, H, factors), dtype=torch.float32, device=device)
+    return int(segments), part, prod
+
+
 def channel_outer(q, k, v, keep, bonus, state, seq_starts, slot_ids, n_seqs: int, n_heads: int, key_dim: int, v_dim: int,
-                  q_scale: float = 1.0) -> torch.Tensor:
+                  q_scale: float = 1.0, longest: int = 1, segments: int | None = None) -> torch.Tensor:
     """A matrix memory with one forgetting factor per key channel and a bonus for the current token, over each sequence's
     tokens in order, from and into state[slot] (float32 [slots, H, V, D], transposed as in `gated_outer`):
         o_t = q_scale (S + diag(bonus) k_t v_t^T)^T q_t;   S <- diag(keep_t) S + k_t v_t^T
-    q, k [T, H*D], v [T, H*V] float32 rows; keep float32 contiguous [T, H*D]; bonus float32 [H, D].  Returns o [T, H*V]."""
+    q, k [T, H*D], v [T, H*V] float32 rows; keep float32 contiguous [T, H*D]; bonus float32 [H, D].  `longest`,
+    `segments`: as in `gated_outer`.  Returns o [T, H*V]."""
     T = q.shape[0]
     H, D, V = int(n_heads), int(key_dim), int(v_dim)
     _f32_rows(q, "channel_outer: q", H * D), _f32_rows(k, "channel_outer: k", H * D), _f32_rows(v, "channel_outer: v", H * V)
@@ -1273,9 +1291,10 @@ def channel_outer(q, k, v, keep, bonus, state, seq_starts, slot_ids, n_seqs: int
     if seq_starts.numel() < n_seqs + 1 or slot_ids.numel() < n_seqs:
         raise KernelError("channel_outer: the step's index tensors are shorter than its sequences")
     out = torch.empty((T, H * V), dtype=torch.float32, device=q.device)
+    segs, part, prod = _segment_room(q.device, n_seqs, H, D, V, False, longest, segments, D)
     _call("recurrent", "fx_channel_outer", _stream(), _p(q), q.stride(0), _p(k), k.stride(0), _p(v), v.stride(0), _p(keep), _p(bonus),
           _p(out), out.stride(0), _p(state), _p(_i32(seq_starts, "seq_starts")), _p(_i32(slot_ids, "slot_ids")), int(n_seqs),
-          H, H, D, V, float(q_scale))
+          H, H, D, V, float(q_scale), segs, _p(part), _p(prod))
     return out
 
 
@@ -1313,11 +1332,12 @@ def lowrank_decay(low, w2t, w0) -> torch.Tensor:
     return out
 
 
-def exp_gate_scan(x_in, x_forget, cap: float, state, seq_starts, slot_ids, n_seqs: int, n_heads: int):
+def exp_gate_scan(x_in, x_forget, cap: float, state, seq_starts, slot_ids, n_seqs: int, n_heads: int, longest: int = 1):
     """Exponential gates under a running maximum, per head over each sequence's tokens in order.  From the float32
     rows x_in, x_forget [T, H]:  i = cap tanh(x_in / cap);  f = logsigmoid(cap tanh(x_forget / cap));
     m_t = max(f + m_(t-1), i);  keep_t = exp(f + m_(t-1) - m_t);  take_t = exp(i - m_t).  m is carried in
-    state [slots, H] (float32).  Returns (keep, take, m), float32 [T, H] each."""
+    state [slots, H] (float32).  `longest`: the most tokens any sequence brings (how many waves share a sequence; the
+    bits are the same).  Returns (keep, take, m), float32 [T, H] each."""
     T, H = x_in.shape[0], int(n_heads)
     _f32_rows(x_in, "exp_gate_scan: x_in", H), _f32_rows(x_forget, "exp_gate_scan: x_forget", H)
     if x_forget.shape[0] != T or state.dtype != torch.float32 or not state.is_contiguous() or tuple(state.shape[1:]) != (H,):
@@ -1327,7 +1347,7 @@ def exp_gate_scan(x_in, x_forget, cap: float, state, seq_starts, slot_ids, n_seq
     keep, take, m = (torch.empty((T, H), dtype=torch.float32, device=x_in.device) for _ in range(3))
     _call("recurrent", "fx_exp_gate_scan", _stream(), _p(x_in), x_in.stride(0), _p(x_forget), x_forget.stride(0), float(cap),
           _p(keep), _p(take), _p(m), _p(state), _p(_i32(seq_starts, "seq_starts")), _p(_i32(slot_ids, "slot_ids")),
-          int(n_seqs), H)
+          int(n_seqs), H, int(longest))
     return keep, take, m
 
 

@@ -100,7 +100,7 @@ class DecayAttention(Mixer):
         gate = matmul(x, self.w_gate, epilogue=ops.EPI_STORE_F32)
         debug.region("linear recurrence")
         o = ops.gated_outer(qkv[:, :QK], qkv[:, QK:2 * QK], qkv[:, 2 * QK:], self.decays, None, cache.state["S"],
-                            sequence_starts(ctx), ctx.slot_ids, ctx.n_seqs, H, H, D, V)
+                            sequence_starts(ctx), ctx.slot_ids, ctx.n_seqs, H, H, D, V, longest=longest_portion(ctx))
         debug.region("linear out")
         y = ops.gated_head_norm(o, gate, self.norm_w, self.norm_eps, 1, H * V, ctx.act_dtype)      # all heads as one row
         _add_out(self.o_proj, y, ctx, residual, out_scale, fresh)
@@ -160,10 +160,10 @@ class MatrixMemory(Mixer):
         starts = sequence_starts(ctx)
         debug.region("memory gates")
         keep, take, m = ops.exp_gate_scan(proj[:, i0:i0 + H], proj[:, i0 + H:i0 + 2 * H], self.gate_cap, cache.state["m"],
-                                          starts, ctx.slot_ids, ctx.n_seqs, H)
+                                          starts, ctx.slot_ids, ctx.n_seqs, H, longest=longest_portion(ctx))
         debug.region("linear recurrence")
         o, nq = ops.gated_outer(proj[:, :QK], proj[:, QK:2 * QK], proj[:, 2 * QK:g0], keep, take, cache.state["S"], starts,
-                                ctx.slot_ids, ctx.n_seqs, H, H, D, V, q_scale=D ** -0.5, normalizer=True)
+                                ctx.slot_ids, ctx.n_seqs, H, H, D, V, q_scale=D ** -0.5, normalizer=True, longest=longest_portion(ctx))
         debug.region("memory out")
         y = ops.gated_head_norm(o, proj[:, g0:i0], self.norm_w, self.norm_eps, H, V, ctx.act_dtype, denominators=(nq, m))
         _add_out(self.o_proj, y, ctx, residual, out_scale, fresh)

@@ -14,7 +14,7 @@ import torch
 
 from .. import debug, ops
 from .base import MIXERS, Mixer, ParamSpec
-from .gated_linear import _add_out
+from .gated_linear import _add_out, longest_portion
 from .linear import Linear, matmul, same_dtype
 from .recurrent import sequence_starts
 
@@ -106,7 +106,8 @@ class TimeMix(Mixer):
         debug.region("time mix decay")
         keep = ops.lowrank_decay(low, self.decay_out_t, self.decay_base)
         debug.region("linear recurrence")
-        o = ops.channel_outer(r, k, v, keep, self.bonus, cache.state["S"], starts, ctx.slot_ids, ctx.n_seqs, H, D, D)
+        o = ops.channel_outer(r, k, v, keep, self.bonus, cache.state["S"], starts, ctx.slot_ids, ctx.n_seqs, H, D, D,
+                              longest=longest_portion(ctx))
         debug.region("time mix out")
         y = ops.gated_head_norm(o, gate, self.norm_w, self.norm_eps, H, D, ctx.act_dtype, gate_activation="silu")
         _add_out(self.o_proj, y, ctx, residual, out_scale, fresh)
