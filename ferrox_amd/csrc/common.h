@@ -130,6 +130,11 @@ __device__ __forceinline__ float lane_pair_other(float v) {
     return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xF, 0xF, false));      // quad_perm [1, 0, 3, 2]
 }
 
+// the value of the lane in the other half of a quad (lane l ^ 2)
+__device__ __forceinline__ float quad_half_other(float v) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xF, 0xF, false));      // quad_perm [2, 3, 0, 1]
+}
+
 // ---- wave (64 lanes) and block reductions in a fixed order ------------------
 // Sum and maximum over the 64 lanes of a wave, in every lane: a butterfly over the lanes 32, 16, 8, 4, 2 and 1
 // away, in that order (the order fixes the sum's bits).  The exchanges stay in the vector unit: the halves of the

@@ -7,6 +7,8 @@
 // tokens [seq_starts[s], seq_starts[s + 1]); its state lives in slot slots[s] of the state slabs.
 #include "common.h"
 
+#include <type_traits>
+
 FX_DEFINE_LAST_ERROR()
 
 // ---------------------------------------------------------------------------
@@ -559,14 +561,7 @@ FX_API int fx_gated_head_norm(void* stream, int out_dtype, const float* o, long 
 // Lanes, columns, the state's transposed layout, the groups of P tokens that a block of waves brings into LDS a
 // group ahead: as in the delta rule's kernel above; a token's work is one pass over the lane's rows (S updated, and
 // its part of S^T q) and one sum over the lanes of a column.
-//
-// A long portion is a long chain of tokens on few waves, so it may be cut into `segs` segments that run at once: PASS 1
-// takes every segment but the last from zero (the first from the carried state) to its local state, with the product
-// of its forgetting factors; PASS 2 puts a segment's start together from the segments before it,
-//   S_g = K_(g-1) S_(g-1) + L_(g-1),   K a segment's product of factors, L its local state,
-// and runs it with its outputs.  Twice the updates, a `segs`-th of the chain.  PASS 0 is the one-launch form.
-// `part` [sequence][segs][H][VS][D]: the carried state, then the local states; `prod` [sequence][segs][H][D or 1].
-// Grid: (ceil(VS / (NW 64 / LPC)), heads, sequences x (1, segs - 1 or segs)).
+// Grid: (ceil(VS / (NW 64 / LPC)), heads, sequences).
 // ---------------------------------------------------------------------------
 struct OuterArgs {
     const float* q;
@@ -586,20 +581,14 @@ struct OuterArgs {
     int keep_const, segs, H, G, D, V, VS;
     float q_scale;
 };
-#define OUTER_GROUP 8            // tokens that travel together
-#define OUTER_MIN_SEGMENT 64     // the fewest tokens of a segment that is not a sequence's last
-__host__ __device__ __forceinline__ int outer_segment(int n, int segs) {      // tokens of a segment of an n-token portion
-    const int per = ((n + segs - 1) / segs + OUTER_GROUP - 1) / OUTER_GROUP * OUTER_GROUP;
-    return per > OUTER_MIN_SEGMENT ? per : OUTER_MIN_SEGMENT;
-}
 
-template <int DR, int LPC, bool VEC, int NW, bool CHANNEL, int PASS>
+template <int DR, int LPC, bool VEC, int NW, bool CHANNEL>
 __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(OuterArgs a) {
     constexpr int DP = LPC * DR;                     // rows as a wave holds them
     constexpr int W = VEC ? 4 : 1;                   // floats per load
-    constexpr int P = OUTER_GROUP;
+    constexpr int P = 8;                             // tokens that travel together
     constexpr int NT = NW * 64;
-    constexpr int OPS = (PASS == 1 ? 1 : 2) + (CHANNEL ? 1 : 0);      // k (, q) (, keep)
+    constexpr int OPS = CHANNEL ? 3 : 2;             // k, q (, keep)
     constexpr int PIECES = OPS * DP / W;             // loads that bring one token's operands
     constexpr int NL = (P * PIECES + NT - 1) / NT;   // loads a thread makes per group
     constexpr int COLS = 64 / LPC;
@@ -608,82 +597,27 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(OuterArgs a) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int r = lane % LPC, j = (blockIdx.x * NW + wave) * COLS + lane / LPC;
     const int H = a.H, D = a.D, V = a.V, VS = a.VS;  // VS = V (+ 1: the normaliser's column, whose value is 1)
-    const int runs = PASS == 0 ? 1 : (PASS == 1 ? a.segs - 1 : a.segs);
-    const int h = blockIdx.y, s = blockIdx.z / runs, seg = blockIdx.z - s * runs, g = h / (H / a.G);
-    int t0 = a.seq_starts[s], t1 = a.seq_starts[s + 1];
-    const int t_end = t1;
-    if constexpr (PASS != 0) {
-        const int per = outer_segment(t1 - t0, a.segs);
-        t0 += seg * per;
-        t1 = min(t0 + per, t_end);
-        if (PASS == 1 && t1 >= t_end) return;        // the last segment's local state is nobody's start
-    }
+    const int h = blockIdx.y, s = blockIdx.z, g = h / (H / a.G);
+    const int t0 = a.seq_starts[s], t1 = a.seq_starts[s + 1];
     if (t1 <= t0) return;                            // (the same in every thread of the block)
     const bool col = j < VS, ones = j == V;
-    auto load_rows = [&](const float* p, float (&x)[DR]) {      // this lane's rows of a [D] column; zeros past D
-#pragma unroll
-        for (int i = 0; i < DR; i += 4) {
-            if constexpr (VEC) {
-                const bool in = col && r * DR + i < D;      // (D % 4 == 0: a piece is inside or outside as a whole)
-                const float4 y = in ? *(const float4*)(p + i) : make_float4(0.f, 0.f, 0.f, 0.f);
-                x[i] = y.x; x[i + 1] = y.y; x[i + 2] = y.z; x[i + 3] = y.w;
-            } else {
-#pragma unroll
-                for (int e = 0; e < 4; ++e) x[i + e] = (col && r * DR + i + e < D) ? p[i + e] : 0.f;
-            }
-        }
-    };
-    auto store_rows = [&](float* p, const float (&x)[DR]) {
-#pragma unroll
-        for (int i = 0; i < DR; i += 4) {
-            if constexpr (VEC) {
-                if (col && r * DR + i < D) *(float4*)(p + i) = make_float4(x[i], x[i + 1], x[i + 2], x[i + 3]);
-            } else {
-#pragma unroll
-                for (int e = 0; e < 4; ++e)
-                    if (col && r * DR + i + e < D) p[i + e] = x[i + e];
-            }
-        }
-    };
-    const size_t at = ((size_t)h * VS + (col ? j : 0)) * D + r * DR;        // this lane's rows inside one sequence's state
-    const size_t one = (size_t)H * VS * D;
-    float* S_g = a.state + (size_t)a.slots[s] * one + at;
-    float* part = PASS == 0 ? nullptr : a.part + (size_t)s * a.segs * one + at;
-    const int pw = CHANNEL ? D : 1;
-    float* prod = PASS == 0 ? nullptr : a.prod + ((size_t)s * a.segs * H + h) * pw;      // + segment * H * pw
+    float* S_g = a.state + (((size_t)a.slots[s] * H + h) * VS + (col ? j : 0)) * D + r * DR;
     float S[DR];
-    if constexpr (PASS == 0) {
-        load_rows(S_g, S);
-    } else if constexpr (PASS == 1) {
-        if (seg == 0) {
-            load_rows(S_g, S);
-            store_rows(part, S);                     // (the state itself is overwritten by the last segment of pass 2)
+#pragma unroll
+    for (int i = 0; i < DR; i += 4) {
+        if constexpr (VEC) {
+            const bool in = col && r * DR + i < D;      // (D % 4 == 0: a piece is inside or outside as a whole)
+            const float4 x = in ? *(const float4*)(S_g + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+            S[i] = x.x; S[i + 1] = x.y; S[i + 2] = x.z; S[i + 3] = x.w;
         } else {
 #pragma unroll
-            for (int i = 0; i < DR; ++i) S[i] = 0.f;
-        }
-    } else {
-        if (seg == 0) {
-            load_rows(t1 == t_end ? S_g : part, S);
-        } else {
-            load_rows(part + one, S);
-            for (int e = 1; e < seg; ++e) {
-                float L[DR];
-                load_rows(part + (size_t)(e + 1) * one, L);
-                const float* K = prod + (size_t)e * H * pw;
-#pragma unroll
-                for (int i = 0; i < DR; ++i) S[i] = fmaf(CHANNEL ? (r * DR + i < D ? K[CHANNEL ? r * DR + i : 0] : 0.f) : K[0], S[i], L[i]);
-            }
+            for (int e = 0; e < 4; ++e) S[i + e] = (col && r * DR + i + e < D) ? S_g[i + e] : 0.f;
         }
     }
-    float u[CHANNEL && PASS != 1 ? DR : 1], K[CHANNEL && PASS == 1 ? DR : 1];
-    if constexpr (CHANNEL && PASS != 1) {
+    float u[CHANNEL ? DR : 1];
+    if constexpr (CHANNEL) {
 #pragma unroll
         for (int i = 0; i < DR; ++i) u[i] = r * DR + i < D ? a.bonus[(size_t)h * D + r * DR + i] : 0.f;
-    }
-    if constexpr (PASS == 1) {
-#pragma unroll
-        for (int i = 0; i < (CHANNEL ? DR : 1); ++i) K[i] = 1.f;
     }
     const float keep_fixed = a.keep_const ? a.keep[h] : 0.f;
     float nxt[NL][W], v_nxt[P], a_nxt[P], b_nxt[P];
@@ -693,9 +627,8 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(OuterArgs a) {
             const int idx = n * NT + tid, p = idx / PIECES, e = (idx - p * PIECES) * W, which = e / DP, row = e - which * DP;
             const int t = first + p;
             const bool ok = idx < P * PIECES && t < t1 && row < D;
-            const float* src = a.k + (size_t)t * a.ldk + (size_t)g * D;
-            if constexpr (PASS != 1) src = which == 1 ? a.q + (size_t)t * a.ldq + (size_t)g * D : src;
-            if constexpr (CHANNEL) src = which == OPS - 1 ? a.keep + ((size_t)t * H + h) * D : src;
+            const float* src = which == 0 ? a.k + (size_t)t * a.ldk + (size_t)g * D : a.q + (size_t)t * a.ldq + (size_t)g * D;
+            if constexpr (CHANNEL) src = which == 2 ? a.keep + ((size_t)t * H + h) * D : src;
             if constexpr (VEC) {
                 const float4 x = ok ? *(const float4*)(src + row) : make_float4(0.f, 0.f, 0.f, 0.f);
                 nxt[n][0] = x.x; nxt[n][W - 3] = x.y; nxt[n][W - 2] = x.z; nxt[n][W - 1] = x.w;
@@ -743,37 +676,28 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(OuterArgs a) {
             float sq = 0.f;
 #pragma unroll
             for (int i = 0; i < DR; i += 4) {
-                const float4 k4 = *(const float4*)(&kq[cur][p][0][r * DR] + i);
-                const float ka[4] = {k4.x, k4.y, k4.z, k4.w};
-                float qa[4] = {0.f, 0.f, 0.f, 0.f}, da[4] = {1.f, 1.f, 1.f, 1.f};
-                if constexpr (PASS != 1) {
-                    const float4 q4 = *(const float4*)(&kq[cur][p][OPS > 1 ? 1 : 0][r * DR] + i);
-                    qa[0] = q4.x; qa[1] = q4.y; qa[2] = q4.z; qa[3] = q4.w;
-                }
+                const float4 k4 = *(const float4*)(&kq[cur][p][0][r * DR] + i), q4 = *(const float4*)(&kq[cur][p][1][r * DR] + i);
+                const float ka[4] = {k4.x, k4.y, k4.z, k4.w}, qa[4] = {q4.x, q4.y, q4.z, q4.w};
                 if constexpr (CHANNEL) {
                     const float4 d4 = *(const float4*)(&kq[cur][p][OPS - 1][r * DR] + i);
-                    da[0] = d4.x; da[1] = d4.y; da[2] = d4.z; da[3] = d4.w;
-                }
+                    const float da[4] = {d4.x, d4.y, d4.z, d4.w};
 #pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    if constexpr (CHANNEL) {
-                        if constexpr (PASS != 1) sq = fmaf(fmaf(u[i + e] * ka[e], bv_cur[p], S[i + e]), qa[e], sq);
-                        else K[i + e] *= da[e];
+                    for (int e = 0; e < 4; ++e) {
+                        sq = fmaf(fmaf(u[i + e] * ka[e], bv_cur[p], S[i + e]), qa[e], sq);
                         S[i + e] = fmaf(ka[e], bv_cur[p], S[i + e] * da[e]);
-                    } else {
+                    }
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
                         S[i + e] = fmaf(ka[e], bv_cur[p], S[i + e] * a_cur[p]);
-                        if constexpr (PASS != 1) sq = fmaf(S[i + e], qa[e], sq);
+                        sq = fmaf(S[i + e], qa[e], sq);
                     }
                 }
             }
-            if constexpr (PASS == 1) {
-                if constexpr (!CHANNEL) K[0] *= a_cur[p];
-            } else {
-                sq = column_sum<LPC>(sq) * a.q_scale;
-                if (col && r == 0) {
-                    if (ones) a.nq[(size_t)t * H + h] = sq;
-                    else a.out[(size_t)t * a.ldo + (size_t)h * V + j] = sq;
-                }
+            sq = column_sum<LPC>(sq) * a.q_scale;
+            if (col && r == 0) {
+                if (ones) a.nq[(size_t)t * H + h] = sq;
+                else a.out[(size_t)t * a.ldo + (size_t)h * V + j] = sq;
             }
         };
         if (first + P <= t1) {
@@ -787,34 +711,282 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(OuterArgs a) {
         if (more) stage(cur ^ 1);                    // (the buffer that every wave left before the last barrier)
         __syncthreads();
     }
+#pragma unroll
+    for (int i = 0; i < DR; i += 4) {
+        if constexpr (VEC) {
+            if (col && r * DR + i < D) *(float4*)(S_g + i) = make_float4(S[i], S[i + 1], S[i + 2], S[i + 3]);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (col && r * DR + i + e < D) S_g[i + e] = S[i + e];
+        }
+    }
+}
+
+// ---------------------------------------------------------------------------
+// The same recurrence for long portions, cut into `segs` segments that run at once.  A portion in one piece is a chain
+// of tokens on few waves; cut, it is three launches:
+//   pass 1   every segment but the last from zero (the first from the carried state) to its local state L, with the
+//            product K of its forgetting factors;
+//   starts   S_(g+1) = K_g S_g + L_g, element by element: the state every segment starts from, in L's place;
+//   pass 2   every segment from its start, with its outputs; a sequence's last one writes the carried state.
+// Twice the updates on a `segs`-th of the chain, so here the work counts and not a token's latency: four lanes share a
+// column, and a lane holds DR rows of CPL columns (the 16-byte pieces 4i + r of the rows, i < DR / 4), so that a piece
+// of k, q or keep read from LDS serves 4 CPL products and a column's sum is two moves inside a quad.
+// Past a portion's end tokens are filled up with k = v = 0 and factors of one, which change nothing.
+// `part` [sequence][segs][H][VS][D]: the carried state, then the segments' local states; `prod` [sequence][segs][H][D or 1].
+// Grid: (ceil(VS / (NW 16 CPL)), heads, sequences x (segs - 1 or segs)).  D is a multiple of 4, operands are aligned.
+// ---------------------------------------------------------------------------
+#define OUTER_GROUP 8            // tokens that travel together
+#define OUTER_MIN_SEGMENT 64     // the fewest tokens of a segment that is not a sequence's last
+__host__ __device__ __forceinline__ int outer_segment(int n, int segs) {      // tokens of a segment of an n-token portion
+    const int per = ((n + segs - 1) / segs + OUTER_GROUP - 1) / OUTER_GROUP * OUTER_GROUP;
+    return per > OUTER_MIN_SEGMENT ? per : OUTER_MIN_SEGMENT;
+}
+
+template <int DR, int CPL, int NW, bool CHANNEL, int PASS>
+__global__ __launch_bounds__(NW * 64) void outer_segment_kernel(OuterArgs a) {
+    constexpr int DP = 4 * DR, P = OUTER_GROUP, NT = NW * 64, PIECES_R = DR / 4;
+    constexpr int OPS = (PASS == 1 ? 1 : 2) + (CHANNEL ? 1 : 0);      // k (, q) (, keep)
+    constexpr int PIECES = OPS * DP / 4;             // 16-byte loads that bring one token's operands
+    constexpr int NL = (P * PIECES + NT - 1) / NT;   // loads a thread makes per group
+    __shared__ __attribute__((aligned(16))) float kq[2][P][OPS][DP];      // two groups of P tokens
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 3;
+    const int H = a.H, D = a.D, V = a.V, VS = a.VS;
+    const int runs = PASS == 1 ? a.segs - 1 : a.segs;
+    const int h = blockIdx.y, s = blockIdx.z / runs, seg = blockIdx.z - s * runs, g = h / (H / a.G);
+    const int begin = a.seq_starts[s], end = a.seq_starts[s + 1], per = outer_segment(end - begin, a.segs);
+    const int t0 = begin + seg * per, t1 = min(t0 + per, end);
+    if (t1 <= t0 || (PASS == 1 && t1 >= end)) return;      // (the same in every thread; the last segment's local state is nobody's start)
+    const int first_col = (blockIdx.x * NW + wave) * 16 * CPL;
+    const bool wave_live = first_col < VS, two = CPL == 1 || first_col + 16 < VS;      // (the same in every lane of the wave)
+    int j[CPL];
+    bool col[CPL];
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) {
+        j[c] = first_col + 16 * c + (lane >> 2);
+        col[c] = j[c] < VS;
+    }
+    const size_t one = (size_t)H * VS * D;
+    const int pw = CHANNEL ? D : 1;
+    float* S_state = a.state + (size_t)a.slots[s] * one + (size_t)h * VS * D;
+    float* part = a.part + (size_t)s * a.segs * one + (size_t)h * VS * D;
+    float S[CPL][DR];
+    auto load_state = [&](const float* base) {
+#pragma unroll
+        for (int c = 0; c < CPL; ++c)
+#pragma unroll
+            for (int i = 0; i < PIECES_R; ++i) {
+                const int row = 16 * i + 4 * r;
+                const float4 x = col[c] && row < D ? *(const float4*)(base + (size_t)j[c] * D + row) : make_float4(0.f, 0.f, 0.f, 0.f);
+                S[c][4 * i] = x.x; S[c][4 * i + 1] = x.y; S[c][4 * i + 2] = x.z; S[c][4 * i + 3] = x.w;
+            }
+    };
+    auto store_state = [&](float* base) {
+#pragma unroll
+        for (int c = 0; c < CPL; ++c)
+#pragma unroll
+            for (int i = 0; i < PIECES_R; ++i) {
+                const int row = 16 * i + 4 * r;
+                if (col[c] && row < D)
+                    *(float4*)(base + (size_t)j[c] * D + row) = make_float4(S[c][4 * i], S[c][4 * i + 1], S[c][4 * i + 2], S[c][4 * i + 3]);
+            }
+    };
+    if (PASS == 1 && seg > 0) {
+#pragma unroll
+        for (int c = 0; c < CPL; ++c)
+#pragma unroll
+            for (int i = 0; i < DR; ++i) S[c][i] = 0.f;
+    } else if (PASS == 1) {
+        load_state(S_state);
+        store_state(part);                           // (the carried state itself is overwritten by pass 2's last segment)
+    } else {
+        load_state(seg == 0 && t1 == end ? S_state : part + (size_t)seg * one);
+    }
+    float u[CHANNEL && PASS == 2 ? DR : 1], K[CHANNEL && PASS == 1 ? DR : 1];
+    if constexpr (CHANNEL && PASS == 2) {
+#pragma unroll
+        for (int i = 0; i < PIECES_R; ++i) {
+            const int row = 16 * i + 4 * r;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) u[4 * i + e] = row < D ? a.bonus[(size_t)h * D + row + e] : 0.f;
+        }
+    }
     if constexpr (PASS == 1) {
-        store_rows(part + (size_t)(seg + 1) * one, S);
-        if (blockIdx.x == 0 && wave == 0 && lane < (CHANNEL ? LPC : 1)) {      // (every column's lanes hold the same products)
-            float* K_g = prod + (size_t)seg * H * pw;
+#pragma unroll
+        for (int i = 0; i < (CHANNEL ? DR : 1); ++i) K[i] = 1.f;
+    }
+    const float keep_fixed = a.keep_const ? a.keep[h] : 0.f;
+    float4 nxt[NL];
+    float v_nxt[P][CPL], a_nxt[P], b_nxt[P];
+    auto fetch = [&](int first) {
+#pragma unroll
+        for (int n = 0; n < NL; ++n) {
+            const int idx = n * NT + tid, p = idx / PIECES, e = (idx - p * PIECES) * 4, which = e / DP, row = e - which * DP;
+            const int t = first + p;
+            const bool ok = idx < P * PIECES && t < t1 && row < D;
+            const float* src = a.k + (size_t)t * a.ldk + (size_t)g * D;
+            float fill = 0.f;
+            if constexpr (PASS == 2) src = which == 1 ? a.q + (size_t)t * a.ldq + (size_t)g * D : src;
+            if constexpr (CHANNEL) {
+                src = which == OPS - 1 ? a.keep + ((size_t)t * H + h) * D : src;
+                fill = which == OPS - 1 ? 1.f : 0.f;
+            }
+            nxt[n] = ok ? *(const float4*)(src + row) : make_float4(fill, fill, fill, fill);
+        }
+#pragma unroll
+        for (int p = 0; p < P; ++p) {
+            const bool live = first + p < t1;
+#pragma unroll
+            for (int c = 0; c < CPL; ++c)
+                v_nxt[p][c] = (live && col[c]) ? (j[c] == V ? 1.0f : a.v[(size_t)(first + p) * a.ldv + (size_t)h * V + j[c]]) : 0.f;
+            if constexpr (CHANNEL) {
+                a_nxt[p] = 1.f;
+                b_nxt[p] = 1.f;
+            } else {
+                a_nxt[p] = live ? (a.keep_const ? keep_fixed : a.keep[(size_t)(first + p) * H + h]) : 1.f;
+                b_nxt[p] = live ? (a.take ? a.take[(size_t)(first + p) * H + h] : 1.f) : 0.f;
+            }
+        }
+    };
+    auto stage = [&](int slot) {
+#pragma unroll
+        for (int n = 0; n < NL; ++n) {
+            const int idx = n * NT + tid;
+            if (idx < P * PIECES) *(float4*)(&kq[slot][0][0][0] + (size_t)idx * 4) = nxt[n];
+        }
+    };
+    fetch(t0);
+    stage(0);
+    __syncthreads();
+    for (int first = t0, cur = 0; first < t1; first += P, cur ^= 1) {
+        float bv_cur[P][CPL], a_cur[P];
+#pragma unroll
+        for (int p = 0; p < P; ++p) {
+#pragma unroll
+            for (int c = 0; c < CPL; ++c) bv_cur[p][c] = b_nxt[p] * v_nxt[p][c];
+            a_cur[p] = a_nxt[p];
+        }
+        const bool more = first + P < t1;
+        if (more) fetch(first + P);                  // the next group's operands leave now and are staged after this group's work
+        auto tokens = [&](auto n_cols) {             // of the first NC of the lane's columns
+            constexpr int NC = decltype(n_cols)::value;
+#pragma unroll
+            for (int p = 0; p < P; ++p) {
+                float sq[NC][2];
+#pragma unroll
+                for (int c = 0; c < NC; ++c) sq[c][0] = sq[c][1] = 0.f;
+#pragma unroll
+                for (int i = 0; i < PIECES_R; ++i) {
+                    const float4 k4 = *(const float4*)&kq[cur][p][0][16 * i + 4 * r];
+                    const float ka[4] = {k4.x, k4.y, k4.z, k4.w};
+                    float qa[4] = {0.f, 0.f, 0.f, 0.f}, da[4] = {1.f, 1.f, 1.f, 1.f};
+                    if constexpr (PASS == 2) {
+                        const float4 q4 = *(const float4*)&kq[cur][p][OPS > 1 ? 1 : 0][16 * i + 4 * r];
+                        qa[0] = q4.x; qa[1] = q4.y; qa[2] = q4.z; qa[3] = q4.w;
+                    }
+                    if constexpr (CHANNEL) {
+                        const float4 d4 = *(const float4*)&kq[cur][p][OPS - 1][16 * i + 4 * r];
+                        da[0] = d4.x; da[1] = d4.y; da[2] = d4.z; da[3] = d4.w;
+                    }
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        const int m = 4 * i + e;
+                        if constexpr (CHANNEL && PASS == 1) K[m] *= da[e];
+                        const float uk = CHANNEL && PASS == 2 ? u[CHANNEL && PASS == 2 ? m : 0] * ka[e] : 0.f;
+#pragma unroll
+                        for (int c = 0; c < NC; ++c) {
+                            if constexpr (CHANNEL) {
+                                if constexpr (PASS == 2) sq[c][i & 1] = fmaf(fmaf(uk, bv_cur[p][c], S[c][m]), qa[e], sq[c][i & 1]);
+                                S[c][m] = fmaf(ka[e], bv_cur[p][c], S[c][m] * da[e]);
+                            } else {
+                                S[c][m] = fmaf(ka[e], bv_cur[p][c], S[c][m] * a_cur[p]);
+                                if constexpr (PASS == 2) sq[c][i & 1] = fmaf(S[c][m], qa[e], sq[c][i & 1]);
+                            }
+                        }
+                    }
+                }
+                if constexpr (PASS == 1) {
+                    if constexpr (!CHANNEL) K[0] *= a_cur[p];
+                } else {
+                    float y[NC];
+#pragma unroll
+                    for (int c = 0; c < NC; ++c) {
+                        y[c] = sq[c][0] + sq[c][1];
+                        y[c] += lane_pair_other(y[c]);
+                        y[c] += quad_half_other(y[c]);
+                    }
+                    // lane r of a quad stores column r of the lane's columns
+                    const int mine = NC == 1 ? j[0] : (r == 0 ? j[0] : j[NC - 1]);
+                    const float v = (NC == 1 || r == 0 ? y[0] : y[NC - 1]) * a.q_scale;
+                    if (r < NC && mine < VS && first + p < t1) {
+                        float* dst = mine == V ? a.nq + (size_t)(first + p) * H + h : a.out + (size_t)(first + p) * a.ldo + (size_t)h * V + mine;
+                        *dst = v;
+                    }
+                }
+            }
+        };
+        if (wave_live) {
+            if (two) tokens(std::integral_constant<int, CPL>{});
+            else tokens(std::integral_constant<int, 1>{});
+        }
+        if (more) stage(cur ^ 1);                    // (the buffer that every wave left before the last barrier)
+        __syncthreads();
+    }
+    if constexpr (PASS == 1) {
+        store_state(part + (size_t)(seg + 1) * one);
+        if (blockIdx.x == 0 && wave == 0 && lane < (CHANNEL ? 4 : 1)) {      // (every column's lanes hold the same products)
+            float* K_g = a.prod + (((size_t)s * a.segs + seg) * H + h) * pw;
             if constexpr (CHANNEL) {
 #pragma unroll
-                for (int i = 0; i < DR; ++i)
-                    if (r * DR + i < D) K_g[r * DR + i] = K[i];
+                for (int i = 0; i < PIECES_R; ++i)
+                    if (16 * i + 4 * r < D) *(float4*)(K_g + 16 * i + 4 * r) = make_float4(K[4 * i], K[4 * i + 1], K[4 * i + 2], K[4 * i + 3]);
             } else {
                 K_g[0] = K[0];
             }
         }
-    } else if (t1 == t_end) {
-        store_rows(S_g, S);
+    } else if (t1 == end) {
+        store_state(S_state);
     }
 }
 
-// columns of a state per block, by the sizes alone (as FX_OUTER dispatches)
-static int outer_columns(int D, int V) { return D <= 64 ? (V <= 32 ? 2 * 4 : 4 * 4) : (D <= 128 ? 4 * 2 : 8 * 2); }
+// The segments' starts, in their local states' place: part[g + 1] <- prod[g] part[g] + part[g + 1], g = 1 .. (part[1] is the
+// first segment's state from the carried one: a start already).  A thread per four elements of a state, which it takes
+// through the segments in order.  Grid: (ceil(H VS D / 1024), sequences).
+template <bool CHANNEL>
+__global__ __launch_bounds__(256) void outer_starts_kernel(OuterArgs a) {
+    const int s = blockIdx.y, D = a.D;
+    const long at = ((long)blockIdx.x * 256 + threadIdx.x) * 4, one = (long)a.H * a.VS * D;
+    const int n = a.seq_starts[s + 1] - a.seq_starts[s], per = outer_segment(n, a.segs);
+    const int used = (n + per - 1) / per;            // segments that hold tokens; those before the last have a local state
+    if (at >= one || used < 3) return;
+    const int h = (int)(at / ((long)a.VS * D)), d = (int)(at % D), pw = CHANNEL ? D : 1;
+    float* part = a.part + (size_t)s * a.segs * one + at;
+    const float* prod = a.prod + ((size_t)s * a.segs * a.H + h) * pw + (CHANNEL ? d : 0);
+    float4 S = *(const float4*)(part + one);
+#pragma unroll 4
+    for (int g = 1; g < used - 1; ++g) {
+        const float4 L = *(const float4*)(part + (size_t)(g + 1) * one);
+        float4 K;
+        if constexpr (CHANNEL) {
+            K = *(const float4*)(prod + (size_t)g * a.H * pw);
+        } else {
+            const float k = prod[(size_t)g * a.H];
+            K = make_float4(k, k, k, k);
+        }
+        S = make_float4(fmaf(K.x, S.x, L.x), fmaf(K.y, S.y, L.y), fmaf(K.z, S.z, L.z), fmaf(K.w, S.w, L.w));
+        *(float4*)(part + (size_t)(g + 1) * one) = S;
+    }
+}
 
-// Into how many segments portions of up to `longest` tokens are cut (1: one launch): enough for about four waves a
-// SIMD, none shorter than 128 tokens.
+// Into how many segments portions of up to `longest` tokens are cut (1: one piece): enough for about two waves a SIMD,
+// none shorter than OUTER_MIN_SEGMENT, at most 16.
 FX_API int fx_outer_segments(int n_seqs, int H, int D, int V, int normalizer, int longest) {
-    if (n_seqs <= 0 || H <= 0 || D <= 0 || V <= 0 || longest < 256) return 1;
-    const long blocks = (long)ceil_div(V + (normalizer ? 1 : 0), outer_columns(D, V)) * H * n_seqs;
-    const long waves = blocks * (D <= 64 ? (V <= 32 ? 2 : 4) : (D <= 128 ? 4 : 8));
-    long segs = 16L * fx_compute_units() / waves;
-    if (segs > longest / 128) segs = longest / 128;
+    if (n_seqs <= 0 || H <= 0 || D <= 0 || D % 4 || V <= 0 || longest < 4 * OUTER_MIN_SEGMENT) return 1;
+    const int cols = D <= 128 ? 32 : 16;             // of a wave
+    const long waves = (long)ceil_div(V + (normalizer ? 1 : 0), cols) * H * n_seqs;
+    long segs = 8L * fx_compute_units() / waves;
+    if (segs > longest / OUTER_MIN_SEGMENT) segs = longest / OUTER_MIN_SEGMENT;
     if (segs > 16) segs = 16;
     return segs < 2 ? 1 : (int)segs;
 }
@@ -830,33 +1002,40 @@ static int launch_gated_outer(const char* who, hipStream_t s, const OuterArgs& a
     FX_REQUIRE(a.keep, "%s: the forgetting factors are missing", who);
     if (n_seqs == 0) return 0;
     const bool vec = a.D % 4 == 0 && a.ldq % 4 == 0 && a.ldk % 4 == 0 &&
-                     (((uintptr_t)a.state | (uintptr_t)a.q | (uintptr_t)a.k | (uintptr_t)a.part | (CHANNEL ? (uintptr_t)a.keep : 0)) % 16) == 0;
-#define FX_OUTER_PASS(DR_, LPC_, NW_, PASS_, RUNS_)                                                                           \
+                     (((uintptr_t)a.state | (uintptr_t)a.q | (uintptr_t)a.k | (CHANNEL ? (uintptr_t)a.keep : 0)) % 16) == 0;
+    if (a.segs > 1 && vec) {
+        FX_REQUIRE((((uintptr_t)a.part | (uintptr_t)a.prod) % 16) == 0, "%s: the segments' room must be 16-byte aligned", who);
+#define FX_SEGMENTS(DR_, CPL_, NW_)                                                                                           \
     do {                                                                                                                      \
-        const int per_block = NW_ * 64 / LPC_;                                                                                \
-        const dim3 grid((a.VS + per_block - 1) / per_block, a.H, n_seqs * (RUNS_));                                           \
-        if (vec) gated_outer_kernel<DR_, LPC_, true, NW_, CHANNEL, PASS_><<<grid, NW_ * 64, 0, s>>>(a);                       \
-        else gated_outer_kernel<DR_, LPC_, false, NW_, CHANNEL, PASS_><<<grid, NW_ * 64, 0, s>>>(a);                          \
+        const int x = ceil_div(a.VS, NW_ * 16 * CPL_);                                                                        \
+        outer_segment_kernel<DR_, CPL_, NW_, CHANNEL, 1><<<dim3(x, a.H, n_seqs * (a.segs - 1)), NW_ * 64, 0, s>>>(a);         \
+        outer_starts_kernel<CHANNEL><<<dim3(ceil_div((long)a.H * a.VS * a.D, 1024), n_seqs), 256, 0, s>>>(a);                 \
+        outer_segment_kernel<DR_, CPL_, NW_, CHANNEL, 2><<<dim3(x, a.H, n_seqs * a.segs), NW_ * 64, 0, s>>>(a);               \
     } while (0)
-#define FX_OUTER(DR_, LPC_, NW_)                                    \
-    do {                                                            \
-        if (a.segs == 1) FX_OUTER_PASS(DR_, LPC_, NW_, 0, 1);       \
-        else {                                                      \
-            FX_OUTER_PASS(DR_, LPC_, NW_, 1, a.segs - 1);           \
-            FX_OUTER_PASS(DR_, LPC_, NW_, 2, a.segs);               \
-        }                                                           \
+        if (a.D <= 32) FX_SEGMENTS(8, 2, 2);
+        else if (a.D <= 64) FX_SEGMENTS(16, 2, 2);
+        else if (a.D <= 128) FX_SEGMENTS(32, 2, 4);
+        else FX_SEGMENTS(64, 1, 4);
+#undef FX_SEGMENTS
+        FX_CHECK_LAUNCH(who);
+        return 0;
+    }
+#define FX_OUTER(DR_, LPC_, NW_)                                                                                              \
+    do {                                                                                                                      \
+        const dim3 grid(ceil_div(a.VS, NW_ * 64 / LPC_), a.H, n_seqs);                                                        \
+        if (vec) gated_outer_kernel<DR_, LPC_, true, NW_, CHANNEL><<<grid, NW_ * 64, 0, s>>>(a);                              \
+        else gated_outer_kernel<DR_, LPC_, false, NW_, CHANNEL><<<grid, NW_ * 64, 0, s>>>(a);                                 \
     } while (0)
     if (a.D <= 64 && a.V <= 32) FX_OUTER(4, 16, 2);
     else if (a.D <= 64) FX_OUTER(4, 16, 4);
     else if (a.D <= 128) FX_OUTER(4, 32, 4);
     else FX_OUTER(8, 32, 8);
 #undef FX_OUTER
-#undef FX_OUTER_PASS
     FX_CHECK_LAUNCH(who);
     return 0;
 }
 
-// `segs` > 1: portions are cut (see above); `part` and `prod` are then float32 [n_seqs, segs, H, V (+ 1), D] and
+// `segs` > 1: portions are cut into segments (where operands are aligned and D is a multiple of 4, else run whole); `part` and `prod` are then float32 [n_seqs, segs, H, V (+ 1), D] and
 // [n_seqs, segs, H] (channel_outer: [n_seqs, segs, H, D]) that the call may overwrite.
 FX_API int fx_gated_outer(void* stream, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
                           const float* keep, int keep_const, const float* take, float* out, long ldo, float* nq, float* state,
@@ -1180,38 +1359,49 @@ FX_API int fx_token_shift(void* stream, int dtype, const void* x, long ldx, cons
 template <int TT, int C>
 __global__ __launch_bounds__(256) void lowrank_decay_kernel(const float* __restrict__ low, long ldl, const float* __restrict__ w2t,
                                                             const float* __restrict__ w0, float* __restrict__ out, int n_tokens, int R, int N) {
-    constexpr int KB = 128;
+    constexpr int KB = 128, KG = TT == 1 ? 16 : 4;   // k in LDS at a time; rows of w2t that are asked for together
     __shared__ __attribute__((aligned(16))) float xs[KB][TT];
     const int n = (blockIdx.x * 256 + threadIdx.x) * C, first = blockIdx.y * TT;      // (N is a multiple of C)
-    float acc[TT][C];
+    const float* w = w2t + min(n, N - C);
+    float acc[TT][C], nxt[KG][C];
 #pragma unroll
     for (int i = 0; i < TT; ++i)
 #pragma unroll
         for (int c = 0; c < C; ++c) acc[i][c] = 0.f;
+    auto fetch = [&](int k) {                        // (past the last row: that row again, which meets zeros in LDS)
+#pragma unroll
+        for (int e = 0; e < KG; ++e) {
+            const float* p = w + (size_t)min(k + e, R - 1) * N;
+            if constexpr (C == 4) {
+                const float4 w4 = *(const float4*)p;
+                nxt[e][0] = w4.x; nxt[e][C - 3] = w4.y; nxt[e][C - 2] = w4.z; nxt[e][C - 1] = w4.w;
+            } else {
+                nxt[e][0] = *p;
+            }
+        }
+    };
+    fetch(0);
     for (int k0 = 0; k0 < R; k0 += KB) {
-        const int kn = min(KB, R - k0);
+        const int kn = (min(KB, R - k0) + KG - 1) / KG * KG;
         if (k0) __syncthreads();
         for (int idx = threadIdx.x; idx < TT * kn; idx += 256) {
             const int i = idx / kn, k = idx - i * kn, t = first + i;
-            xs[k][i] = t < n_tokens ? tanhf(low[(size_t)t * ldl + k0 + k]) : 0.f;
+            xs[k][i] = t < n_tokens && k0 + k < R ? tanhf(low[(size_t)t * ldl + k0 + k]) : 0.f;
         }
         __syncthreads();
-        if (n < N) {
-            const float* w = w2t + (size_t)k0 * N + n;
-#pragma unroll 8
-            for (int k = 0; k < kn; ++k) {
-                float wv[C];
-                if constexpr (C == 4) {
-                    const float4 w4 = *(const float4*)(w + (size_t)k * N);
-                    wv[0] = w4.x; wv[1] = w4.y; wv[2] = w4.z; wv[3] = w4.w;
-                } else {
-                    wv[0] = w[(size_t)k * N];
-                }
+        for (int k = 0; k < kn; k += KG) {
+            float wv[KG][C];
+#pragma unroll
+            for (int e = 0; e < KG; ++e)
+#pragma unroll
+                for (int c = 0; c < C; ++c) wv[e][c] = nxt[e][c];
+            fetch(k0 + k + KG);                      // the next rows leave now and are used a group later
+#pragma unroll
+            for (int e = 0; e < KG; ++e)
 #pragma unroll
                 for (int i = 0; i < TT; ++i)
 #pragma unroll
-                    for (int c = 0; c < C; ++c) acc[i][c] = fmaf(xs[k][i], wv[c], acc[i][c]);
-            }
+                    for (int c = 0; c < C; ++c) acc[i][c] = fmaf(xs[k + e][i], wv[e][c], acc[i][c]);
         }
     }
     if (n >= N) return;
