@@ -733,7 +733,6 @@ __global__ __launch_bounds__(NW * 64) void gated_outer_kernel(OuterArgs a) {
 // Twice the updates on a `segs`-th of the chain, so here the work counts and not a token's latency: four lanes share a
 // column, and a lane holds DR rows of CPL columns (the 16-byte pieces 4i + r of the rows, i < DR / 4), so that a piece
 // of k, q or keep read from LDS serves 4 CPL products and a column's sum is two moves inside a quad.
-// Past a portion's end tokens are filled up with k = v = 0 and factors of one, which change nothing.
 // `part` [sequence][segs][H][VS][D]: the carried state, then the segments' local states; `prod` [sequence][segs][H][D or 1].
 // Grid: (ceil(VS / (NW 16 CPL)), heads, sequences x (segs - 1 or segs)).  D is a multiple of 4, operands are aligned.
 // ---------------------------------------------------------------------------
@@ -745,8 +744,8 @@ __host__ __device__ __forceinline__ int outer_segment(int n, int segs) {      //
 }
 
 template <int DR, int CPL, int NW, bool CHANNEL, int PASS>
-__global__ __launch_bounds__(NW * 64) void outer_segment_kernel(OuterArgs a) {
-    constexpr int DP = 4 * DR, P = OUTER_GROUP, NT = NW * 64, PIECES_R = DR / 4;
+__global__ __launch_bounds__(NW * 64, CHANNEL && DR > 32 ? 1 : 2) void outer_segment_kernel(OuterArgs a) {
+    constexpr int DP = 4 * DR, P = DR > 16 ? OUTER_GROUP / 2 : OUTER_GROUP, NT = NW * 64, PIECES_R = DR / 4;
     constexpr int OPS = (PASS == 1 ? 1 : 2) + (CHANNEL ? 1 : 0);      // k (, q) (, keep)
     constexpr int PIECES = OPS * DP / 4;             // 16-byte loads that bring one token's operands
     constexpr int NL = (P * PIECES + NT - 1) / NT;   // loads a thread makes per group
@@ -816,36 +815,49 @@ __global__ __launch_bounds__(NW * 64) void outer_segment_kernel(OuterArgs a) {
 #pragma unroll
         for (int i = 0; i < (CHANNEL ? DR : 1); ++i) K[i] = 1.f;
     }
-    const float keep_fixed = a.keep_const ? a.keep[h] : 0.f;
+    // What a thread brings of every group: piece idx = n NT + tid of the group's P PIECES, which is token idx / PIECES, then
+    // k, q or keep, then four rows.  Every load below is unconditional (a load under a condition is waited for where it
+    // stands): tokens past the segment's end read its last token again, rows past D the last four rows, whose values
+    // are multiplied away on their way into LDS, columns past V the last column, whose value is multiplied away too.
+    constexpr bool EXACT = (P * PIECES) % NT == 0;
+    const float* piece[NL];
+    long piece_ld[NL];
+    float piece_in[NL];
+    int piece_tok[NL];
+#pragma unroll
+    for (int n = 0; n < NL; ++n) {
+        const int idx = n * NT + tid, p = min(idx / PIECES, P - 1), e = (idx % PIECES) * 4, which = e / DP, row = e - which * DP;
+        const bool is_q = PASS == 2 && which == 1, is_keep = CHANNEL && which == OPS - 1;
+        piece[n] = (is_keep ? a.keep + (size_t)h * D : (is_q ? a.q + (size_t)g * D : a.k + (size_t)g * D)) + min(row, D - 4);
+        piece_ld[n] = is_keep ? (long)H * D : (is_q ? a.ldq : a.ldk);
+        piece_in[n] = row < D ? 1.f : 0.f;
+        piece_tok[n] = p;
+    }
+    const float* v_col[CPL];
+    float v_mul[CPL], v_add[CPL];                    // a column's value is v_mul v + v_add (the normaliser's: 1)
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) {
+        v_col[c] = a.v + (size_t)h * V + min(j[c], V - 1);
+        v_mul[c] = j[c] < V ? 1.f : 0.f;
+        v_add[c] = j[c] == V ? 1.f : 0.f;
+    }
+    const float* keep_h = a.keep + (CHANNEL ? 0 : h);
+    const float* take_h = (a.take ? a.take : a.keep) + (CHANNEL ? 0 : h);
+    const long keep_ld = CHANNEL || a.keep_const ? 0 : H, take_ld = !CHANNEL && a.take ? H : 0;
+    const bool takes = !CHANNEL && a.take != nullptr;
     float4 nxt[NL];
     float v_nxt[P][CPL], a_nxt[P], b_nxt[P];
     auto fetch = [&](int first) {
 #pragma unroll
-        for (int n = 0; n < NL; ++n) {
-            const int idx = n * NT + tid, p = idx / PIECES, e = (idx - p * PIECES) * 4, which = e / DP, row = e - which * DP;
-            const int t = first + p;
-            const bool ok = idx < P * PIECES && t < t1 && row < D;
-            const float* src = a.k + (size_t)t * a.ldk + (size_t)g * D;
-            float fill = 0.f;
-            if constexpr (PASS == 2) src = which == 1 ? a.q + (size_t)t * a.ldq + (size_t)g * D : src;
-            if constexpr (CHANNEL) {
-                src = which == OPS - 1 ? a.keep + ((size_t)t * H + h) * D : src;
-                fill = which == OPS - 1 ? 1.f : 0.f;
-            }
-            nxt[n] = ok ? *(const float4*)(src + row) : make_float4(fill, fill, fill, fill);
-        }
+        for (int n = 0; n < NL; ++n) nxt[n] = *(const float4*)(piece[n] + (size_t)min(first + piece_tok[n], t1 - 1) * piece_ld[n]);
 #pragma unroll
         for (int p = 0; p < P; ++p) {
-            const bool live = first + p < t1;
+            const int t = min(first + p, t1 - 1);
 #pragma unroll
-            for (int c = 0; c < CPL; ++c)
-                v_nxt[p][c] = (live && col[c]) ? (j[c] == V ? 1.0f : a.v[(size_t)(first + p) * a.ldv + (size_t)h * V + j[c]]) : 0.f;
-            if constexpr (CHANNEL) {
-                a_nxt[p] = 1.f;
-                b_nxt[p] = 1.f;
-            } else {
-                a_nxt[p] = live ? (a.keep_const ? keep_fixed : a.keep[(size_t)(first + p) * H + h]) : 1.f;
-                b_nxt[p] = live ? (a.take ? a.take[(size_t)(first + p) * H + h] : 1.f) : 0.f;
+            for (int c = 0; c < CPL; ++c) v_nxt[p][c] = v_col[c][(size_t)t * a.ldv];
+            if constexpr (!CHANNEL) {
+                a_nxt[p] = keep_h[(size_t)t * keep_ld];
+                b_nxt[p] = take_h[(size_t)t * take_ld];
             }
         }
     };
@@ -853,82 +865,99 @@ __global__ __launch_bounds__(NW * 64) void outer_segment_kernel(OuterArgs a) {
 #pragma unroll
         for (int n = 0; n < NL; ++n) {
             const int idx = n * NT + tid;
-            if (idx < P * PIECES) *(float4*)(&kq[slot][0][0][0] + (size_t)idx * 4) = nxt[n];
+            const float in = piece_in[n];
+            if (EXACT || idx < P * PIECES)
+                *(float4*)(&kq[slot][0][0][0] + (size_t)idx * 4) = make_float4(nxt[n].x * in, nxt[n].y * in, nxt[n].z * in, nxt[n].w * in);
         }
     };
+    // lane r of a quad stores column r of the lane's columns
+    const int mine = CPL == 1 ? j[0] : (r == 0 ? j[0] : j[CPL - 1]);
+    const bool stores = PASS == 2 && r < CPL && mine < VS;
+    float* dst = mine == V ? a.nq + (size_t)t0 * H + h : a.out + (size_t)t0 * a.ldo + (size_t)h * V + min(mine, V - 1);
+    const long dst_ld = mine == V ? H : a.ldo;
     fetch(t0);
     stage(0);
     __syncthreads();
     for (int first = t0, cur = 0; first < t1; first += P, cur ^= 1) {
-        float bv_cur[P][CPL], a_cur[P];
+        float bv_cur[P][CPL], a_cur[P], y_cur[P];
 #pragma unroll
         for (int p = 0; p < P; ++p) {
+            const float b = !takes ? 1.f : b_nxt[p];
 #pragma unroll
-            for (int c = 0; c < CPL; ++c) bv_cur[p][c] = b_nxt[p] * v_nxt[p][c];
+            for (int c = 0; c < CPL; ++c) bv_cur[p][c] = b * fmaf(v_nxt[p][c], v_mul[c], v_add[c]);
             a_cur[p] = a_nxt[p];
         }
         const bool more = first + P < t1;
         if (more) fetch(first + P);                  // the next group's operands leave now and are staged after this group's work
-        auto tokens = [&](auto n_cols) {             // of the first NC of the lane's columns
+        auto token = [&](int p, auto n_cols) {       // of the first NC of the lane's columns
             constexpr int NC = decltype(n_cols)::value;
+            float sq[NC][2];
 #pragma unroll
-            for (int p = 0; p < P; ++p) {
-                float sq[NC][2];
+            for (int c = 0; c < NC; ++c) sq[c][0] = sq[c][1] = 0.f;
 #pragma unroll
-                for (int c = 0; c < NC; ++c) sq[c][0] = sq[c][1] = 0.f;
+            for (int i = 0; i < PIECES_R; ++i) {
+                const float4 k4 = *(const float4*)&kq[cur][p][0][16 * i + 4 * r];
+                const float ka[4] = {k4.x, k4.y, k4.z, k4.w};
+                float qa[4] = {0.f, 0.f, 0.f, 0.f}, da[4] = {1.f, 1.f, 1.f, 1.f};
+                if constexpr (PASS == 2) {
+                    const float4 q4 = *(const float4*)&kq[cur][p][OPS > 1 ? 1 : 0][16 * i + 4 * r];
+                    qa[0] = q4.x; qa[1] = q4.y; qa[2] = q4.z; qa[3] = q4.w;
+                }
+                if constexpr (CHANNEL) {
+                    const float4 d4 = *(const float4*)&kq[cur][p][OPS - 1][16 * i + 4 * r];
+                    da[0] = d4.x; da[1] = d4.y; da[2] = d4.z; da[3] = d4.w;
+                }
 #pragma unroll
-                for (int i = 0; i < PIECES_R; ++i) {
-                    const float4 k4 = *(const float4*)&kq[cur][p][0][16 * i + 4 * r];
-                    const float ka[4] = {k4.x, k4.y, k4.z, k4.w};
-                    float qa[4] = {0.f, 0.f, 0.f, 0.f}, da[4] = {1.f, 1.f, 1.f, 1.f};
-                    if constexpr (PASS == 2) {
-                        const float4 q4 = *(const float4*)&kq[cur][p][OPS > 1 ? 1 : 0][16 * i + 4 * r];
-                        qa[0] = q4.x; qa[1] = q4.y; qa[2] = q4.z; qa[3] = q4.w;
-                    }
-                    if constexpr (CHANNEL) {
-                        const float4 d4 = *(const float4*)&kq[cur][p][OPS - 1][16 * i + 4 * r];
-                        da[0] = d4.x; da[1] = d4.y; da[2] = d4.z; da[3] = d4.w;
-                    }
+                for (int e = 0; e < 4; ++e) {
+                    const int m = 4 * i + e;
+                    if constexpr (CHANNEL && PASS == 1) K[m] *= da[e];
+                    const float uk = CHANNEL && PASS == 2 ? u[CHANNEL && PASS == 2 ? m : 0] * ka[e] : 0.f;
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        const int m = 4 * i + e;
-                        if constexpr (CHANNEL && PASS == 1) K[m] *= da[e];
-                        const float uk = CHANNEL && PASS == 2 ? u[CHANNEL && PASS == 2 ? m : 0] * ka[e] : 0.f;
-#pragma unroll
-                        for (int c = 0; c < NC; ++c) {
-                            if constexpr (CHANNEL) {
-                                if constexpr (PASS == 2) sq[c][i & 1] = fmaf(fmaf(uk, bv_cur[p][c], S[c][m]), qa[e], sq[c][i & 1]);
-                                S[c][m] = fmaf(ka[e], bv_cur[p][c], S[c][m] * da[e]);
-                            } else {
-                                S[c][m] = fmaf(ka[e], bv_cur[p][c], S[c][m] * a_cur[p]);
-                                if constexpr (PASS == 2) sq[c][i & 1] = fmaf(S[c][m], qa[e], sq[c][i & 1]);
-                            }
+                    for (int c = 0; c < NC; ++c) {
+                        if constexpr (CHANNEL) {
+                            if constexpr (PASS == 2) sq[c][i & 1] = fmaf(fmaf(uk, bv_cur[p][c], S[c][m]), qa[e], sq[c][i & 1]);
+                            S[c][m] = fmaf(ka[e], bv_cur[p][c], S[c][m] * da[e]);
+                        } else {
+                            S[c][m] = fmaf(ka[e], bv_cur[p][c], S[c][m] * a_cur[p]);
+                            if constexpr (PASS == 2) sq[c][i & 1] = fmaf(S[c][m], qa[e], sq[c][i & 1]);
                         }
                     }
                 }
-                if constexpr (PASS == 1) {
-                    if constexpr (!CHANNEL) K[0] *= a_cur[p];
-                } else {
-                    float y[NC];
+            }
+            if constexpr (PASS == 1) {
+                if constexpr (!CHANNEL) K[0] *= a_cur[p];
+            } else {
+                float y[NC];
 #pragma unroll
-                    for (int c = 0; c < NC; ++c) {
-                        y[c] = sq[c][0] + sq[c][1];
-                        y[c] += lane_pair_other(y[c]);
-                        y[c] += quad_half_other(y[c]);
-                    }
-                    // lane r of a quad stores column r of the lane's columns
-                    const int mine = NC == 1 ? j[0] : (r == 0 ? j[0] : j[NC - 1]);
-                    const float v = (NC == 1 || r == 0 ? y[0] : y[NC - 1]) * a.q_scale;
-                    if (r < NC && mine < VS && first + p < t1) {
-                        float* dst = mine == V ? a.nq + (size_t)(first + p) * H + h : a.out + (size_t)(first + p) * a.ldo + (size_t)h * V + mine;
-                        *dst = v;
-                    }
+                for (int c = 0; c < NC; ++c) {
+                    y[c] = sq[c][0] + sq[c][1];
+                    y[c] += lane_pair_other(y[c]);
+                    y[c] += quad_half_other(y[c]);
                 }
+                y_cur[p] = (NC == 1 || r == 0 ? y[0] : y[NC - 1]) * a.q_scale;
             }
         };
+        auto group = [&](auto n_cols) {
+            if (first + P <= t1) {                   // a whole group: one stretch of code
+#pragma unroll
+                for (int p = 0; p < P; ++p) token(p, n_cols);
+                if (stores) {
+#pragma unroll
+                    for (int p = 0; p < P; ++p) dst[p * dst_ld] = y_cur[p];
+                }
+            } else {
+#pragma unroll
+                for (int p = 0; p < P; ++p)
+                    if (first + p < t1) {
+                        token(p, n_cols);
+                        if (stores) dst[p * dst_ld] = y_cur[p];
+                    }
+            }
+            dst += P * dst_ld;
+        };
         if (wave_live) {
-            if (two) tokens(std::integral_constant<int, CPL>{});
-            else tokens(std::integral_constant<int, 1>{});
+            if (two) group(std::integral_constant<int, CPL>{});
+            else group(std::integral_constant<int, 1>{});
         }
         if (more) stage(cur ^ 1);                    // (the buffer that every wave left before the last barrier)
         __syncthreads();
@@ -979,16 +1008,19 @@ __global__ __launch_bounds__(256) void outer_starts_kernel(OuterArgs a) {
     }
 }
 
-// Into how many segments portions of up to `longest` tokens are cut (1: one piece): enough for about two waves a SIMD,
-// none shorter than OUTER_MIN_SEGMENT, at most 16.
+// Into how many segments portions of up to `longest` tokens are cut (1: one piece): enough for two waves a SIMD, none
+// shorter than OUTER_MIN_SEGMENT, at least 4 and at most 32.  (Where many sequences fill the GPU anyway four segments are
+// still ahead of one piece, whose 16 or 32 lanes to a column spend more instructions a token: 16 sequences of 1,024
+// tokens, 16 heads of 128 x 128 with a normaliser 1.39 -> 1.08 ms, 32 heads of 64 x 64 with decays per channel 0.65 -> 0.55;
+// one sequence of 2,048 tokens: 608 -> 169 us and 473 -> 88 us.)
 FX_API int fx_outer_segments(int n_seqs, int H, int D, int V, int normalizer, int longest) {
     if (n_seqs <= 0 || H <= 0 || D <= 0 || D % 4 || V <= 0 || longest < 4 * OUTER_MIN_SEGMENT) return 1;
-    const int cols = D <= 128 ? 32 : 16;             // of a wave
-    const long waves = (long)ceil_div(V + (normalizer ? 1 : 0), cols) * H * n_seqs;
+    const int nw = D <= 64 ? 2 : 4, cols = D <= 128 ? 32 : 16;      // waves of a block, columns of a wave
+    const long waves = (long)ceil_div(V + (normalizer ? 1 : 0), nw * cols) * nw * H * n_seqs;
     long segs = 8L * fx_compute_units() / waves;
+    if (segs < 4) segs = 4;
     if (segs > longest / OUTER_MIN_SEGMENT) segs = longest / OUTER_MIN_SEGMENT;
-    if (segs > 16) segs = 16;
-    return segs < 2 ? 1 : (int)segs;
+    return segs > 32 ? 32 : (int)segs;
 }
 
 template <bool CHANNEL>
