@@ -139,6 +139,22 @@ __device__ __forceinline__ void store_lane(const AttnArgs& a, int tok, int h, in
     store_out<T>(a, tok, h, d, v);
 }
 
+// the same for a lane's elements 16 cb + li of one row, all of its angles asked for together (elements past vd are not
+// stored: they read the last pair's angle)
+template <int CB>
+__device__ __forceinline__ void turn_back_row(const AttnArgs& a, int tok, int li, float (&y)[CB]) {
+    if (!a.turns) return;
+    const float2* angles = a.turns + (size_t)tok * (a.vd >> 1);
+    float2 cs[CB];
+#pragma unroll
+    for (int cb = 0; cb < CB; ++cb) cs[cb] = angles[min(16 * cb + li, a.vd - 1) >> 1];
+#pragma unroll
+    for (int cb = 0; cb < CB; ++cb) {
+        const float other = lane_pair_other(y[cb]) * cs[cb].y;
+        y[cb] = fmaf(y[cb], cs[cb].x, (li & 1) ? -other : other);
+    }
+}
+
 // block of the table and slot in its page of key t (a shift when the page size is a power of two)
 __device__ __forceinline__ void page_slot(const AttnArgs& a, int t, int& blk, int& slot) {
     if (a.bs_shift >= 0) {
@@ -1120,10 +1136,14 @@ __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(
         const int row = 4 * g + r;
         const float fr = __shfl(fin, row, 64);
         if (row < n) {
+            float y[CB];
+#pragma unroll
+            for (int cb = 0; cb < CB; ++cb) y[cb] = o[cb][r] * fr;
+            turn_back_row(a, tok0 + row, li, y);
 #pragma unroll
             for (int cb = 0; cb < CB; ++cb) {
                 const int d = 16 * cb + li;
-                if (d < vd) store_lane<bf16>(a, tok0 + row, h, d, o[cb][r] * fr);
+                if (d < vd) store_out<bf16>(a, tok0 + row, h, d, y[cb]);
             }
         }
     }
@@ -1338,8 +1358,12 @@ __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(Att
         const int row = 4 * g + r;
         const float fr = __shfl(fin, row, 64);
         if (row < n) {
+            float y[CB];
 #pragma unroll
-            for (int cb = 0; cb < CB; ++cb) store_lane<bf16>(a, tok0 + row, h, 16 * cb + li, o[cb][r] * fr);
+            for (int cb = 0; cb < CB; ++cb) y[cb] = o[cb][r] * fr;
+            turn_back_row(a, tok0 + row, li, y);
+#pragma unroll
+            for (int cb = 0; cb < CB; ++cb) store_out<bf16>(a, tok0 + row, h, 16 * cb + li, y[cb]);
         }
     }
 }
