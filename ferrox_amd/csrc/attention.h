@@ -12,7 +12,8 @@ int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void* out, l
                   const void* v_pages, const int* block_table, int max_blocks, const int* positions, const int* item_seq,
                   const int* item_tok, const int* item_n, int n_items, int nh, int nkv, int hd, int bs, int window, float scale,
                   int tile_q, int vd, int mask_chunk, int keep_first, const float* sinks, const void* gate, long ldg,
-                  float softcap, const float* slopes, int gate_per_head, const float* turns);
+                  float softcap, const float* slopes, int gate_per_head, const float* turns, int gate_f32, const float* bias,
+                  int bias_n);
 
 // `vd`: size of a value (and output) head, 0 for hd; part_o is then [n_items, nh, splits, vd].  `mask_chunk` > 0: a query
 // at position p sees the keys t <= p with floor(t / mask_chunk) == floor(p / mask_chunk) (instead of a window).
@@ -22,7 +23,10 @@ int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void* out, l
 // [tokens, nh], one number for all outputs of a head.  `softcap` > 0: a scaled score s
 // becomes softcap * tanh(s / softcap).  `slopes` (float32 [nh] or null): the score of key t for the query at
 // position p then loses slopes[h] * (p - t).  `turns` ([tokens, vd / 2] pairs (cos, sin), 8-byte aligned, or null): the
-// output pair (2m, 2m + 1) of every head is turned back by the token's angle m, before the gate.
+// output pair (2m, 2m + 1) of every head is turned back by the token's angle m, before the gate.  `gate_f32`: the gate is
+// float32 whatever the type of `out`.  `bias` (float32 [nh, 16 + bias_n + 16] or null): the score of a key at distance d
+// gains bias[h][16 + bias_n - 1 - min(d, bias_n - 1)]; the 16 floats in front repeat the farthest distance's, those behind
+// may hold anything finite.
 // Single queries.  The keys are cut into `splits` chunks of `chunk` positions; the chunks' partial results go through
 // part_o [n_items, nh, splits, hd] and part_ml [n_items, nh, splits, 2] (float32, brought by the caller).
 int fx_attn_decode(void* stream, int dtype, const void* q, long ldq, void* out, long ldo, const void* k_pages,
@@ -30,7 +34,7 @@ int fx_attn_decode(void* stream, int dtype, const void* q, long ldq, void* out, 
                    const int* item_tok, int n_items, int nh, int nkv, int hd, int bs, int window, float scale,
                    float* part_o, float* part_ml, int splits, int chunk, int waves, int vd, int mask_chunk, int keep_first,
                    const float* sinks, const void* gate, long ldg, float softcap, const float* slopes, int gate_per_head,
-                   const float* turns);
+                   const float* turns, int gate_f32, const float* bias, int bias_n);
 
 // The same for callers that cannot allocate device memory: code under HIP graph capture, tight serving loops,
 // harnesses that forbid hipMalloc.  It has no counterpart in the reference.  The partial results live in an array

@@ -43,12 +43,15 @@ struct AttnArgs {
     int mask_chunk;      // > 0: the chunked mask
     int keep_first;      // > 0 (with a window): keys t < keep_first stay visible to every later query
     const float* sinks;  // [n_heads] or null: a logit per head that joins the softmax's denominator
-    const void* gate;    // [tokens, n_heads * vd] or null (type of out): the output is multiplied by sigmoid(gate)
+    const void* gate;    // [tokens, n_heads * vd] or null (type of out, or float32): the output is multiplied by sigmoid(gate)
     long ldg;
     int gate_per_head;   // 1: the gate is [tokens, n_heads], one number for all of a head's outputs
     float softcap;       // > 0: a scaled score s becomes softcap * tanh(s / softcap)
     const float* slopes; // [n_heads] or null: the score of key t for the query at p then loses slopes[h] * (p - t)
     const float2* turns; // [tokens, vd / 2] (cos, sin) or null: output pair (2m, 2m + 1) is turned back by that angle
+    int gate_f32;        // 1: the gate is float32, whatever the type of out
+    const float* bias;   // or null: a number per head and distance that joins the (scaled, capped) score; see below
+    int bias_n;          // distances 0 .. bias_n - 1 have a number of their own, longer ones that of bias_n - 1
     int bs_shift;        // log2(bs) if bs is a power of two, else -1
     int n_items;
     float scale;
@@ -70,14 +73,42 @@ __device__ __forceinline__ int first_visible(const AttnArgs& a, int p) {
     if (a.mask_chunk > 0) return p - p % a.mask_chunk;
     return a.window > 0 ? max(0, p - a.window + 1) : 0;
 }
-// A scaled score on its way into the softmax: capped, then less the head's penalty for the distance p - t.
-__device__ __forceinline__ float shaped_score(const AttnArgs& a, float slope, float s, int distance) {
-    if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
-    return fmaf(-slope, (float)distance, s);
-}
-__host__ __device__ __forceinline__ bool shapes_scores(const AttnArgs& a) { return a.softcap > 0.f || a.slopes != nullptr; }
+__host__ __device__ __forceinline__ bool shapes_scores(const AttnArgs& a) { return a.softcap > 0.f || a.slopes != nullptr || a.bias != nullptr; }
 // whether queries see a bounded stretch of keys (a window or a chunk) rather than all before them
 __device__ __forceinline__ bool bounded_keys(const AttnArgs& a) { return a.window > 0 || a.mask_chunk > 0; }
+
+// The distance bias of a head is a row of BIAS_PAD + bias_n + BIAS_PAD floats that runs from far to near: the number for
+// distance d stands at BIAS_PAD + bias_n - 1 - d, so the numbers of consecutive keys follow each other; in front of them
+// stands the farthest one BIAS_PAD times, behind them what keys later than the query read and nobody uses.
+#define BIAS_PAD 16
+__host__ __device__ __forceinline__ int bias_row_len(const AttnArgs& a) { return a.bias_n + 2 * BIAS_PAD; }
+__device__ __forceinline__ float bias_at(const AttnArgs& a, int h, int distance) {      // distance >= 0
+    return a.bias[(size_t)h * bias_row_len(a) + BIAS_PAD + a.bias_n - 1 - min(distance, a.bias_n - 1)];
+}
+// A scaled score on its way into the softmax: capped, less the head's penalty for the distance p - t, plus the head's
+// bias for it (keys later than the query are masked: theirs is not looked up).
+__device__ __forceinline__ float shaped_score(const AttnArgs& a, int h, float slope, float s, int distance) {
+    if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
+    s = fmaf(-slope, (float)distance, s);
+    return a.bias ? s + bias_at(a, h, max(distance, 0)) : s;
+}
+// where in the row the numbers of 16 consecutive keys begin, `distance` being that of the first of them (which may be
+// later than the query, if all of them are)
+__device__ __forceinline__ int bias_first(const AttnArgs& a, int distance) {
+    return min(max(BIAS_PAD + a.bias_n - 1 - distance, 0), a.bias_n + 2 * BIAS_PAD - 16);
+}
+// the numbers themselves, from memory: rows start and distances fall at any multiple of four bytes
+typedef float fx_f32x4_any __attribute__((ext_vector_type(4), aligned(4)));
+struct BiasRow {
+    fx_f32x4_any v[4];
+};
+__device__ __forceinline__ BiasRow fetch_bias(const AttnArgs& a, int h, int distance) {
+    const float* p = a.bias + (size_t)h * bias_row_len(a) + bias_first(a, distance);
+    BiasRow b;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) b.v[i] = *(const fx_f32x4_any*)(p + 4 * i);
+    return b;
+}
 
 // The keys a block may touch: t < end and (t >= begin or t < keep), keep being the kept first keys of the
 // sequence (0: none).  Pages of other keys may have been given back.
@@ -119,7 +150,8 @@ __device__ __forceinline__ float finish_row(const AttnArgs& a, int h, float m, f
 template <typename T>
 __device__ __forceinline__ void store_out(const AttnArgs& a, int tok, int h, int d, float v) {
     if (a.gate) {
-        const float gv = to_float(((const T*)a.gate)[(size_t)tok * a.ldg + (a.gate_per_head ? (size_t)h : (size_t)h * a.vd + d)]);
+        const size_t at = (size_t)tok * a.ldg + (a.gate_per_head ? (size_t)h : (size_t)h * a.vd + d);
+        const float gv = a.gate_f32 ? ((const float*)a.gate)[at] : to_float(((const T*)a.gate)[at]);
         v *= 1.f / (1.f + expf(-gv));
     }
     from_float((T*)a.out + (size_t)tok * a.ldo + (size_t)h * a.vd + d, v);
@@ -263,7 +295,7 @@ __global__ __launch_bounds__(64) void attn_tile_kernel(AttnArgs a) {
 #pragma unroll
         for (int i = 0; i < TQ; ++i) {
             const bool vis = in_range && t <= pos[i] && (t >= first_visible(a, pos[i]) || t < a.keep_first);
-            if (shaped) s[i] = shaped_score(a, slope, s[i], pos[i] - t);
+            if (shaped) s[i] = shaped_score(a, h, slope, s[i], pos[i] - t);
             const float sv = vis ? s[i] : NEG_INF;
             const float m_new = fmaxf(m[i], wave_max(sv));
             al[i] = (m_new == NEG_INF) ? 1.f : expf(m[i] - m_new);
@@ -344,7 +376,7 @@ __global__ __launch_bounds__(64) void attn_decode_kernel(AttnArgs a) {
             const T* kr = key_row<T>(a, bt, kvh, t);
             for (int d = 0; d < hd; ++d) s = fmaf(Qs[d], to_float(kr[d]), s);
         }
-        if (shapes_scores(a)) s = shaped_score(a, a.slopes ? a.slopes[h] : 0.f, s, p - t);
+        if (shapes_scores(a)) s = shaped_score(a, h, a.slopes ? a.slopes[h] : 0.f, s, p - t);
         const float sv = vis ? s : NEG_INF;
         const float m_new = fmaxf(m, wave_max(sv));
         const float al = (m_new == NEG_INF) ? 1.f : expf(m - m_new);
@@ -477,8 +509,17 @@ __device__ __forceinline__ float quad_sum(float x) {
 // A lane's 16 raw scores sc[kb][r] of keys key0 + 4*kb + r, scaled, capped and less the head's penalty for the
 // distance from the row's query at qpos (`shaped_score` with a tanh made of one exponential and one reciprocal, whose
 // error, some 1e-7 of the cap, is far below what bfloat16 operands leave of a score): afterwards they are scores in natural
-// units, and the softmax step takes them with c = log2(e).
-__device__ __forceinline__ void shape_scores(f32x4_t (&sc)[4], int key0, const AttnArgs& a, float slope, int qpos) {
+// units, and the softmax step takes them with c = log2(e).  `bias(i)`: the head's bias for key key0 + i (asked for where
+// the launch has one).
+template <typename B>
+__device__ __forceinline__ void shape_scores(f32x4_t (&sc)[4], int key0, const AttnArgs& a, float slope, int qpos, B&& bias) {
+    if (a.bias && a.softcap <= 0.f && !a.slopes) {      // a bias alone: one multiply-add a score
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) sc[kb][r] = fmaf(sc[kb][r], a.scale, bias(4 * kb + r));
+        return;
+    }
     // tanh(x) = 1 - 2 / (1 + e^2x): the exponent in base 2 with the scale folded in, the quotient from the hardware's
     // reciprocal (1 ulp), cap and -2 cap as the multiply-add's constants
     const bool capped = a.softcap > 0.f;
@@ -494,6 +535,12 @@ __device__ __forceinline__ void shape_scores(f32x4_t (&sc)[4], int key0, const A
             else s = sc[kb][r] * a.scale;
             sc[kb][r] = fmaf(-slope, d0 - (float)(4 * kb + r), s);
         }
+    if (a.bias) {
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) sc[kb][r] += bias(4 * kb + r);
+    }
 }
 
 // One step of the one-pass softmax on a lane's 16 raw scores sc[kb][r] of keys key0 + 4*kb + r
@@ -598,9 +645,9 @@ struct WaveAttn {
     }
 
     // keys [kt0, kt0 + 64); this lane's row sees key t iff t <= hi and (lo <= t or t < span.keep) (hi < lo: row unused)
-    // `slope`, `qpos`: the row's distance penalty and its query's position, where the scores are shaped
+    // `slope`, `qpos`, `head`: the row's distance penalty, its query's position and its head, where the scores are shaped
     __device__ __forceinline__ void tile(const AttnArgs& a, const PageLookup& pl, int kvh, int kt0, const KeySpan& span,
-                                         int lo, int hi, float slope = 0.f, int qpos = 0) {
+                                         int lo, int hi, float slope, int qpos, int head) {
         const int kv_end = span.end;
         const int lane = threadIdx.x & 63, li = lane & 15, g = lane >> 4;
         const int l8 = li & 7, lh = li >> 3;
@@ -639,6 +686,8 @@ struct WaveAttn {
             page_slot(a, span.has(key_b) ? key_b : safe_group, kblk, kslots_b[kb]);
             kpage_b[kb] = pl.page(kblk);
         }
+        BiasRow bias = {};
+        if (a.bias) bias = fetch_bias(a, head, qpos - (kt0 + 16 * g));
         const bf16* vbase = (const bf16*)a.v_pages + ((size_t)vpage * a.nkv + kvh) * vd * bs + vslot;
         uint4 vv[EARLY_V ? CB : 1][2];
         const uint32_t vmask = opaque_mask(vlive);
@@ -710,7 +759,7 @@ struct WaveAttn {
         // softmax on this lane's 16 scores (keys kt0 + 16g + 4kb + r); the row's four lanes share max and sum
         uint4 p_lo, p_hi;
         const bool shaped = shapes_scores(a);
-        if (shaped) shape_scores(sc, kt0 + 16 * g, a, slope, qpos);
+        if (shaped) shape_scores(sc, kt0 + 16 * g, a, slope, qpos, [&](int i) { return bias.v[i >> 2][i & 3]; });
         const float alpha = softmax_step<true>(sc, kt0 + 16 * g, lo, hi, shaped ? LOG2E : a.scale * LOG2E, m, l, p_lo, p_hi, span.keep);
         const bool rescale = __builtin_amdgcn_ballot_w64(alpha != 1.f) != 0;
         float al[4] = {1.f, 1.f, 1.f, 1.f};
@@ -773,7 +822,7 @@ __global__ __launch_bounds__(64) void attn_mfma_tile_kernel(AttnArgs a) {
     const KeySpan span = {kv_begin, kv_end, a.keep_first};
     const TileWalk walk = tile_walk(span);
     const float slope = a.slopes ? a.slopes[h] : 0.f;
-    for (int ti = 0; ti < walk.n; ++ti) w.tile(a, pl, kvh, walk.start(ti), span, lo, hi, slope, hi);
+    for (int ti = 0; ti < walk.n; ++ti) w.tile(a, pl, kvh, walk.start(ti), span, lo, hi, slope, max(hi, 0), h);
     const float fin = li < n ? finish_row<true>(a, h, w.m, w.l) : 0.f;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -846,7 +895,7 @@ __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(Att
         const TileWalk walk = tile_walk(span);
         const int lo = row_ok ? kv_begin : 1, hi = row_ok ? kv_end - 1 : 0;
         const float slope = (a.slopes && row_ok) ? a.slopes[h0 + li] : 0.f;      // (a row is a query head here)
-        for (int ti = wave; ti < walk.n; ti += n_waves) w.tile(a, pl, kvh, walk.start(ti), span, lo, hi, slope, p);
+        for (int ti = wave; ti < walk.n; ti += n_waves) w.tile(a, pl, kvh, walk.start(ti), span, lo, hi, slope, p, h0 + min(li, n - 1));
     }
     if (n_waves == 1) {
         // one wave: nothing to merge, the rows go out from the registers that hold them (lane (li, g) has rows
@@ -949,6 +998,30 @@ __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(Att
     }
 }
 
+// A head's row of biases for a block that walks over many tiles: a copy in LDS (dynamic, sized by the launch; a load from
+// memory inside the walk would be waited for behind the tiles that are on their way), or the row itself where it is too
+// long for that.
+#define BIAS_LDS_MAX 2048      // floats
+__device__ __forceinline__ bool bias_in_lds(const AttnArgs& a) { return bias_row_len(a) <= BIAS_LDS_MAX; }
+__device__ __forceinline__ void stage_bias(const AttnArgs& a, int h, float* lds) {      // every thread; a barrier follows before its use
+    if (!a.bias || !bias_in_lds(a)) return;
+    const float* row = a.bias + (size_t)h * bias_row_len(a);
+    for (int i = threadIdx.x; i < bias_row_len(a); i += blockDim.x) lds[i] = row[i];
+}
+// the numbers of 16 consecutive keys, `distance` that of the first (one branch around all of them, so that the reads are
+// plain LDS or plain memory reads)
+__device__ __forceinline__ BiasRow read_bias(const AttnArgs& a, int h, const float* lds, int distance) {
+    if (!bias_in_lds(a)) return fetch_bias(a, h, distance);
+    BiasRow b;
+    const float* p = lds + bias_first(a, distance);
+#pragma unroll
+    for (int i = 0; i < 16; ++i) b.v[i >> 2][i & 3] = p[i];
+    return b;
+}
+static size_t bias_lds_bytes(const AttnArgs& a) {
+    return a.bias && bias_row_len(a) <= BIAS_LDS_MAX ? (size_t)bias_row_len(a) * sizeof(float) : 0;
+}
+
 // Prefill with the keys and values of a tile shared through LDS: a block of four waves owns up
 // to 64 consecutive queries of one head (16 each); per tile of 64 keys the block stages K
 // (rows permuted so that the 16 keys an MFMA operand needs lie in consecutive rows) and the
@@ -963,6 +1036,7 @@ __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(
     constexpr int NK = (KCH + 255) / 256, NV = (VCH + 255) / 256;
     __shared__ __attribute__((aligned(16))) bf16 Ks[64 * KROW];
     __shared__ __attribute__((aligned(16))) bf16 Vs[HD * VROW];
+    extern __shared__ float bias_lds[];
     // Blocks go to the 8 XCDs in turn, each with an L2 of its own: block b runs on XCD b % 8.  The
     // (head, item) pairs are dealt out so that an XCD works through whole heads, whose keys and
     // values then stay in its L2, and the items with the longest key range start first.
@@ -1026,6 +1100,7 @@ __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(
     int first_blk, last_blk, unused;
     page_slot(a, kv_begin, first_blk, unused);
     page_slot(a, kv_end - 1, last_blk, unused);
+    stage_bias(a, h, bias_lds);
     const PageLookup pl = stage_pages(bt, page_copy, first_blk, last_blk);
     auto fetch = [&](uint4* kreg, uint4* vreg, int kt0) {
         size_t kbase[4], vbase[4];     // page and slot of each group of 16 keys of the tile (the same for all threads)
@@ -1114,7 +1189,11 @@ __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(
         // tiles that every row of this wave sees whole need no mask
         const bool whole = kt0 >= w_lo_max && kt0 + 63 <= w_hi_min && kt0 >= kv_begin;
         uint4 p_lo, p_hi;
-        if (shaped) shape_scores(sc, kt0 + 16 * g, a, slope, hi);
+        if (shaped) {
+            BiasRow bias = {};
+            if (a.bias) bias = read_bias(a, h, bias_lds, max(hi, 0) - (kt0 + 16 * g));
+            shape_scores(sc, kt0 + 16 * g, a, slope, hi, [&](int i) { return bias.v[i >> 2][i & 3]; });
+        }
         const float alpha = whole ? softmax_step<false>(sc, kt0 + 16 * g, lo, hi, cs, m, l, p_lo, p_hi)
                                   : softmax_step<true>(sc, kt0 + 16 * g, lo, hi, cs, m, l, p_lo, p_hi, span.keep);
         const bool rescale = __builtin_amdgcn_ballot_w64(alpha != 1.f) != 0;
@@ -1180,6 +1259,7 @@ __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(Att
     constexpr int TILE = 2 * 64 * HD;           // elements of a stage: keys, then values
     static_assert(NS == 2 || NS == 3, "two or three stages");
     __shared__ __attribute__((aligned(1024))) bf16 tiles[G * NS * TILE];
+    extern __shared__ float bias_lds[];
     __shared__ int page_copy[PAGE_COPY];
     const int per_xcd = (a.n_items * a.nh + 7) / 8;
     const int logical = (blockIdx.x % 8) * per_xcd + blockIdx.x / 8;
@@ -1232,6 +1312,7 @@ __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(Att
     int first_blk, last_blk, unused;
     page_slot(a, kv_begin, first_blk, unused);
     page_slot(a, kv_end - 1, last_blk, unused);
+    stage_bias(a, h, bias_lds);
     const PageLookup pl = stage_pages(bt, page_copy, first_blk, last_blk);
     const KeySpan span = {kv_begin, kv_end, a.keep_first};
     const TileWalk walk = tile_walk(span);
@@ -1310,7 +1391,11 @@ __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(Att
         }
         const bool whole = kt0 >= w_lo_max && kt0 + 63 <= w_hi_min && kt0 >= kv_begin;
         uint4 p_lo, p_hi;
-        if (shaped) shape_scores(sc, kt0 + 16 * g, a, slope, hi);
+        if (shaped) {
+            BiasRow bias = {};
+            if (a.bias) bias = read_bias(a, h, bias_lds, max(hi, 0) - (kt0 + 16 * g));
+            shape_scores(sc, kt0 + 16 * g, a, slope, hi, [&](int i) { return bias.v[i >> 2][i & 3]; });
+        }
         const float alpha = whole ? softmax_step<false>(sc, kt0 + 16 * g, lo, hi, cs, m, l, p_lo, p_hi)
                                   : softmax_step<true>(sc, kt0 + 16 * g, lo, hi, cs, m, l, p_lo, p_hi, span.keep);
         const bool rescale = __builtin_amdgcn_ballot_w64(alpha != 1.f) != 0;
@@ -1416,8 +1501,10 @@ FX_API int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void*
                          const int* positions, const int* item_seq, const int* item_tok, const int* item_n,
                          int n_items, int nh, int nkv, int hd, int bs, int window, float scale, int tile_q,
                          int vd, int mask_chunk, int keep_first, const float* sinks, const void* gate, long ldg,
-                         float softcap, const float* slopes, int gate_per_head, const float* turns) {
+                         float softcap, const float* slopes, int gate_per_head, const float* turns, int gate_f32, const float* bias,
+                         int bias_n) {
     if (vd <= 0) vd = hd;
+    FX_REQUIRE(!bias || bias_n >= 1, "attn_tiles: a distance bias for %d distances", bias_n);
     FX_REQUIRE(!turns || vd % 2 == 0, "attn_tiles: outputs that are turned back come in pairs, a value head has %d", vd);
     FX_REQUIRE(softcap >= 0.f && softcap < INFINITY, "attn_tiles: a cap of %g on the scores", (double)softcap);
     if (check_common("attn_tiles", dtype, nh, nkv, hd, bs, window, scale, vd, mask_chunk, keep_first)) return 1;
@@ -1433,10 +1520,12 @@ FX_API int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void*
     a.keep_first = window > 0 ? keep_first : 0; a.sinks = sinks; a.gate = gate; a.ldg = ldg;
     a.gate_per_head = gate_per_head ? 1 : 0;
     a.softcap = softcap; a.slopes = slopes; a.turns = (const float2*)turns;
+    a.gate_f32 = gate_f32 ? 1 : 0; a.bias = bias; a.bias_n = bias_n;
     a.bs_shift = log2_or_minus_one(bs);
     a.n_items = n_items;
     dim3 grid(n_items * 4, nh), grid_blocks(8 * ceil_div((long)n_items * nh, 8));     // a wave per 16 queries / a block per item
     hipStream_t s = (hipStream_t)stream;
+    const size_t shm = bias_lds_bytes(a);
     // no more blocks than CUs: a block's chain of tiles is what takes the time, and two groups of waves halve it
     // (measured: 512-token portions at depth 8k-24k 130 and 360 us against 214 and 616 us; from 448 blocks on, one
     // group and two blocks to a CU are as fast or faster)
@@ -1450,23 +1539,23 @@ FX_API int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void*
         attn_tile_kernel<bf16, HD_MAX_ANY><<<grid, 64, 0, s>>>(a);
     else if (mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd) && hd > 128) {
         // the widest heads: tiles of 64 keys (34 KB) and their values (36 KB) staged in LDS for the block's 64 queries
-        attn_mfma_block_kernel<256><<<grid_blocks, 256, 0, s>>>(a);
+        attn_mfma_block_kernel<256><<<grid_blocks, 256, shm, s>>>(a);
     } else if (mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd) && vd != hd) {
         if (hd <= 64) attn_mfma_tile_kernel<64><<<grid, 64, 0, s>>>(a);
         else attn_mfma_tile_kernel<128><<<grid, 64, 0, s>>>(a);
     } else if (mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd)) {
-        if (tile_q == 128 && hd == 128 && two_groups) attn_mfma_direct_kernel<128, 2, 8, 2><<<grid_blocks, 1024, 0, s>>>(a);
-        else if (tile_q == 128 && hd == 64 && two_groups) attn_mfma_direct_kernel<64, 2, 8, 2><<<grid_blocks, 1024, 0, s>>>(a);
-        else if (tile_q == 128 && hd == 128) attn_mfma_direct_kernel<128, 2, 8><<<grid_blocks, 512, 0, s>>>(a);
-        else if (tile_q == 128) attn_mfma_direct_kernel<64, 2, 8><<<grid_blocks, 512, 0, s>>>(a);
-        else if (bs % 64 == 0 && hd == 128 && g_direct == 2 && two_groups) attn_mfma_direct_kernel<128, 2, 4, 2><<<grid_blocks, 512, 0, s>>>(a);
-        else if (bs % 64 == 0 && hd == 64 && g_direct == 2 && two_groups) attn_mfma_direct_kernel<64, 2, 4, 2><<<grid_blocks, 512, 0, s>>>(a);
-        else if (bs % 64 == 0 && hd == 128 && g_direct == 3) attn_mfma_direct_kernel<128, 3><<<grid_blocks, 256, 0, s>>>(a);
-        else if (bs % 64 == 0 && hd == 128 && g_direct) attn_mfma_direct_kernel<128, 2><<<grid_blocks, 256, 0, s>>>(a);
-        else if (bs % 64 == 0 && hd == 64 && g_direct) attn_mfma_direct_kernel<64, 2><<<grid_blocks, 256, 0, s>>>(a);
-        else if (hd <= 32) attn_mfma_block_kernel<32><<<grid_blocks, 256, 0, s>>>(a);
-        else if (hd <= 64) attn_mfma_block_kernel<64><<<grid_blocks, 256, 0, s>>>(a);
-        else if (hd <= 128) attn_mfma_block_kernel<128><<<grid_blocks, 256, 0, s>>>(a);
+        if (tile_q == 128 && hd == 128 && two_groups) attn_mfma_direct_kernel<128, 2, 8, 2><<<grid_blocks, 1024, shm, s>>>(a);
+        else if (tile_q == 128 && hd == 64 && two_groups) attn_mfma_direct_kernel<64, 2, 8, 2><<<grid_blocks, 1024, shm, s>>>(a);
+        else if (tile_q == 128 && hd == 128) attn_mfma_direct_kernel<128, 2, 8><<<grid_blocks, 512, shm, s>>>(a);
+        else if (tile_q == 128) attn_mfma_direct_kernel<64, 2, 8><<<grid_blocks, 512, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 128 && g_direct == 2 && two_groups) attn_mfma_direct_kernel<128, 2, 4, 2><<<grid_blocks, 512, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 64 && g_direct == 2 && two_groups) attn_mfma_direct_kernel<64, 2, 4, 2><<<grid_blocks, 512, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 128 && g_direct == 3) attn_mfma_direct_kernel<128, 3><<<grid_blocks, 256, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 128 && g_direct) attn_mfma_direct_kernel<128, 2><<<grid_blocks, 256, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 64 && g_direct) attn_mfma_direct_kernel<64, 2><<<grid_blocks, 256, shm, s>>>(a);
+        else if (hd <= 32) attn_mfma_block_kernel<32><<<grid_blocks, 256, shm, s>>>(a);
+        else if (hd <= 64) attn_mfma_block_kernel<64><<<grid_blocks, 256, shm, s>>>(a);
+        else if (hd <= 128) attn_mfma_block_kernel<128><<<grid_blocks, 256, shm, s>>>(a);
         else return fx_fail("attn_tiles: no kernel for a head size of %d", hd);
     } else
         attn_tile_kernel<bf16><<<grid, 64, 0, s>>>(a);
@@ -1482,9 +1571,11 @@ static int attn_decode_launch(void* stream, int dtype, const void* q, long ldq, 
                               int nh, int nkv, int hd, int bs, int window, float scale,
                               float* part_o, float* part_ml, int splits, int chunk, int waves, int vd = 0, int mask_chunk = 0,
                               int keep_first = 0, const float* sinks = nullptr, const void* gate = nullptr, long ldg = 0,
-                              float softcap = 0.f, const float* slopes = nullptr, int gate_per_head = 0, const float* turns = nullptr) {
+                              float softcap = 0.f, const float* slopes = nullptr, int gate_per_head = 0, const float* turns = nullptr,
+                           int gate_f32 = 0, const float* bias = nullptr, int bias_n = 0) {
     if (vd <= 0) vd = hd;
     AttnArgs a = {};
+    a.gate_f32 = gate_f32 ? 1 : 0; a.bias = bias; a.bias_n = bias_n;
     a.softcap = softcap; a.slopes = slopes; a.gate_per_head = gate_per_head ? 1 : 0; a.turns = (const float2*)turns;
     a.q = q; a.ldq = ldq; a.out = out; a.ldo = ldo; a.k_pages = k_pages; a.v_pages = v_pages;
     a.block_table = block_table; a.max_blocks = max_blocks; a.positions = positions;
@@ -1552,7 +1643,8 @@ FX_API int fx_attn_decode(void* stream, int dtype, const void* q, long ldq, void
                           int nh, int nkv, int hd, int bs, int window, float scale,
                           float* part_o, float* part_ml, int splits, int chunk, int waves, int vd, int mask_chunk,
                           int keep_first, const float* sinks, const void* gate, long ldg, float softcap, const float* slopes,
-                          int gate_per_head, const float* turns) {
+                          int gate_per_head, const float* turns, int gate_f32, const float* bias, int bias_n) {
+    FX_REQUIRE(!bias || bias_n >= 1, "attn_decode: a distance bias for %d distances", bias_n);
     FX_REQUIRE(!turns || (vd > 0 ? vd : hd) % 2 == 0, "attn_decode: outputs that are turned back come in pairs, a value head has %d", vd > 0 ? vd : hd);
     if (attn_decode_check(dtype, nh, nkv, hd, bs, window, scale, splits, chunk)) return 1;
     FX_REQUIRE(softcap >= 0.f && softcap < INFINITY, "attn_decode: a cap of %g on the scores", (double)softcap);
@@ -1560,7 +1652,8 @@ FX_API int fx_attn_decode(void* stream, int dtype, const void* q, long ldq, void
     if (n_items <= 0) return 0;
     return attn_decode_launch(stream, dtype, q, ldq, out, ldo, k_pages, v_pages, block_table, max_blocks, positions,
                               item_seq, item_tok, n_items, nh, nkv, hd, bs, window, scale, part_o, part_ml, splits,
-                              chunk, waves, vd, mask_chunk, keep_first, sinks, gate, ldg, softcap, slopes, gate_per_head, turns);
+                              chunk, waves, vd, mask_chunk, keep_first, sinks, gate, ldg, softcap, slopes, gate_per_head, turns,
+                              gate_f32, bias, bias_n);
 }
 
 // ---------------------------------------------------------------------------

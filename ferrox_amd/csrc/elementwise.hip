@@ -858,6 +858,76 @@ FX_API int fx_gated_add_layernorm(void* stream, int out_dtype, float* h, const f
 }
 
 // ---------------------------------------------------------------------------
+// A sublayer's float32 output rows y, layer-normed as they join the residual stream:
+//   h[t] += (y[t] - mean) / sqrt(var + eps) * w + b      (b may be null; var the mean of the squared deviations)
+// and, with `out`, the new rows of h once more in the type that the next sublayer's products read.  Rows of up to
+// 4,096 columns stay in registers; longer ones are read again.  One block per row.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void layernorm_add_kernel(float* __restrict__ h, const float* __restrict__ y,
+                                                            const void* __restrict__ w, const void* __restrict__ b, int w_dtype,
+                                                            T* __restrict__ out, int H, float eps) {
+    __shared__ float red[4];
+    const size_t row = (size_t)blockIdx.x * H;
+    if (H <= 256 * 16) {
+        float yv[16], hv[16], wv[16], bv[16];
+        float sum = 0.f;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) yv[i] = y[row + min((int)threadIdx.x + i * 256, H - 1)];
+#pragma unroll
+        for (int i = 0; i < 16; ++i) hv[i] = h[row + min((int)threadIdx.x + i * 256, H - 1)];
+        load_strided_as_float<16, 256>(w, w_dtype, threadIdx.x, H, wv);
+        if (b) load_strided_as_float<16, 256>(b, w_dtype, threadIdx.x, H, bv);
+#pragma unroll
+        for (int i = 0; i < 16; ++i) sum += (int)threadIdx.x + i * 256 < H ? yv[i] : 0.f;
+        const float mean = block_sum<4>(sum, red) / (float)H;
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const float d = (int)threadIdx.x + i * 256 < H ? yv[i] - mean : 0.f;
+            ss = fmaf(d, d, ss);
+        }
+        const float rstd = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)H + eps);
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int c = threadIdx.x + i * 256;
+            if (c >= H) continue;
+            const float v = hv[i] + ((yv[i] - mean) * rstd * wv[i] + (b ? bv[i] : 0.f));
+            h[row + c] = v;
+            if (out) from_float(out + row + c, v);
+        }
+        return;
+    }
+    float sum = 0.f;
+    for (int c = threadIdx.x; c < H; c += 256) sum += y[row + c];
+    const float mean = block_sum<4>(sum, red) / (float)H;
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < H; c += 256) {
+        const float d = y[row + c] - mean;
+        ss = fmaf(d, d, ss);
+    }
+    const float rstd = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)H + eps);
+    for (int c = threadIdx.x; c < H; c += 256) {
+        const float v = h[row + c] + ((y[row + c] - mean) * rstd * load_as_float(w, w_dtype, c) + (b ? load_as_float(b, w_dtype, c) : 0.f));
+        h[row + c] = v;
+        if (out) from_float(out + row + c, v);
+    }
+}
+
+FX_API int fx_layernorm_add(void* stream, int out_dtype, float* h, const float* y, const void* w, const void* b, int w_dtype,
+                            void* out, int T, int H, float eps) {
+    FX_REQUIRE(T >= 0 && H > 0 && w, "layernorm_add: bad sizes T=%d H=%d", T, H);
+    FX_REQUIRE(w_dtype == FX_F32 || w_dtype == FX_BF16, "layernorm_add: unknown weight dtype %d", w_dtype);
+    if (T == 0) return 0;
+    hipStream_t s = (hipStream_t)stream;
+    if (!out || out_dtype == FX_F32) layernorm_add_kernel<float><<<T, 256, 0, s>>>(h, y, w, b, w_dtype, (float*)out, H, eps);
+    else if (out_dtype == FX_BF16) layernorm_add_kernel<bf16><<<T, 256, 0, s>>>(h, y, w, b, w_dtype, (bf16*)out, H, eps);
+    else return fx_fail("layernorm_add: unknown output dtype %d", out_dtype);
+    FX_CHECK_LAUNCH("layernorm_add");
+    return 0;
+}
+
+// ---------------------------------------------------------------------------
 // Latent attention, what a layer keeps per position.  `down` [T, R + rd] float32 is the down-projection of a
 // token: R latent channels, then a key part of rd dimensions that all heads share.  One block per token:
 //   c = down[:R] / sqrt(mean(down[:R]^2) + eps) * w          (statistics and product in float32)
@@ -869,7 +939,10 @@ FX_API int fx_gated_add_layernorm(void* stream, int out_dtype, float* h, const f
 // up-projection is applied to afterwards.
 // With `q_src` (the queries' down-projection of the same tokens, [T, Rq] float32, usually the columns beside `down` in
 // one product's output) a second row of blocks norms that latent too, q_out[t] = q_src[t] / rms * q_w in the pages'
-// type: the two norms that follow the down-projection are one launch.
+// type: the two norms that follow the down-projection are one launch.  Without a norm weight `q_src` holds the queries
+// themselves, nh heads of (R | rd) a token (their unrotated part already taken through the keys' up-projection): their
+// rotated parts are turned as the key part is, in float32, and the heads rounded once into q_out; blocks
+// (token, 1 ..) share the heads.
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void latent_kv_write_kernel(
@@ -877,9 +950,48 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
     const int* __restrict__ positions, const int* __restrict__ token_seq, const int* __restrict__ block_table, int max_blocks,
     T* __restrict__ k_pages, T* __restrict__ v_pages, int R, int rd, int rot, int bs, const float* __restrict__ inv_freq,
     float magnitude, const float* __restrict__ q_src, long ldqs, const void* __restrict__ q_w, float q_eps,
-    T* __restrict__ q_out, long ldq, int Rq) {
+    T* __restrict__ q_out, long ldq, int Rq, int q_heads) {
     __shared__ float red[4];
     const int t = blockIdx.x, tid = threadIdx.x;
+    if (blockIdx.y >= 1 && q_heads > 0) {          // the queries' heads
+        __shared__ float cs[256], sn[256];
+        const int half = rot >> 1, width = R + rd;
+        for (int p = tid; p < half; p += 256) {
+            float s_, c_;
+            sincosf((float)positions[t] * inv_freq[p], &s_, &c_);
+            cs[p] = c_ * magnitude;
+            sn[p] = s_ * magnitude;
+        }
+        const int share = (q_heads + gridDim.y - 2) / (gridDim.y - 1);
+        const int h0 = (blockIdx.y - 1) * share, n = min(share, q_heads - h0) * width;
+        const float* src = q_src + (size_t)t * ldqs + (size_t)h0 * width;
+        T* dst = q_out + (size_t)t * ldq + (size_t)h0 * width;
+        __syncthreads();
+        if (((R | rd) & 1) == 0 && (ldqs & 1) == 0 && ((uintptr_t)src & 7) == 0) {      // pairs of columns, rotated or not
+#pragma unroll 4
+            for (int i = 2 * tid; i < n; i += 512) {
+                const int c = i % width - R;
+                const float2 x = *(const float2*)(src + i);
+                float y0 = x.x, y1 = x.y;
+                if (c >= 0 && c < rot) rotate_pair(x.x, x.y, cs[c >> 1], sn[c >> 1], y0, y1);
+                from_float(dst + i, y0);
+                from_float(dst + i + 1, y1);
+            }
+            return;
+        }
+        for (int i = tid; i < n; i += 256) {
+            const int c = i % width - R;
+            float y = src[i];
+            if (c >= 0 && c < rot) {
+                float y0, y1;
+                if (c & 1) rotate_pair(src[i - 1], y, cs[c >> 1], sn[c >> 1], y0, y1);
+                else rotate_pair(y, src[i + 1], cs[c >> 1], sn[c >> 1], y0, y1);
+                y = (c & 1) ? y1 : y0;
+            }
+            from_float(dst + i, y);
+        }
+        return;
+    }
     if (blockIdx.y == 1) {          // the queries' latent
         const float* xq = q_src + (size_t)t * ldqs;
         float sq = 0.f;
@@ -919,24 +1031,28 @@ FX_API int fx_latent_kv_write(void* stream, int dtype, const float* down, long l
                               const int* positions, const int* token_seq, const int* block_table, int max_blocks,
                               void* k_pages, void* v_pages, int T, int R, int rd, int rot, int bs, const float* inv_freq,
                               float magnitude, const float* q_src, long ldqs, const void* q_w, float q_eps, void* q_out,
-                              long ldq, int Rq) {
+                              long ldq, int Rq, int q_heads) {
     FX_REQUIRE(T >= 0 && R > 0 && rd >= 0 && bs > 0 && ldd >= R + rd, "latent_kv_write: bad sizes T=%d R=%d rd=%d", T, R, rd);
     FX_REQUIRE(rot >= 0 && rot <= rd && rot % 2 == 0, "latent_kv_write: %d rotated dimensions of %d", rot, rd);
     FX_REQUIRE(inv_freq || rot == 0, "latent_kv_write: a rotation needs the table of its %d frequencies", rot / 2);
     FX_REQUIRE(w_dtype == FX_F32 || w_dtype == FX_BF16, "latent_kv_write: unknown weight dtype %d", w_dtype);
     FX_REQUIRE(k_pages && v_pages && w, "latent_kv_write: pages and the norm's weight are needed");
-    FX_REQUIRE(!q_src || (q_w && q_out && Rq > 0 && ldqs >= Rq && ldq >= Rq), "latent_kv_write: the queries' latent needs a weight, an output and %d columns", Rq);
+    FX_REQUIRE(!q_src || (q_out && Rq > 0 && ldqs >= Rq && ldq >= Rq && (q_w != nullptr) == (q_heads == 0)),
+               "latent_kv_write: the queries' latent needs a weight, an output and %d columns", Rq);
+    FX_REQUIRE(q_heads >= 0 && (q_heads == 0 || (q_src && (long)q_heads * (R + rd) == Rq && rot <= 512)),
+               "latent_kv_write: %d query heads of %d columns in rows of %d", q_heads, R + rd, Rq);
     if (T == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    const dim3 grid(T, q_src ? 2 : 1);
+    // few tokens: a token's query heads are shared between blocks
+    const dim3 grid(T, !q_src ? 1 : (q_heads == 0 || T > 256 ? 2 : 1 + (q_heads < 8 ? q_heads : 8)));
     if (dtype == FX_F32)
         latent_kv_write_kernel<float><<<grid, 256, 0, s>>>(down, ldd, w, w_dtype, eps, positions, token_seq, block_table, max_blocks,
                                                            (float*)k_pages, (float*)v_pages, R, rd, rot, bs, inv_freq, magnitude,
-                                                           q_src, ldqs, q_w, q_eps, (float*)q_out, ldq, Rq);
+                                                           q_src, ldqs, q_w, q_eps, (float*)q_out, ldq, Rq, q_heads);
     else if (dtype == FX_BF16)
         latent_kv_write_kernel<bf16><<<grid, 256, 0, s>>>(down, ldd, w, w_dtype, eps, positions, token_seq, block_table, max_blocks,
                                                           (bf16*)k_pages, (bf16*)v_pages, R, rd, rot, bs, inv_freq, magnitude,
-                                                          q_src, ldqs, q_w, q_eps, (bf16*)q_out, ldq, Rq);
+                                                          q_src, ldqs, q_w, q_eps, (bf16*)q_out, ldq, Rq, q_heads);
     else
         return fx_fail("latent_kv_write: unknown dtype %d", dtype);
     FX_CHECK_LAUNCH("latent_kv_write");
@@ -998,19 +1114,19 @@ FX_API int fx_latent_q_rot(void* stream, int dtype, const void* q, long ldq, voi
 }
 
 // ---------------------------------------------------------------------------
-// Queries and keys normed over their whole projection, keys that are their own values.  From the float32 product
-// qk [T, nh * hd + nkv * hd] (a token's queries, then its keys), one launch writes
+// Queries and keys normed over their whole projection.  From the float32 product qk [T, nh * hd + nkv * hd] (a token's
+// queries, then its keys; with vd > 0 then its values, nkv heads of vd), one launch writes
 //   q_out [T, nh * hd]: the queries normed over all nh * hd columns, x / sqrt(mean + eps) * wq[column]
 //   the key page: the keys normed over all nkv * hd columns with wk
-//   the transposed value page: the keys as they are, not normed
-// Blocks (token, 0) take the queries, blocks (token, 1) the keys (left out when there are no pages to write).
+//   the transposed value page: the values or, with vd = 0, the keys as they are, not normed
+// Blocks (token, 0) take the queries, blocks (token, 1) the keys and values (left out when there are no pages to write).
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void span_norm_kv_write_kernel(
     const float* __restrict__ qk, long ldqk, T* __restrict__ q_out, long ldq, const void* __restrict__ wq,
     const void* __restrict__ wk, int w_dtype, float eps,
     const int* __restrict__ positions, const int* __restrict__ token_seq, const int* __restrict__ block_table, int max_blocks,
-    T* __restrict__ k_pages, T* __restrict__ v_pages, int nh, int nkv, int hd, int bs) {
+    T* __restrict__ k_pages, T* __restrict__ v_pages, int nh, int nkv, int hd, int bs, int vd) {
     __shared__ float red[4];
     const int t = blockIdx.x, tid = threadIdx.x;
     const bool keys = blockIdx.y == 1;
@@ -1030,16 +1146,18 @@ __global__ __launch_bounds__(256) void span_norm_kv_write_kernel(
     for (int c = tid; c < n; c += 256) {
         const int g = c / hd, d = c - g * hd;
         from_float(k_pages + (((size_t)page * nkv + g) * bs + slot) * hd + d, x[c] * scale * load_as_float(w, w_dtype, c));
-        from_float(v_pages + (((size_t)page * nkv + g) * hd + d) * bs + slot, x[c]);
+        if (vd == 0) from_float(v_pages + (((size_t)page * nkv + g) * hd + d) * bs + slot, x[c]);
     }
+    // (a page's value rows of the kv heads follow each other: channel c of all heads is row c)
+    for (int c = tid; c < nkv * vd; c += 256) from_float(v_pages + ((size_t)page * nkv * vd + c) * bs + slot, x[n + c]);
 }
 
 FX_API int fx_span_norm_kv_write(void* stream, int dtype, const float* qk, long ldqk, void* q_out, long ldq, const void* wq,
                                  const void* wk, int w_dtype, float eps, const int* positions, const int* token_seq,
                                  const int* block_table, int max_blocks, void* k_pages, void* v_pages, int T, int nh, int nkv,
-                                 int hd, int bs) {
-    FX_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && hd > 0 && bs > 0, "span_norm_kv_write: bad sizes");
-    FX_REQUIRE(ldq >= (long)nh * hd && ldqk >= (long)(nh + (k_pages ? nkv : 0)) * hd, "span_norm_kv_write: rows shorter than their heads");
+                                 int hd, int bs, int vd) {
+    FX_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && hd > 0 && bs > 0 && vd >= 0, "span_norm_kv_write: bad sizes");
+    FX_REQUIRE(ldq >= (long)nh * hd && ldqk >= (long)(nh + (k_pages ? nkv : 0)) * hd + (k_pages ? (long)nkv * vd : 0), "span_norm_kv_write: rows shorter than their heads");
     FX_REQUIRE(w_dtype == FX_F32 || w_dtype == FX_BF16, "span_norm_kv_write: unknown weight dtype %d", w_dtype);
     FX_REQUIRE((k_pages == nullptr) == (v_pages == nullptr), "span_norm_kv_write: key and value pages must come together");
     FX_REQUIRE(wq && (wk || !k_pages), "span_norm_kv_write: the norms' weights are needed");
@@ -1048,10 +1166,10 @@ FX_API int fx_span_norm_kv_write(void* stream, int dtype, const float* qk, long 
     const dim3 grid(T, k_pages ? 2 : 1);
     if (dtype == FX_F32)
         span_norm_kv_write_kernel<float><<<grid, 256, 0, s>>>(qk, ldqk, (float*)q_out, ldq, wq, wk, w_dtype, eps, positions, token_seq,
-                                                              block_table, max_blocks, (float*)k_pages, (float*)v_pages, nh, nkv, hd, bs);
+                                                              block_table, max_blocks, (float*)k_pages, (float*)v_pages, nh, nkv, hd, bs, vd);
     else if (dtype == FX_BF16)
         span_norm_kv_write_kernel<bf16><<<grid, 256, 0, s>>>(qk, ldqk, (bf16*)q_out, ldq, wq, wk, w_dtype, eps, positions, token_seq,
-                                                             block_table, max_blocks, (bf16*)k_pages, (bf16*)v_pages, nh, nkv, hd, bs);
+                                                             block_table, max_blocks, (bf16*)k_pages, (bf16*)v_pages, nh, nkv, hd, bs, vd);
     else
         return fx_fail("span_norm_kv_write: unknown dtype %d", dtype);
     FX_CHECK_LAUNCH("span_norm_kv_write");

@@ -68,6 +68,9 @@ struct GemmArgs {
     const float* pre_scale;       // EPI_GATED: [.] or null: gate and up of logical row m are multiplied by
     const int* pre_scale_rows;    //   pre_scale[pre_scale_rows ? pre_scale_rows[m] : m] before the activation (a row of A scaled)
     int store_act;   // EPI_STORE: what the product goes through before it is stored (SACT_*), 0 for nothing
+    const float* out_gate;   // SACT_GATE: gate logits; row m of C belongs to row m / gate_div of it and to its columns
+    long ld_gate;            //   (m % gate_div) * N + n
+    int gate_div;
     int vec_ok;  // 16-byte loads are legal for A and W
     int n_col_tiles, n_row_tiles;  // tiled kernels: the grid they decode block ids with
 };
@@ -200,9 +203,19 @@ __device__ __forceinline__ float gated_c(float gate, float up, float limit, floa
 // down(act(up x)).  Uniform over the launch; SACT_NONE costs one scalar compare per element.
 //   SACT_RELU2    max(x, 0)^2
 //   SACT_SOFTCAP  limit * tanh(x / limit)      (logits kept within +-limit)
-enum { SACT_NONE = 0, SACT_RELU2 = 1, SACT_RELU = 2, SACT_SILU = 3, SACT_GELU_TANH = 4, SACT_SOFTCAP = 5, SACT_COUNT = 6 };
-__device__ __forceinline__ float stored_f(int act, float x, float limit) {
+//   SACT_GATE     x * sigmoid(gate), gate a float32 matrix of the output's elements (`out_gate`)
+enum { SACT_NONE = 0, SACT_RELU2 = 1, SACT_RELU = 2, SACT_SILU = 3, SACT_GELU_TANH = 4, SACT_SOFTCAP = 5, SACT_GATE = 6, SACT_COUNT = 7 };
+// the gate logit of output element (m, n); 0 without a gate
+__device__ __forceinline__ float gate_of(const GemmArgs& g, int m, int n) {
+    if (!g.out_gate) return 0.f;
+    const int row = m / g.gate_div;
+    return g.out_gate[(size_t)row * g.ld_gate + (size_t)(m - row * g.gate_div) * g.N + n];
+}
+__device__ __forceinline__ float stored_f(const GemmArgs& g, float x, float gate) {
+    const int act = g.store_act;
+    const float limit = g.act_limit;
     if (act == SACT_NONE) return x;
+    if (act == SACT_GATE) return x / (1.0f + expf(-gate));
     if (act == SACT_RELU2) {
         const float r = fmaxf(x, 0.0f);
         return r * r;
@@ -212,12 +225,25 @@ __device__ __forceinline__ float stored_f(int act, float x, float limit) {
     if (act == SACT_SOFTCAP) return limit * tanhf(x / limit);
     return 0.5f * x * (1.0f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
 }
-// f(whether outputs are stored as they are, as a compile-time constant): the tiled epilogues call this once around their
-// loops (with every activation inside the loops of a plain product's epilogue those were 10-16 % of the q/k/v product)
+// f(what happens to an output on its way out, as a compile-time constant; SACT_COUNT: one of the rarer activations, looked
+// up per element): the tiled epilogues call this once around their loops (with every activation inside the loops of a
+// plain product's epilogue those were 10-16 % of the q/k/v product)
 template <bool STORES, typename F>
-__device__ __forceinline__ void with_plain_stores(int act, F&& f) {
-    if (!STORES || act == SACT_NONE) f(std::true_type{});
-    else f(std::false_type{});
+__device__ __forceinline__ void with_stored(int act, F&& f) {
+    if (!STORES || act == SACT_NONE) f(std::integral_constant<int, SACT_NONE>{});
+    else if (act == SACT_RELU2) f(std::integral_constant<int, SACT_RELU2>{});
+    else if (act == SACT_GATE) f(std::integral_constant<int, SACT_GATE>{});
+    else f(std::integral_constant<int, SACT_COUNT>{});
+}
+template <int ACT>
+__device__ __forceinline__ float stored_c(const GemmArgs& g, float x, float gate) {
+    if constexpr (ACT == SACT_NONE) return x;
+    if constexpr (ACT == SACT_GATE) return x / (1.0f + expf(-gate));
+    if constexpr (ACT == SACT_RELU2) {
+        const float r = fmaxf(x, 0.0f);
+        return r * r;
+    }
+    return stored_f(g, x, gate);
 }
 // what gate and up of logical row m are multiplied by before the activation (1 without a pre-scale)
 #define FX_PRE_SCALE(g, ml) ((g).pre_scale ? (g).pre_scale[(g).pre_scale_rows ? (g).pre_scale_rows[ml] : (ml)] : 1.0f)
@@ -392,7 +418,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs g) {
         });
         return;
     }
-    with_plain_stores<EPI == EPI_STORE || EPI == EPI_STORE_F32>(g.store_act, [&](auto plain) {
+    with_stored<EPI == EPI_STORE || EPI == EPI_STORE_F32>(g.store_act, [&](auto kind) {
 #pragma unroll
     for (int i = 0; i < MT; ++i) {
 #pragma unroll
@@ -408,9 +434,9 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmArgs g) {
                     float v = acc[i][j][r];
                     if (g.bias) v += bias_v[j];
                     if (EPI == EPI_STORE) {
-                        from_float((bf16*)g.C + (size_t)m * g.ldc + n, decltype(plain)::value ? v : stored_f(g.store_act, v, g.act_limit));
+                        from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_c<decltype(kind)::value>(g, v, decltype(kind)::value == SACT_GATE ? gate_of(g, m, n) : 0.f));
                     } else if (EPI == EPI_STORE_F32) {
-                        ((float*)g.C)[(size_t)m * g.ldc + n] = decltype(plain)::value ? v : stored_f(g.store_act, v, g.act_limit);
+                        ((float*)g.C)[(size_t)m * g.ldc + n] = stored_c<decltype(kind)::value>(g, v, decltype(kind)::value == SACT_GATE ? gate_of(g, m, n) : 0.f);
                     } else {
                         if (g.row_scale) v *= g.row_scale[ml];
                         ((float*)g.C)[(size_t)m * g.ldc + n] += v;
@@ -649,10 +675,16 @@ __global__ __launch_bounds__(512) void gemm_bf16_wide_kernel(GemmArgs g) {
         });
         return;
     }
-    with_plain_stores<EPI == EPI_STORE || EPI == EPI_STORE_F32>(g.store_act, [&](auto plain) {
+    with_stored<EPI == EPI_STORE || EPI == EPI_STORE_F32>(g.store_act, [&](auto kind) {
 #pragma unroll
     for (int i = 0; i < MT; ++i) {
-        float old[4][NT];
+        float old[4][NT], gates[4][NT] = {};      // (the gates' logits of a row block, fetched together)
+        if (decltype(kind)::value == SACT_GATE) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+#pragma unroll
+                for (int j = 0; j < NT; ++j) gates[r][j] = gate_of(g, m_of[i][r], min(n0 + wn * WN + j * 16 + (lane & 15), g.N - 1));
+        }
         if (EPI == EPI_RESID) {
 #pragma unroll
             for (int r = 0; r < 4; ++r)
@@ -675,9 +707,9 @@ __global__ __launch_bounds__(512) void gemm_bf16_wide_kernel(GemmArgs g) {
                     float v = acc[i][j][r];
                     if (g.bias) v += bias_v[j];
                     if (EPI == EPI_STORE) {
-                        from_float((bf16*)g.C + (size_t)m * g.ldc + n, decltype(plain)::value ? v : stored_f(g.store_act, v, g.act_limit));
+                        from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_c<decltype(kind)::value>(g, v, gates[r][j]));
                     } else if (EPI == EPI_STORE_F32) {
-                        ((float*)g.C)[(size_t)m * g.ldc + n] = decltype(plain)::value ? v : stored_f(g.store_act, v, g.act_limit);
+                        ((float*)g.C)[(size_t)m * g.ldc + n] = stored_c<decltype(kind)::value>(g, v, gates[r][j]);
                     } else {
                         if (g.row_scale) {
                             v *= scale_of[i][r];
@@ -1109,6 +1141,11 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(GemmArgs g
                     old[r] = ((const float*)g.C)[(size_t)m * g.ldc + min(n0 + a * 16 + (L >> 4) * 4 + r, g.N - 1)];
             }
         }
+        float gates[4] = {0.f, 0.f, 0.f, 0.f};
+        if ((EPI == EPI_STORE || EPI == EPI_STORE_F32) && g.out_gate) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) gates[r] = gate_of(g, m, min(n0 + a * 16 + (L >> 4) * 4 + r, g.N - 1));
+        }
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int n = n0 + a * 16 + (L >> 4) * 4 + r;
@@ -1122,9 +1159,9 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(GemmArgs g
             }
             if (g.bias) o += bias_v[r];
             if (EPI == EPI_STORE) {
-                from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_f(g.store_act, o, g.act_limit));
+                from_float((bf16*)g.C + (size_t)m * g.ldc + n, stored_f(g, o, gates[r]));
             } else if (EPI == EPI_STORE_F32) {
-                ((float*)g.C)[(size_t)m * g.ldc + n] = stored_f(g.store_act, o, g.act_limit);
+                ((float*)g.C)[(size_t)m * g.ldc + n] = stored_f(g, o, gates[r]);
             } else {
                 if (g.row_scale) {
                     o *= row_scale;
@@ -1221,7 +1258,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmArgs g) {
                     if (g.row_scale) v *= g.row_scale[ml];
                     *out += v;
                 } else {
-                    *out = stored_f(g.store_act, v, g.act_limit);      // (the host sets store_act for stored products only)
+                    *out = stored_f(g, v, gate_of(g, m, n));      // (the host sets store_act for stored products only)
                 }
             }
         }
@@ -1408,7 +1445,9 @@ FX_API int fx_gemm(void* stream, int dtype, int epi, const void* A, long lda, co
                    int E, int M, int N, int K, const void* norm_w, int norm_dtype, float norm_eps,
                    const int* pair_ids, int pair_div, int n_always, int always_rows, int always_from_a, long kb_rows,
                    const float* row_ss, int row_ss_n, int act, int store_act, float act_limit, float act_alpha,
-                   const float* pre_scale, const int* pre_scale_rows) {
+                   const float* pre_scale, const int* pre_scale_rows, const float* out_gate, long ld_gate, int gate_div) {
+    FX_REQUIRE((store_act == SACT_GATE) == (out_gate != nullptr) && (!out_gate || (gate_div >= 1 && ld_gate >= (long)gate_div * N)),
+               "gemm: gated outputs need gate rows of %d x %d columns, got a row distance of %ld", gate_div, N, ld_gate);
     FX_REQUIRE(store_act >= 0 && store_act < SACT_COUNT && (store_act == 0 || ((epi == EPI_STORE || epi == EPI_STORE_F32) && !bias)),
                "gemm: a stored activation (%d) goes with the plain stored product without bias", store_act);
     FX_REQUIRE(!pre_scale || epi == EPI_GATED, "gemm: a scale in front of the activation goes with the gate/up epilogue");
@@ -1444,6 +1483,7 @@ FX_API int fx_gemm(void* stream, int dtype, int epi, const void* A, long lda, co
     g.a_rows = a_rows; g.c_rows = c_rows; g.expert_offsets = expert_offsets; g.E = E; g.M = M; g.N = N; g.K = K;
     g.pair_ids = pair_ids; g.pair_div = pair_div; g.act = act; g.store_act = store_act;
     g.act_limit = act_limit; g.act_alpha = act_alpha; g.pre_scale = pre_scale; g.pre_scale_rows = pre_scale_rows;
+    g.out_gate = out_gate; g.ld_gate = ld_gate; g.gate_div = gate_div;
     g.kb_stride = kb_rows * 64;
     FX_REQUIRE(kb_rows >= 0 && (kb_rows == 0 || (dtype == FX_BF16 && K % 64 == 0 && ((uintptr_t)W % 16) == 0 && lda % 8 == 0 &&
                                                  ((uintptr_t)A % 16) == 0 && (up_offset % K) == 0)),

@@ -95,6 +95,9 @@ def _register_builtin():
     from ..config.besulix import BesulixConfig
     from .besulix import build_spec as besulix_spec
     register_architecture(Architecture(BesulixConfig.architecture, BesulixConfig.model_type, BesulixConfig, besulix_spec))
+    from ..config.zazerax import ZazeraxConfig
+    from .zazerax import build_spec as zazerax_spec
+    register_architecture(Architecture(ZazeraxConfig.architecture, ZazeraxConfig.model_type, ZazeraxConfig, zazerax_spec))
 
 
 _register_builtin()

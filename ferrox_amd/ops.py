@@ -22,6 +22,7 @@ ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "gelu": 2, "relu": 3, "swiglu_clamped"
 # what a stored product (EPI_STORE) may go through on its way out, the activation of a feed-forward without a
 # gate; SACT_* in csrc/gemm.hip
 STORED_ACTIVATIONS = {None: 0, "relu2": 1, "relu": 2, "silu": 3, "gelu_tanh": 4, "softcap": 5}
+_SACT_GATE = 6       # (set by gemm's `out_gate`)
 GATE_SOFTMAX, GATE_SIGMOID = 0, 1
 ROPE_NEOX, ROPE_INTERLEAVED = 0, 1
 
@@ -74,12 +75,13 @@ _sigs = {
                                                c_float, c_int, c_int, c_float],
     ("elementwise", "fx_latent_kv_write"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_float, c_void_p, c_void_p,
                                             c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p,
-                                            c_float, c_void_p, c_long, c_void_p, c_float, c_void_p, c_long, c_int],
+                                            c_float, c_void_p, c_long, c_void_p, c_float, c_void_p, c_long, c_int, c_int],
     ("elementwise", "fx_latent_q_rot"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_int, c_int,
                                          c_int, c_int, c_int, c_void_p, c_float],
     ("elementwise", "fx_span_norm_kv_write"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_int,
                                                c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int,
-                                               c_int, c_int, c_int],
+                                               c_int, c_int, c_int, c_int],
+    ("elementwise", "fx_layernorm_add"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float],
     ("elementwise", "fx_rmsnorm"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float, c_long],
     ("elementwise", "fx_rope_kv_write"): [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int,
                                           c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
@@ -127,20 +129,20 @@ _sigs = {
     ("gemm", "fx_gemm"): [c_void_p, c_int, c_int, c_void_p, c_long, c_void_p, c_long, c_long, c_void_p, c_int,
                           c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                           c_void_p, c_int, c_float, c_void_p, c_int, c_int, c_int, c_int, c_long, c_void_p, c_int, c_int, c_int,
-                          c_float, c_float, c_void_p, c_void_p],
+                          c_float, c_float, c_void_p, c_void_p, c_void_p, c_long, c_int],
     ("gemm", "fx_qkv_rope"): [c_void_p, c_void_p, c_long, c_void_p, c_long, c_void_p, c_int, c_void_p, c_long, c_int, c_int,
                               c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                               c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p],
     ("attention", "fx_attn_tiles"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p,
                                      c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                                      c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int,
-                                     c_int, c_void_p, c_void_p, c_long, c_float, c_void_p, c_int, c_void_p],
+                                     c_int, c_void_p, c_void_p, c_long, c_float, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int],
     ("attention", "fx_attn_tile_queries"): [c_int, c_int, c_int],
     ("attention", "fx_attn_decode"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p,
                                       c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                       c_int, c_int, c_int, c_int, c_int, c_float,
                                       c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
-                                      c_int, c_void_p, c_void_p, c_long, c_float, c_void_p, c_int, c_void_p],
+                                      c_int, c_void_p, c_void_p, c_long, c_float, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int],
     ("moe", "fx_router_select"): [c_void_p, c_void_p, c_long, c_long, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
                                   c_void_p, c_void_p, c_void_p, c_void_p],
     ("moe", "fx_router_select_align"): [c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
@@ -253,6 +255,24 @@ def gated_add_layernorm(h: torch.Tensor, y: torch.Tensor, gate_logits: torch.Ten
     _call("elementwise", "fx_gated_add_layernorm", _stream(), dtype_code(out_dtype), _p(h), _p(y), _p(gate_logits), _p(weight),
           _p(bias), dtype_code(weight.dtype), _p(out), T, H, float(eps))
     return out
+
+
+def layernorm_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, eps: float,
+                  rows_dtype: torch.dtype | None = None):
+    """h[t] += (y[t] - mean) / sqrt(var + eps) * weight + bias: float32 rows of a sublayer's output, layer-normed as they
+    join the stream.  With `rows_dtype` the new rows of h are returned in that type (h itself where it is float32), made
+    by the same launch."""
+    for t in (h, y):
+        if t.dtype != torch.float32 or not t.is_contiguous() or t.shape != h.shape or t.dim() != 2:
+            raise KernelError("layernorm_add wants contiguous float32 matrices of one shape")
+    T, H = h.shape
+    if weight.numel() != H or not weight.is_contiguous() or (bias is not None and (bias.numel() != H or bias.dtype != weight.dtype
+                                                                                     or not bias.is_contiguous())):
+        raise KernelError(f"layernorm_add: weight and bias must hold {H} elements of one type")
+    out = torch.empty((T, H), dtype=rows_dtype, device=h.device) if rows_dtype not in (None, torch.float32) else None
+    _call("elementwise", "fx_layernorm_add", _stream(), dtype_code(rows_dtype or torch.float32), _p(h), _p(y), _p(weight), _p(bias),
+          dtype_code(weight.dtype), _p(out), T, H, float(eps))
+    return h if rows_dtype == torch.float32 else out
 
 
 def temp_unit_kv_write(qkv, q_out, positions, token_seq, block_table, k_pages, v_pages, n_heads: int, n_kv_heads: int,
@@ -403,14 +423,16 @@ def head_norm_kv_write(qk, q_out, v, q_weight, k_weight, eps, positions, token_s
 
 
 def latent_kv_write(down, weight, eps, positions, token_seq, block_table, k_pages, v_pages, kv_rank: int, rot_dim: int,
-                    rotary_dim: int, block_size: int, inv_freq, magnitude: float = 1.0, q_latent=None):
+                    rotary_dim: int, block_size: int, inv_freq, magnitude: float = 1.0, q_latent=None, q_heads=None):
     """What a latent-attention layer keeps per position, from the float32 down-projection `down` [T, kv_rank +
     rot_dim]: the first kv_rank columns through an RMS norm with `weight` (the latent c), the last rot_dim with the
     pairs (2i, 2i+1), i < rotary_dim / 2, turned by pos * inv_freq[i] and stretched by `magnitude`.  The key page
     [pages, 1, block_size, kv_rank + rot_dim] receives (c | rotated part), the value page [pages, 1, kv_rank,
     block_size] c transposed.  `q_latent` = (rows, weight, eps): the same launch also norms the queries' latent, float32
     `rows` [T, q_rank] (any row distance, unit inner stride) with a weight of the keys' norm's type, and returns it
-    [T, q_rank] in the pages' type (None without `q_latent`)."""
+    [T, q_rank] in the pages' type (None without `q_latent`).  `q_heads` = (rows, n) instead: float32 `rows` [T, n *
+    (kv_rank + rot_dim)] hold the queries themselves, n heads of (part that went through the keys' up-projection | part
+    to rotate); the same launch turns the latter like the shared key part and returns the heads in the pages' type."""
     T = down.shape[0]
     R, rd = int(kv_rank), int(rot_dim)
     _f32_rows(down, "latent_kv_write: the down-projection", R + rd)
@@ -433,11 +455,21 @@ def latent_kv_write(down, weight, eps, positions, token_seq, block_table, k_page
                 or q_w.dtype != weight.dtype or not q_w.is_contiguous() or Rq < 1:
             raise KernelError(f"latent_kv_write: the queries' latent {tuple(q_rows.shape)} with a weight of {Rq} ({q_w.dtype})")
         q_out = torch.empty((T, Rq), dtype=k_pages.dtype, device=k_pages.device)
+    n_q = 0
+    if q_heads is not None:
+        q_rows, n_q = q_heads
+        Rq = int(n_q) * (R + rd)
+        if q_latent is not None or n_q < 1:
+            raise KernelError("latent_kv_write: the queries come as a latent or as heads")
+        _f32_rows(q_rows, "latent_kv_write: the queries' heads", Rq)
+        if q_rows.shape[0] < T:
+            raise KernelError(f"latent_kv_write: {q_rows.shape[0]} rows of queries for {T} tokens")
+        q_out = torch.empty((T, Rq), dtype=k_pages.dtype, device=k_pages.device)
     _call("elementwise", "fx_latent_kv_write", _stream(), dtype_code(k_pages.dtype), _p(down), down.stride(0), _p(weight),
           dtype_code(weight.dtype), float(eps), _p(_i32(positions, "positions")), _p(_i32(token_seq, "token_seq")),
           _p(_i32(block_table, "block_table")), block_table.shape[1], _p(k_pages), _p(v_pages), T, R, rd, int(rotary_dim),
           int(block_size), _p(inv_freq), float(magnitude), _p(q_rows), q_rows.stride(0) if q_rows is not None else 0, _p(q_w),
-          float(q_eps), _p(q_out), q_out.stride(0) if q_out is not None else 0, int(Rq))
+          float(q_eps), _p(q_out), q_out.stride(0) if q_out is not None else 0, int(Rq), int(n_q))
     return q_out
 
 
@@ -460,16 +492,18 @@ def latent_q_rot(q, q_lat, positions, n_heads: int, dim: int, rot_dim: int, rota
 
 
 def span_norm_kv_write(qk, q_out, q_weight, k_weight, eps, positions, token_seq, block_table, k_pages, v_pages,
-                       n_heads: int, n_kv_heads: int, head_dim: int, block_size: int) -> None:
-    """Queries and keys normed over their whole projection, keys that are their own values, in one launch: from the
-    float32 product qk [T, (n_heads + n_kv_heads) * head_dim], the queries go, normed over all their columns with
+                       n_heads: int, n_kv_heads: int, head_dim: int, block_size: int, v_dim: int = 0) -> None:
+    """Queries and keys normed over their whole projection in one launch: from the float32 product qk [T, (n_heads +
+    n_kv_heads) * head_dim] (with `v_dim`, then n_kv_heads * v_dim columns of values; without, the keys are their own
+    values), the queries go, normed over all their columns with
     `q_weight` (one element a column), to q_out [T, n_heads * head_dim]; the keys, normed over all theirs with
-    `k_weight`, into the key page, and as they are into the transposed value page (`k_pages` None: q alone, and qk
-    may hold the queries only)."""
+    `k_weight`, into the key page; the values, or the keys as they are, into the transposed value page (`k_pages` None:
+    q alone, and qk may hold the queries only)."""
     T = qk.shape[0]
     qw, kw = int(n_heads) * int(head_dim), int(n_kv_heads) * int(head_dim)
     with_keys = k_pages is not None
-    _f32_rows(qk, "span_norm_kv_write: the q/k product", qw + (kw if with_keys else 0))
+    vd = int(v_dim or 0)
+    _f32_rows(qk, "span_norm_kv_write: the q/k product", qw + (kw + int(n_kv_heads) * vd if with_keys else 0))
     if q_out.stride(-1) != 1 or q_out.shape[0] < T or q_out.shape[1] < qw:
         raise KernelError(f"span_norm_kv_write: q_out {tuple(q_out.shape)} for {T} tokens of {qw} columns")
     if q_weight.numel() != qw or not q_weight.is_contiguous():
@@ -479,7 +513,7 @@ def span_norm_kv_write(qk, q_out, q_weight, k_weight, eps, positions, token_seq,
             raise KernelError(f"span_norm_kv_write: the key norm's weight must hold {kw} elements of the query norm's type")
         if k_pages.dtype != q_out.dtype or v_pages.dtype != q_out.dtype or \
                 tuple(k_pages.shape[1:]) != (n_kv_heads, block_size, head_dim) or \
-                tuple(v_pages.shape[1:]) != (n_kv_heads, head_dim, block_size) or not k_pages.is_contiguous() or not v_pages.is_contiguous():
+                tuple(v_pages.shape[1:]) != (n_kv_heads, vd or head_dim, block_size) or not k_pages.is_contiguous() or not v_pages.is_contiguous():
             raise KernelError(f"span_norm_kv_write: pages {tuple(k_pages.shape)}, {tuple(v_pages.shape)} ({k_pages.dtype})")
     if positions.numel() < T or token_seq.numel() < T:
         raise KernelError("span_norm_kv_write: the step's index tensors are shorter than its tokens")
@@ -487,7 +521,7 @@ def span_norm_kv_write(qk, q_out, q_weight, k_weight, eps, positions, token_seq,
           q_out.stride(0), _p(q_weight), _p(k_weight) if with_keys else None, dtype_code(q_weight.dtype), float(eps),
           _p(_i32(positions, "positions")), _p(_i32(token_seq, "token_seq")), _p(_i32(block_table, "block_table")),
           block_table.shape[1] if block_table is not None else 0, _p(k_pages), _p(v_pages) if with_keys else None, T,
-          int(n_heads), int(n_kv_heads), int(head_dim), int(block_size))
+          int(n_heads), int(n_kv_heads), int(head_dim), int(block_size), vd)
 
 
 def angle_table(positions, n_tokens: int, inv_freq: torch.Tensor) -> torch.Tensor:
@@ -629,7 +663,8 @@ def gemm(a: torch.Tensor, w: torch.Tensor, *, epilogue: int = EPI_STORE, out: to
          norm: tuple | None = None, pair_ids: torch.Tensor | None = None, pair_div: int = 1,
          always: tuple | None = None, w_kblocked: bool = False, row_ss: tuple | None = None,
          activation: str = "silu", store_activation: str | None = None, activation_params: tuple = (0.0, 0.0),
-         pre_scale: torch.Tensor | None = None, pre_scale_rows: torch.Tensor | None = None) -> torch.Tensor:
+         pre_scale: torch.Tensor | None = None, pre_scale_rows: torch.Tensor | None = None,
+         out_gate: tuple | None = None) -> torch.Tensor:
     """C[m, n] = sum_k a[m, k] * w[n, k] with an epilogue.
 
     `w` is [N, K], or [E, N, K] with `expert_offsets` [E+1] (rows sorted by expert).
@@ -657,7 +692,14 @@ def gemm(a: torch.Tensor, w: torch.Tensor, *, epilogue: int = EPI_STORE, out: to
     `pre_scale` (EPI_GATED; float32): gate and up of logical row m are multiplied by pre_scale[m] (or by
     pre_scale[pre_scale_rows[m]]) before the activation, which is what the activation sees when row m of `a` is
     scaled by that number.
+    `out_gate` = (logits float32 [rows, >= div * N], div) (EPI_STORE or EPI_STORE_F32 without bias): element n of output row m
+    is multiplied by sigmoid(logits[m // div, (m % div) * N + n]); div > 1 where the output's rows are parts of the gate's.
     """
+    gate_logits, gate_div = out_gate if out_gate is not None else (None, 0)
+    if gate_logits is not None and (store_activation is not None or epilogue not in (EPI_STORE, EPI_STORE_F32) or bias is not None
+                                    or gate_logits.dtype != torch.float32 or gate_logits.dim() != 2 or gate_logits.stride(1) != 1
+                                    or pair_ids is not None):
+        raise KernelError("gemm: gated outputs are plain stored products without bias, the gate's logits float32 rows")
     if store_activation not in STORED_ACTIVATIONS:
         raise KernelError(f"gemm: stored activation '{store_activation}' is not one of {sorted(k for k in STORED_ACTIVATIONS if k)}")
     if store_activation is not None and (epilogue not in (EPI_STORE, EPI_STORE_F32) or bias is not None):
@@ -720,6 +762,8 @@ def gemm(a: torch.Tensor, w: torch.Tensor, *, epilogue: int = EPI_STORE, out: to
         raise KernelError(f"gemm: output {tuple(out.shape)} {out.dtype} does not fit [{M},{N}] {out_dtype}")
     if bias is not None and bias.numel() != N:
         raise KernelError(f"gemm: bias has {bias.numel()} elements for {N} columns")
+    if gate_logits is not None and (gate_div < 1 or gate_logits.shape[1] < gate_div * N or gate_logits.shape[0] * gate_div < out.shape[0]):
+        raise KernelError(f"gemm: gate {tuple(gate_logits.shape)} for {tuple(out.shape)} outputs in parts of {gate_div}")
     if pre_scale is not None:
         if epilogue != EPI_GATED or pre_scale.dtype != torch.float32 or not pre_scale.is_contiguous() \
                 or (pre_scale_rows is None and pre_scale.numel() < M) or (pre_scale_rows is not None and pre_scale_rows.numel() < M):
@@ -734,8 +778,9 @@ def gemm(a: torch.Tensor, w: torch.Tensor, *, epilogue: int = EPI_STORE, out: to
           _p(_i32(pair_ids, "pair_ids")), int(pair_div),
           n_always, always_rows, always_from_a, n_w if w_kblocked else 0,
           _p(row_ss[0]) if row_ss is not None else None, row_ss[0].shape[1] if row_ss is not None else 0,
-          ACTIVATIONS[activation], STORED_ACTIVATIONS[store_activation], float(activation_params[0]),
-          float(activation_params[1]), _p(pre_scale), _p(_i32(pre_scale_rows, "pre_scale_rows")))
+          ACTIVATIONS[activation], STORED_ACTIVATIONS[store_activation] if gate_logits is None else _SACT_GATE,
+          float(activation_params[0]), float(activation_params[1]), _p(pre_scale), _p(_i32(pre_scale_rows, "pre_scale_rows")),
+          _p(gate_logits), gate_logits.stride(0) if gate_logits is not None else 0, int(gate_div))
     return out
 
 
@@ -818,7 +863,7 @@ def attention_tile_queries(dtype, head_dim: int, block_size: int) -> int:
 def attention_tiles(q, out, k_pages, v_pages, block_table, positions, item_seq, item_tok, item_n,
                     n_heads, n_kv_heads, head_dim, block_size, window, scale, tile_q: int = 64, mask_chunk: int = 0,
                     v_dim: int | None = None, keep_first: int = 0, sinks=None, gate=None, softcap: float = 0.0,
-                    slopes=None, gate_per_head: bool = False, turns=None) -> None:
+                    slopes=None, gate_per_head: bool = False, turns=None, distance_bias=None) -> None:
     """Blocks of queries: item i is item_n[i] <= tile_q consecutive tokens of sequence item_seq[i] from token
     item_tok[i] on; tile_q is 64 or attention_tile_queries(...).  `mask_chunk` > 0: the chunked mask (a query sees
     the keys of its own chunk of that many positions) instead of a window.  `v_dim`: size of a value head where it
@@ -827,9 +872,10 @@ def attention_tiles(q, out, k_pages, v_pages, block_table, positions, item_seq, 
     softmax's denominator and has no value.  `gate` (shape and type of `out`): the output is multiplied by sigmoid(gate).
     `softcap` > 0: a scaled score s becomes softcap * tanh(s / softcap).  `slopes` (float32 [n_heads]): the score of
     key t for the query at position p then loses slopes[h] * (p - t).  `turns` (an `angle_table` of v_dim / 2 angles a
-    token): the output pair (2m, 2m + 1) of every head is turned back by the token's angle m, before the gate."""
+    token): the output pair (2m, 2m + 1) of every head is turned back by the token's angle m, before the gate.
+    `distance_bias` (a `distance_bias_rows` table): a number per head and distance that joins the scaled score."""
     _check_attention_shapes(q, out, k_pages, v_pages, n_heads, n_kv_heads, head_dim, int(v_dim or head_dim), block_size)
-    _check_attention_extras(out, n_heads, 1 if gate_per_head else int(v_dim or head_dim), window, keep_first, sinks, gate, softcap, slopes)
+    _check_attention_extras(out, n_heads, 1 if gate_per_head else int(v_dim or head_dim), window, keep_first, sinks, gate, softcap, slopes, distance_bias)
     _check_turns(turns, q.shape[0], int(v_dim or head_dim), "attention")
     _call("attention", "fx_attn_tiles", _stream(), dtype_code(q.dtype), _p(q), q.stride(0), _p(out), out.stride(0),
           _p(k_pages), _p(v_pages), _p(_i32(block_table, "block_table")), block_table.shape[1],
@@ -837,7 +883,21 @@ def attention_tiles(q, out, k_pages, v_pages, block_table, positions, item_seq, 
           _p(_i32(item_n, "item_n")), item_seq.numel(), n_heads, n_kv_heads, head_dim, block_size,
           int(window or 0), float(scale), int(tile_q), int(v_dim or head_dim), int(mask_chunk or 0),
           int(keep_first or 0), _p(sinks), _p(gate), gate.stride(0) if gate is not None else 0, float(softcap or 0.0),
-          _p(slopes), 1 if gate_per_head else 0, _p(turns))
+          _p(slopes), 1 if gate_per_head else 0, _p(turns), 1 if gate is not None and gate.dtype == torch.float32 else 0,
+          _p(distance_bias), distance_bias.shape[1] - 2 * BIAS_PAD if distance_bias is not None else 0)
+
+
+BIAS_PAD = 16       # floats on either side of a head's row of distance biases (csrc/attention.hip)
+
+
+def distance_bias_rows(bias: torch.Tensor) -> torch.Tensor:
+    """The table the attention kernels read a bias per head and distance from: `bias` float32 [n_heads, n], element d the
+    number for a key d positions back (the last one also for every longer distance), laid out from far to near with the
+    farthest repeated in front and zeros behind: [n_heads, BIAS_PAD + n + BIAS_PAD]."""
+    if bias.dtype != torch.float32 or bias.dim() != 2 or bias.shape[1] < 1:
+        raise KernelError(f"distance biases are float32 [heads, distances], got {tuple(bias.shape)} ({bias.dtype})")
+    far = bias[:, -1:].expand(-1, BIAS_PAD)
+    return torch.cat([far, bias.flip(1), torch.zeros_like(far)], dim=1).contiguous()
 
 
 def _check_turns(turns, n_tokens: int, dims: int, what: str) -> None:
@@ -846,7 +906,11 @@ def _check_turns(turns, n_tokens: int, dims: int, what: str) -> None:
         raise KernelError(f"{what}: a table of angles {tuple(turns.shape)} for {n_tokens} tokens of {dims} turned dimensions")
 
 
-def _check_attention_extras(out, n_heads, v_dim, window, keep_first, sinks, gate, softcap=0.0, slopes=None) -> None:
+def _check_attention_extras(out, n_heads, v_dim, window, keep_first, sinks, gate, softcap=0.0, slopes=None,
+                            distance_bias=None) -> None:
+    if distance_bias is not None and (distance_bias.dtype != torch.float32 or not distance_bias.is_contiguous() or distance_bias.dim() != 2
+                                      or distance_bias.shape[0] != n_heads or distance_bias.shape[1] <= 2 * BIAS_PAD):
+        raise KernelError(f"attention: distance biases {tuple(distance_bias.shape)} ({distance_bias.dtype}) for {n_heads} heads")
     if keep_first and not window:
         raise KernelError("attention: kept first keys go with a window")
     if not 0.0 <= float(softcap or 0.0) < math.inf:
@@ -855,7 +919,7 @@ def _check_attention_extras(out, n_heads, v_dim, window, keep_first, sinks, gate
         raise KernelError(f"attention: distance slopes must be {n_heads} contiguous float32 values")
     if sinks is not None and (sinks.dtype != torch.float32 or not sinks.is_contiguous() or sinks.numel() != n_heads):
         raise KernelError(f"attention: sinks must be {n_heads} contiguous float32 values")
-    if gate is not None and (gate.dtype != out.dtype or gate.stride(-1) != 1 or gate.shape[0] < out.shape[0]
+    if gate is not None and (gate.dtype not in (out.dtype, torch.float32) or gate.stride(-1) != 1 or gate.shape[0] < out.shape[0]
                              or gate.shape[1] < n_heads * v_dim):
         raise KernelError(f"attention: gate {tuple(gate.shape)} ({gate.dtype}) for an output {tuple(out.shape)} ({out.dtype})")
 
@@ -900,7 +964,8 @@ def decode_attention_chunk(n_items: int, n_heads: int, n_kv_heads: int, max_kv_l
 def attention_decode(q, out, k_pages, v_pages, block_table, positions, item_seq, item_tok,
                      n_heads, n_kv_heads, head_dim, block_size, window, scale, max_kv_len, chunk=None,
                      waves=0, mask_chunk: int = 0, v_dim: int | None = None, keep_first: int = 0, sinks=None,
-                     gate=None, softcap: float = 0.0, slopes=None, gate_per_head: bool = False, turns=None) -> None:
+                     gate=None, softcap: float = 0.0, slopes=None, gate_per_head: bool = False, turns=None,
+                     distance_bias=None) -> None:
     """Single queries.  The keys go to ceil(max_kv_len / chunk) blocks whose results are merged in ascending
     order.  float32 cuts them at multiples of `chunk`, 256 by default (so that a result does not depend on the
     batch); bfloat16, whose blocks of up to eight waves share a chunk, cuts every sequence's own range of keys (from
@@ -909,7 +974,7 @@ def attention_decode(q, out, k_pages, v_pages, block_table, positions, item_seq,
     n = item_seq.numel()
     v_dim = int(v_dim or head_dim)
     _check_attention_shapes(q, out, k_pages, v_pages, n_heads, n_kv_heads, head_dim, v_dim, block_size)
-    _check_attention_extras(out, n_heads, 1 if gate_per_head else v_dim, window, keep_first, sinks, gate, softcap, slopes)
+    _check_attention_extras(out, n_heads, 1 if gate_per_head else v_dim, window, keep_first, sinks, gate, softcap, slopes, distance_bias)
     _check_turns(turns, q.shape[0], v_dim, "attention")
     if chunk is None:
         chunk = 256
@@ -924,7 +989,8 @@ def attention_decode(q, out, k_pages, v_pages, block_table, positions, item_seq,
           n_heads, n_kv_heads, head_dim, block_size, int(window or 0), float(scale),
           _p(part_o), _p(part_ml), splits, chunk, int(waves), v_dim, int(mask_chunk or 0),
           int(keep_first or 0), _p(sinks), _p(gate), gate.stride(0) if gate is not None else 0, float(softcap or 0.0),
-          _p(slopes), 1 if gate_per_head else 0, _p(turns))
+          _p(slopes), 1 if gate_per_head else 0, _p(turns), 1 if gate is not None and gate.dtype == torch.float32 else 0,
+          _p(distance_bias), distance_bias.shape[1] - 2 * BIAS_PAD if distance_bias is not None else 0)
 
 
 def router_select(logits, n_experts, top_k, renorm, gating=GATE_SOFTMAX, has_gate=False, selection_bias=None,

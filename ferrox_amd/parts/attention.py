@@ -11,6 +11,7 @@ decoder.rs:2099-2104, 3256-3267; this architecture has none).
 """
 from __future__ import annotations
 
+import bisect
 import math
 
 import torch
@@ -22,6 +23,26 @@ from .linear import Linear, matmul, same_dtype
 NO_ROTATION = Rotary(0, 1.0)
 FUSE_HEAD_NORMS = True      # (a switch for tests: the norms of q's and k's heads and the cache write as one launch)
 EVEN_BLOCKS_PER_CU = 250 / 256     # items of 128 queries pay from about one evenly loaded block per CU on (measured on 256 CUs)
+
+
+def bucket_starts(rows: int, far: int) -> list:
+    """The first distance of every row of a table of distance biases: the first rows // 2 distances have a row each;
+    row half + k begins at half * (far / half)^(k / (rows - half)), rounded up, so the rows widen with the logarithm of
+    the distance and the last one holds `far` and everything beyond.  Found in whole numbers (the power is compared, not
+    its logarithm), so no start is off by a rounding."""
+    half = rows // 2
+    m = rows - half
+    starts = list(range(half))
+    for k in range(m):
+        lo, hi = half, max(half, far)
+        while lo < hi:
+            mid = (lo + hi) // 2
+            if mid ** m * half ** k >= far ** k * half ** m:
+                hi = mid
+            else:
+                lo = mid + 1
+        starts.append(lo)
+    return starts
 
 
 def attention_items(ctx, tile_q: int = 64):
@@ -64,7 +85,8 @@ class PagedAttention(Mixer):
     takes_post_norm = True     # forward(..., post_norm=(weight, eps)) norms the output rows before they join the stream
     TENSORS = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
                "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias",
-               "q_norm": "q_norm.", "k_norm": "k_norm.", "sink": "sinks", "gate": "gate_proj.weight", "temperature": "temperature"}
+               "q_norm": "q_norm.", "k_norm": "k_norm.", "sink": "sinks", "gate": "gate_proj.weight", "temperature": "temperature",
+               "distance": "distance_bias"}
 
     def __init__(self, hidden_size: int, n_heads: int, n_kv_heads: int, head_dim: int, bias: bool,
                  position: PartSpec, window: int | None = None, scale: float | None = None,
@@ -73,7 +95,7 @@ class PagedAttention(Mixer):
                  own_kv: bool = True, retain: tuple | None = None, softcap: float | None = None,
                  distance_slopes=None, values_from_keys: bool = False, qk_norm_span: str = "head",
                  q_temperature: tuple | None = None, unit_values: float | None = None, head_temperature: bool = False,
-                 value_rotation: float | None = None):
+                 value_rotation: float | None = None, sink_value: float | None = None, distance_buckets: tuple | None = None):
         """`qk_norm`: kind and arguments of a norm over head_dim; two of them are built, with tensors under
         `q_norm.` and `k_norm.`, and applied to every head of q and of k before the rotation.
         `v_dim`: size of a value head where it differs from head_dim (the size of a query and key head).
@@ -83,6 +105,10 @@ class PagedAttention(Mixer):
         the two norms among them).
         `keep_first` (with a window): the first so many keys of a sequence stay visible to every later query.
         `sink`: a learned logit per head ([n_heads]) joins the softmax's denominator; it has no key and no value.
+        `sink_value`: a constant logit, the same for every head, in place of a learned sink (0: one is added to the
+        softmax's denominator).
+        `distance_buckets` = (rows, far): a learned table [rows, n_heads] of numbers that join a head's scaled score by
+        how far back the key is (`bucket_starts` says which row serves which distances).
         `out_gate`: the heads' outputs are multiplied by sigmoid(W_g x), x the mixer's input, before the output
         projection (W_g: [n_heads * v_dim, hidden]); "head": one gate per head, W_g: [n_heads, hidden].
         `q_temperature` = (coef, every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1),
@@ -120,6 +146,14 @@ class PagedAttention(Mixer):
             raise ValueError(f"keep_first {keep_first} is negative")
         self.has_sink, self.out_gate, self.own_kv = bool(sink), bool(out_gate), bool(own_kv)
         self.gate_per_head = out_gate == "head"
+        self.sink_value = float(sink_value) if sink_value is not None else None
+        if self.sink_value is not None and (self.has_sink or not math.isfinite(self.sink_value)):
+            raise ValueError("an attention layer's sinks are learned or one finite constant")
+        self.distance_buckets = (int(distance_buckets[0]), int(distance_buckets[1])) if distance_buckets is not None else None
+        if self.distance_buckets is not None:
+            rows, far = self.distance_buckets
+            if rows < 2 or (far <= rows // 2 and not (self.window and self.window <= rows // 2)):
+                raise ValueError(f"a table of {rows} distance biases whose last row begins at {far}")
         self.q_temperature = (float(q_temperature[0]), int(q_temperature[1])) if q_temperature else None
         if self.q_temperature and self.q_temperature[1] < 1:
             raise ValueError(f"a query temperature that steps every {q_temperature[1]} positions")
@@ -179,7 +213,7 @@ class PagedAttention(Mixer):
             self.kvw = self.vw = 0       # (no rows of k and v in the mixer's matrix)
         if self.values_from_keys:
             self.vw = 0                  # (no rows of v: the key rows are the values)
-        self.qkv = self.o_proj = self.sinks = self.slopes = self.temperature = self.value_frequencies = None
+        self.qkv = self.o_proj = self.sinks = self.slopes = self.temperature = self.value_frequencies = self.distance_bias = None
         self.q_norm = self.k_norm = None
         if qk_norm is not None and self.span_norms:
             self.q_norm = NORMS.build(PartSpec(qk_norm.kind, dict(qk_norm.args, size=self.qw)))
@@ -215,6 +249,8 @@ class PagedAttention(Mixer):
             specs[n["sink"]] = ParamSpec((self.n_heads,))
         if self.head_temperature:
             specs[n["temperature"]] = ParamSpec((self.n_heads,), init="ones")
+        if self.distance_buckets is not None:
+            specs[n["distance"]] = ParamSpec((self.distance_buckets[0], self.n_heads))
         if self.out_gate:
             specs[n["gate"]] = ParamSpec((self.n_heads if self.gate_per_head else self.ow, H))
         return specs
@@ -249,6 +285,21 @@ class PagedAttention(Mixer):
             self.sinks = fetch(n["sink"]).float().contiguous()
         if self.distance_slopes is not None:
             self.slopes = torch.tensor(self.distance_slopes, dtype=torch.float64).to(torch.float32).to(w.device)
+        if self.sink_value is not None:
+            self.sinks = torch.full((self.n_heads,), self.sink_value, dtype=torch.float32, device=w.device)
+        if self.distance_buckets is not None:
+            # a number per distance instead of per row: what the kernels look up
+            rows = torch.tensor(self.distance_rows(), dtype=torch.int64, device=w.device)
+            self.distance_bias = ops.distance_bias_rows(fetch(n["distance"]).float()[rows].t())
+
+    def distance_rows(self) -> list:
+        """The table's row for every distance that a query can see and that has not reached the last row for good."""
+        rows, far = self.distance_buckets
+        starts = bucket_starts(rows, far) if far > rows // 2 else list(range(rows // 2))
+        n = starts[-1] + 1
+        if self.window:
+            n = min(n, self.window)
+        return [bisect.bisect_right(starts, d) - 1 for d in range(n)]
 
     def value_pair_order(self) -> torch.Tensor:
         """Element i of a value head as the pages hold it is element order[i] of the head as the checkpoint has it."""
@@ -276,22 +327,20 @@ class PagedAttention(Mixer):
 
     def normed_spans_and_cache(self, x, ctx, table, cache):
         """As `normed_heads_and_cache` for norms over the whole projection: q [T, qw] normed over all its columns, the
-        keys normed over all theirs into the key page and, where they are their own values, as projected into the
-        value page, in one launch; returns q and the rest of the product (v, the output gate's rows)."""
+        keys normed over all theirs into the key page and the values (or the keys as projected, where they are their own
+        values) into the value page, in one launch behind a float32 product; returns q and the output gate's rows."""
         wq, eps = self.q_norm.rms_params()
         w = self.qkv.weight
-        cut = self.qw + self.kvw
+        cut = self.qw + self.kvw + self.vw
         qk = matmul(x, w[:cut], epilogue=ops.EPI_STORE_F32)
         rest = matmul(x, w[cut:]) if w.shape[0] > cut else None
         q = torch.empty((ctx.n_tokens, self.qw), dtype=ctx.act_dtype, device=qk.device)
         writes = self.own_kv and cache.writes
-        if writes and not self.values_from_keys:
-            raise ValueError("norms over the whole projection with a value projection of their own have no kernel yet")
         debug.region("rope + cache write")
         wk = self.k_norm.rms_params()[0] if self.k_norm is not None else None
         ops.span_norm_kv_write(qk, q, wq, wk, eps, ctx.positions, ctx.token_seq, table,
                                cache.pages["k"] if writes else None, cache.pages["v"] if writes else None,
-                               self.n_heads, self.n_kv_heads, self.head_dim, cache.block_size)
+                               self.n_heads, self.n_kv_heads, self.head_dim, cache.block_size, v_dim=self.vw // self.n_kv_heads)
         return q, rest
 
     def page_shapes(self, block_size: int) -> dict:
@@ -454,9 +503,10 @@ class PagedAttention(Mixer):
                 else:
                     q, k, rest = self.normed_heads(x, ctx)
                 qkv = q
-                v = rest[:, :self.vw] if rest is not None else None
+                in_rest = 0 if self.span_norms else self.vw      # (columns of v in front of the gate's)
+                v = rest[:, :in_rest] if rest is not None else None
                 if self.out_gate:
-                    gate = rest[:, self.vw:]
+                    gate = rest[:, in_rest:]
             else:
                 if qkv is None:
                     if isinstance(x, ops.ScaleLater):     # rows of a norm whose scale the product applies
@@ -485,7 +535,7 @@ class PagedAttention(Mixer):
         # (the gate multiplies the heads' outputs as the attention kernels write them)
         mask = dict(mask_chunk=self.chunk or 0, v_dim=self.v_dim, keep_first=self.keep_first, sinks=self.sinks,
                     gate=None if fused else gate, softcap=self.softcap, slopes=self.slopes,
-                    gate_per_head=self.gate_per_head and gate is not None, turns=v_turns)
+                    gate_per_head=self.gate_per_head and gate is not None, turns=v_turns, distance_bias=self.distance_bias)
         if items["n_tiles"]:
             ops.attention_tiles(q, out, k_pages, v_pages, table, ctx.positions,
                                 items["tile_seq"], items["tile_tok"], items["tile_n"], *common, tile_q=tile_q, **mask)

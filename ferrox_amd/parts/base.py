@@ -215,6 +215,8 @@ def walk_parts(part: "Part", prefix: str = ""):
 
 
 class Norm(Part):
+    as_is = False            # True: forward hands out the rows unchanged (a place for a norm where a design has none)
+
     def forward(self, h, ctx: StepContext, rows=None):
         raise NotImplementedError
 
@@ -228,6 +230,11 @@ class Norm(Part):
         """(weight or None, eps) if this norm is y = x * rsqrt(mean(x^2) + eps) (* weight): what `rms_params` gives,
         and also a norm of that form without a weight; None for any other norm."""
         return self.rms_params()
+
+    def add_normed(self, h, y, ctx: StepContext, rows: bool = False):
+        """h += norm(y) for a sublayer's float32 output rows y; with `rows` the new rows of h in the activation type are
+        returned, else None.  Norms that do not offer it cannot stand behind a sublayer of a `postnorm` block."""
+        raise NotImplementedError(f"{type(self).__name__} does not norm what joins the stream")
 
 
 @dataclass(frozen=True)

@@ -4,7 +4,7 @@ from __future__ import annotations
 import torch
 
 from .. import debug
-from .base import BLOCKS, FEED_FORWARDS, MIXERS, NORMS, Block, ParamSpec
+from .base import BLOCKS, FEED_FORWARDS, MIXERS, NORMS, Block, ParamSpec, PartSpec
 from .linear import Linear
 
 
@@ -126,6 +126,58 @@ class ParallelBlock(Block):
             self.ffn.forward(x, ctx, h)
 
 
+def sublayer_rows(part, out, x, ctx, *cache):
+    """The sublayer's output rows in `out`: a part that says `takes_fresh` stores them with its last product,
+    any other adds them into a zeroed buffer."""
+    from .. import ops
+    if getattr(part, "takes_fresh", False):
+        part.forward(x, ctx, *cache, out, fresh=True)
+    else:
+        ops.fill_u32(out, 0)
+        part.forward(x, ctx, *cache, out)
+
+
+@BLOCKS.register("postnorm")
+class PostNormBlock(Block):
+    """h += norm1(mixer(h)); h += norm2(ffn(h)): the sublayers read the stream as it is, and a norm stands behind each of
+    them.  A layer without a feed-forward has the first half only.
+
+    A sublayer leaves its output in a float32 buffer; one launch norms it, adds it into the stream and writes the new
+    rows in the type that the next sublayer reads (the next block's too, if that block's mixer reads the stream as it is)."""
+    slots = {"norm1": NORMS, "mixer": MIXERS, "norm2": NORMS, "ffn": FEED_FORWARDS}
+    optional_slots = ("norm2", "ffn")
+    chains_norms = True     # forward takes `normed` and `then` and returns what the next block may take as `normed`
+
+    def __init__(self, parts: dict, prefixes: dict):
+        self.norm1, self.mixer, self.norm2, self.ffn = parts["norm1"], parts["mixer"], parts.get("norm2"), parts.get("ffn")
+        if (self.ffn is None) != (self.norm2 is None):
+            raise ValueError("a post-norm block has a feed-forward and its norm, or neither")
+        self.first_norm = NORMS.build(PartSpec("unnormed"))
+        self._prefixes = prefixes
+
+    def children(self):
+        return [(self._prefixes[s], getattr(self, s)) for s in ("norm1", "mixer", "norm2", "ffn") if getattr(self, s) is not None] \
+            + [("", self.first_norm)]
+
+    def forward(self, h, ctx, cache, normed=None, then=None):
+        """`normed`: the stream's rows in the activation type, if the block before has made them.  `then`: (what the next
+        block puts in front of its mixer, ...)."""
+        after = then is not None and then[0].as_is
+        x = normed
+        if x is None:
+            debug.region("norm")
+            x = self.first_norm.forward(h, ctx)
+        out = torch.empty_like(h)
+        sublayer_rows(self.mixer, out, x, ctx, cache)
+        debug.region("norm")
+        x = self.norm1.add_normed(h, out, ctx, rows=self.ffn is not None or after)
+        if self.ffn is None:
+            return x
+        sublayer_rows(self.ffn, out, x, ctx)
+        debug.region("norm")
+        return self.norm2.add_normed(h, out, ctx, rows=after)
+
+
 @BLOCKS.register("gated_prenorm")
 class GatedPreNormBlock(Block):
     """h += G1 * mixer(C(x1)),  x1 = norm1(h);  h += G2 * ffn(x2),  x2 = norm2(h), with two optional additions to the
@@ -182,17 +234,6 @@ class GatedPreNormBlock(Block):
     def state_shapes(self) -> dict:
         return {"conv": ((self.hidden_size, self.conv_taps - 1), torch.float32)} if self.conv_taps else {}
 
-    @staticmethod
-    def _into(part, out, x, ctx, *cache):
-        """The sublayer's output rows in `out`: a part that says `takes_fresh` stores them with its last product,
-        any other adds them into a zeroed buffer."""
-        from .. import ops
-        if getattr(part, "takes_fresh", False):
-            part.forward(x, ctx, *cache, out, fresh=True)
-        else:
-            ops.fill_u32(out, 0)
-            part.forward(x, ctx, *cache, out)
-
     def _join(self, h, out, gate, x, ctx=None, then=None):
         """The sublayer's rows through their gate into the stream.  `then`: the norm that reads the stream next; if it
         offers `after_gated_add`, the add and that norm are one launch, and its rows are returned."""
@@ -231,12 +272,12 @@ class GatedPreNormBlock(Block):
             read = ops.short_conv(x, self.taps, cache.state["block.conv"], ctx.token_seq, sequence_starts(ctx), ctx.slot_ids,
                                   ctx.n_seqs, activation=None, add_input=True, out_dtype=x.dtype)
         out = torch.empty_like(h)
-        self._into(self.mixer, out, read, ctx, cache)
+        sublayer_rows(self.mixer, out, read, ctx, cache)
         x = self._join(h, out, self.gate1, x, ctx, self.norm2 if self.ffn is not None else after)
         if self.ffn is None:
             return x
         if x is None:
             debug.region("norm")
             x = self.norm2.forward(h, ctx)
-        self._into(self.ffn, out, x, ctx)
+        sublayer_rows(self.ffn, out, x, ctx)
         return self._join(h, out, self.gate2, x, ctx, after)

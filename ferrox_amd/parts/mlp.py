@@ -57,6 +57,35 @@ class GatedMLP(FeedForward):
         self.down(act, epilogue=ops.EPI_RESID, out=residual, row_scale=row_scale)
 
 
+@FEED_FORWARDS.register("mlp")
+class UngatedMLP(FeedForward):
+    """down( act(up x) ): a feed-forward without a gate; the activation is the first product's epilogue
+    (`ops.STORED_ACTIVATIONS`), e.g. "relu2", the square of relu."""
+    kernel_libraries = ("gemm",)
+    TENSORS = {"up": "up_proj.weight", "down": "down_proj.weight"}
+    takes_fresh = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "relu2", names: dict | None = None):
+        if activation is None or activation not in ops.STORED_ACTIVATIONS:
+            raise ValueError(f"activation '{activation}' is not one of {sorted(k for k in ops.STORED_ACTIVATIONS if k)}")
+        self.hidden_size, self.intermediate_size, self.activation = int(hidden_size), int(intermediate_size), activation
+        self.names = dict(self.TENSORS, **(names or {}))
+        self.up = self.down = None
+
+    def param_specs(self):
+        return {self.names["up"]: ParamSpec((self.intermediate_size, self.hidden_size)),
+                self.names["down"]: ParamSpec((self.hidden_size, self.intermediate_size))}
+
+    def load(self, fetch):
+        self.up, self.down = Linear(fetch(self.names["up"])), Linear(fetch(self.names["down"]))
+
+    def forward(self, x, ctx, residual, fresh: bool = False) -> None:
+        debug.region("mlp up")
+        act = self.up(x, store_activation=self.activation)
+        debug.region("mlp down")
+        self.down(act, epilogue=ops.EPI_STORE_F32 if fresh else ops.EPI_RESID, out=residual)
+
+
 @FEED_FORWARDS.register("swiglu")
 class SwiGLU(GatedMLP):
     """The gated feed-forward with silu, under the name this architecture's description uses."""

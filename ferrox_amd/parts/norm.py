@@ -41,6 +41,13 @@ class RMSNorm(Norm):
             else:
                 self.weight = w.contiguous()
 
+    def add_normed(self, h, y, ctx, rows: bool = False):
+        """As `LayerNorm.add_normed` (the rows are a launch of their own here)."""
+        if not self.has_weight:
+            raise ValueError("an RMS norm without a weight does not norm what joins the stream here")
+        ops.rmsnorm_add(h, y, self.weight, self.eps)
+        return ops.cast(h, ctx.act_dtype) if rows else None
+
     def rms_params(self):
         """(weight, eps) of a norm that other parts' kernels may apply themselves; a norm without a weight declines."""
         return (self.weight, self.eps) if self.has_weight else None
@@ -77,9 +84,25 @@ class LayerNorm(Norm):
     def forward(self, h, ctx, rows=None):
         return ops.layernorm(h, self.weight, self.bias, self.eps, ctx.act_dtype, rows=rows)
 
+    def add_normed(self, h, y, ctx, rows: bool = False):
+        """h += norm(y), y a sublayer's float32 output rows, in one launch; with `rows` the new rows of h are returned in
+        the step's activation type, made by the same launch (else None)."""
+        return ops.layernorm_add(h, y, self.weight, self.bias, self.eps, ctx.act_dtype if rows else None)
+
     def after_gated_add(self, h, y, gate_logits, ctx):
         """h += y * sigmoid(gate_logits), then this norm of the new rows, in one launch; None where the kernel does
         not take the rows (the caller then does the two by themselves)."""
         if self.size > ops.GATED_ADD_NORM_MAX:
             return None
         return ops.gated_add_layernorm(h, y, gate_logits, self.weight, self.bias, self.eps, ctx.act_dtype)
+
+
+@NORMS.register("unnormed")
+class Unnormed(Norm):
+    """The rows of the stream as they are, in the type that products read: what a sublayer without a norm in front of it
+    reads.  (In float32 that is the stream itself: a reader must be done with it before the stream changes.)"""
+    kernel_libraries = ("elementwise",)
+    as_is = True
+
+    def forward(self, h, ctx, rows=None):
+        return ops.cast(h if rows is None else h.index_select(0, rows), ctx.act_dtype)
