@@ -80,10 +80,11 @@ def test_stop_ids_are_one_or_several():
 
 
 def test_registry_is_closed(tmp_path):
-    assert known_architectures() == ["Besulix", "Fokinex", "Kovalorn", "Panarax", "Qwen2MoeForCausalLM", "Rafilix"]
+    assert known_architectures() == ["Besulix", "Fokinex", "Kovalorn", "Panarax", "Qwen2MoeForCausalLM", "Rafilix", "Zazerax"]
     assert resolve({"architecture": "Fokinex"}).model_type == "fokinex"
     assert resolve({"architecture": "Panarax"}).model_type == "panarax"
     assert resolve({"architecture": "Besulix"}).model_type == "besulix"
+    assert resolve({"architecture": "Zazerax"}).model_type == "zazerax"
     assert resolve({"architecture": "Rafilix"}).model_type == "rafilix"
     assert resolve({"architecture": "Kovalorn"}).model_type == "kovalorn"
     with pytest.raises(ConfigError) as e:
