@@ -409,7 +409,7 @@ def test_keys_at_window_edges_and_page_borders(tmp_path_factory, dtype):
     base = plain.forward(cfg, w, reqs["long"])
     for change in ({"mask": {"size": 39}}, {"mask": {"size": 41}}, {"bias_max": 36}):
         off = u.row_errors(plain.forward(u.changed(cfg, 0, **change), w, reqs["long"]), base)
-        assert int((off > 2 * limit).sum()) > 150, f"{change} would not show"
+        assert float(off.max()) > 3 * limit and int((off > limit).sum()) > 60, f"{change} would not show"
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -434,6 +434,7 @@ def test_a_far_key_among_hundreds(tmp_path_factory, dtype, kind):
         w["l0.mix.uk"] = uk.to(torch.bfloat16)
         if second:
             q_in = plain.rms_norm((wf["l0.mix.dq"] @ q_in)[None], wf["l0.mix.dq.norm"], 1e-6)[0]
+        w["l0.norm1"] = (2.0 * wf["l0.norm1"]).to(torch.bfloat16)
         name = "l0.mix.uq" if second else "l0.mix.q"
         q = wf[name]
         q[:24] += torch.outer(direction - q[:24] @ q_in, q_in) / (q_in @ q_in)

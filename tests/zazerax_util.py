@@ -116,6 +116,8 @@ def make_weights(cfg: dict, seed: int, bias_rows: int = BIAS_ROWS) -> dict:
         last = name.split(".")[-1]
         if last.startswith("norm"):
             t = 1.0 + 0.2 * torch.randn(shape, generator=gen)
+            if last in ("norm1", "norm2"):      # behind a sublayer: half the stream's size, or eight layers multiply every rounding
+                t = 0.5 * t
         elif last == "rel":
             t = 1.2 * torch.randn(shape, generator=gen)
         elif name == "embed":
