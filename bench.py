@@ -7,7 +7,7 @@
                                                                  per-kernel times under rocprofv3 (a child process)
     python bench.py --compare-designs [--design TEXT] [--design-size 1k|2k]
                                                                  four layers of each other design (Rafilix, Kovalorn, Fokinex, Panarax,
-                                                                 Besulix)
+                                                                 Besulix, Zazerax)
                                                                  beside the closest models at equal sizes: prefill and decode
 
 Model: the layer sizes of Qwen1.5-MoE-A2.7B with seeded random bf16 weights
@@ -409,7 +409,7 @@ def run_workload(name: str, args) -> int:
     return 0
 
 
-# ---- Rafilix, Kovalorn, Fokinex, Panarax and Besulix beside the closest existing model, at equal layer sizes ----------------------------------
+# ---- Rafilix, Kovalorn, Fokinex, Panarax, Besulix and Zazerax beside the closest existing model, at equal layer sizes ----------------------------------
 # Layer sizes that resemble a real model's; every model is four layers of random weights.  The Rafilix layers are
 # measured by kind (all attention, all recurrent) and in the design's usual mixture, the Qwen2-MoE layers have the
 # same width, heads, experts and expert width and no shared expert (Rafilix has none).
@@ -517,11 +517,35 @@ def design_configs(s: dict) -> dict:
         return {"architecture": "Besulix", "vocab": s["vocab"], "width": s["width"], "max_positions": 16384, "norm": {"eps": 1e-5},
                 "logit_softcap": 30.0, "layers": [{"type": kind, "mixer": mixers[kind], "mlp": None if i in bare else dense}
                                                   for i, kind in enumerate(kinds)]}
+
+    # Zazerax: post-norm layers (layer norms) around windowed attention with distance biases and a constant sink, or latent
+    # attention with queries from the stream or from a latent and an output gate (a latent and a rotated key part of 256
+    # numbers, as above); feed-forwards of two matrices of half as many columns again, so that the weights are as many.  In
+    # the mixed variant the last layer runs the first layer's weights.  Beside it (above): Kovalorn's attention and
+    # Fokinex's latent attention.
+    def zazerax(kinds, again=None):
+        H, D = s["heads"], s["dim"]
+        latent = {"heads": H, "dim": D, "rot_dim": s["rot_dim"], "vdim": D, "kv_rank": s["kv_rank"], "scale": (D + s["rot_dim"]) ** -0.5}
+        mixers = {
+            "attention": {"heads": H, "kv_heads": s["kv_heads"], "dim": D, "vdim": D, "scale": D ** -0.5, "bias_max": 1024,
+                          "bias_rows": 32, "mask": {"size": 8192}},
+            "latent_attention": {**latent, "rot": {"base": 10000.0, "dims": s["rot_dim"],
+                                                   "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}},
+            "latent_attention_2": {**latent, "q_rank": s["q_rank"], "rot": {"base": 500000.0, "dims": s["rot_dim"]}},
+        }
+        layers = [{"type": kind, "mixer": mixers[kind], "mlp": {"kind": "dense", "ff": s["dense_ff"] * 3 // 2}} for kind in kinds]
+        for i, j in (again or {}).items():
+            layers[i] = {**layers[j], "weights_of": j}
+        return {"architecture": "Zazerax", "vocab": s["vocab"], "width": s["width"], "max_positions": 16384, "norm": {"eps": 1e-5},
+                "embedding": {"scale": 1.0}, "layers": layers}
     more = {"panarax lightning": panarax(["lightning"] * 4), "panarax lru": panarax(["rglru"] * 4),
             "panarax side by side": panarax(["parallel"] * 4), "panarax experts": panarax(["lightning"] * 4, sparse=(0, 1, 2, 3)),
             "panarax mixed": panarax(["lightning", "rglru", "parallel", "lightning"], sparse=(1, 3)),
             "besulix side by side": besulix(["parallel"] * 4), "besulix memory": besulix(["mlstm"] * 4),
             "besulix mixed": besulix(["parallel", "mlstm", "parallel", "mlstm"], bare=(1, 3)),
+            "zazerax attention": zazerax(["attention"] * 4), "zazerax latent": zazerax(["latent_attention"] * 4),
+            "zazerax latent 2": zazerax(["latent_attention_2"] * 4),
+            "zazerax mixed": zazerax(["latent_attention", "attention", "latent_attention_2", "latent_attention"], again={3: 0}),
             "kovalorn dense": kovalorn_dense(), "fokinex latent": fokinex(["latent"] * 4),
             "fokinex side by side": fokinex(["parallel"] * 4),
             "fokinex mixed": fokinex(["latent", "latent", "reader", "parallel"])}
