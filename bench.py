@@ -520,8 +520,8 @@ def design_configs(s: dict) -> dict:
 
     # Zazerax: post-norm layers (layer norms) around windowed attention with distance biases and a constant sink, or latent
     # attention with queries from the stream or from a latent and an output gate (a latent and a rotated key part of 256
-    # numbers, as above); feed-forwards of two matrices of half as many columns again, so that the weights are as many.  In
-    # the mixed variant the last layer runs the first layer's weights.  Beside it (above): Kovalorn's attention and
+    # numbers, as above); feed-forwards of two matrices of about half as many columns again (4,096 and 8,192), so that the weights
+    # are about as many.  In the mixed variant the last layer runs the first layer's weights.  Beside it (above): Kovalorn's attention and
     # Fokinex's latent attention.
     def zazerax(kinds, again=None):
         H, D = s["heads"], s["dim"]
@@ -533,7 +533,7 @@ def design_configs(s: dict) -> dict:
                                                    "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}},
             "latent_attention_2": {**latent, "q_rank": s["q_rank"], "rot": {"base": 500000.0, "dims": s["rot_dim"]}},
         }
-        layers = [{"type": kind, "mixer": mixers[kind], "mlp": {"kind": "dense", "ff": s["dense_ff"] * 3 // 2}} for kind in kinds]
+        layers = [{"type": kind, "mixer": mixers[kind], "mlp": {"kind": "dense", "ff": s["dense_ff"] * 3 // 2048 * 1024}} for kind in kinds]
         for i, j in (again or {}).items():
             layers[i] = {**layers[j], "weights_of": j}
         return {"architecture": "Zazerax", "vocab": s["vocab"], "width": s["width"], "max_positions": 16384, "norm": {"eps": 1e-5},

@@ -17,6 +17,7 @@
 // query's result does not depend on what else is computed with it.
 #include "common.h"
 #include "attention.h"
+#include <type_traits>
 
 FX_DEFINE_LAST_ERROR()
 
@@ -506,20 +507,16 @@ __device__ __forceinline__ float quad_sum(float x) {
     return __uint_as_float(b[0]) + __uint_as_float(b[1]);
 }
 
+// What the scores of a launch go through between the product and the softmax (the matrix-unit kernels have an instance for
+// each: code that a launch does not run still takes registers).
+enum { SHAPE_NONE = 0, SHAPE_CAP_SLOPE = 1, SHAPE_BIAS = 2 };
+static inline int shape_of(const AttnArgs& a) { return a.bias ? SHAPE_BIAS : (shapes_scores(a) ? SHAPE_CAP_SLOPE : SHAPE_NONE); }
+
 // A lane's 16 raw scores sc[kb][r] of keys key0 + 4*kb + r, scaled, capped and less the head's penalty for the
 // distance from the row's query at qpos (`shaped_score` with a tanh made of one exponential and one reciprocal, whose
 // error, some 1e-7 of the cap, is far below what bfloat16 operands leave of a score): afterwards they are scores in natural
-// units, and the softmax step takes them with c = log2(e).  `bias(i)`: the head's bias for key key0 + i (asked for where
-// the launch has one).
-template <typename B>
-__device__ __forceinline__ void shape_scores(f32x4_t (&sc)[4], int key0, const AttnArgs& a, float slope, int qpos, B&& bias) {
-    if (a.bias && a.softcap <= 0.f && !a.slopes) {      // a bias alone: one multiply-add a score
-#pragma unroll
-        for (int kb = 0; kb < 4; ++kb)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) sc[kb][r] = fmaf(sc[kb][r], a.scale, bias(4 * kb + r));
-        return;
-    }
+// units, and the softmax step takes them with c = log2(e).
+__device__ __forceinline__ void cap_and_slope(f32x4_t (&sc)[4], int key0, const AttnArgs& a, float slope, int qpos) {
     // tanh(x) = 1 - 2 / (1 + e^2x): the exponent in base 2 with the scale folded in, the quotient from the hardware's
     // reciprocal (1 ulp), cap and -2 cap as the multiply-add's constants
     const bool capped = a.softcap > 0.f;
@@ -535,12 +532,19 @@ __device__ __forceinline__ void shape_scores(f32x4_t (&sc)[4], int key0, const A
             else s = sc[kb][r] * a.scale;
             sc[kb][r] = fmaf(-slope, d0 - (float)(4 * kb + r), s);
         }
-    if (a.bias) {
-#pragma unroll
-        for (int kb = 0; kb < 4; ++kb)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) sc[kb][r] += bias(4 * kb + r);
+}
+// the same with the head's bias for key key0 + i, `bias(i)`
+template <typename B>
+__device__ __forceinline__ void shape_with_bias(f32x4_t (&sc)[4], int key0, const AttnArgs& a, float slope, int qpos, B&& bias) {
+    float scale = a.scale;
+    if (a.softcap > 0.f || a.slopes) {
+        cap_and_slope(sc, key0, a, slope, qpos);
+        scale = 1.f;
     }
+#pragma unroll
+    for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sc[kb][r] = fmaf(sc[kb][r], scale, bias(4 * kb + r));
 }
 
 // One step of the one-pass softmax on a lane's 16 raw scores sc[kb][r] of keys key0 + 4*kb + r
@@ -621,7 +625,7 @@ __device__ __forceinline__ uint32_t opaque_mask(bool ok) {
 }
 __device__ __forceinline__ uint4 and_mask(uint4 x, uint32_t m) { return make_uint4(x.x & m, x.y & m, x.z & m, x.w & m); }
 
-template <int HD>   // compile-time bound of head_dim (a.hd <= HD)
+template <int HD, int SHAPE>   // HD: compile-time bound of head_dim (a.hd <= HD)
 struct WaveAttn {
     static constexpr int KS = HD / 32;   // k-steps of S^T = K Q^T
     static constexpr int CB = HD / 16;   // column blocks of O
@@ -686,8 +690,6 @@ struct WaveAttn {
             page_slot(a, span.has(key_b) ? key_b : safe_group, kblk, kslots_b[kb]);
             kpage_b[kb] = pl.page(kblk);
         }
-        BiasRow bias = {};
-        if (a.bias) bias = fetch_bias(a, head, qpos - (kt0 + 16 * g));
         const bf16* vbase = (const bf16*)a.v_pages + ((size_t)vpage * a.nkv + kvh) * vd * bs + vslot;
         uint4 vv[EARLY_V ? CB : 1][2];
         const uint32_t vmask = opaque_mask(vlive);
@@ -725,6 +727,8 @@ struct WaveAttn {
                 }
             }
         }
+        BiasRow bias = {};      // (behind the keys: in front of them it would take the registers that their addresses need)
+        if (SHAPE == SHAPE_BIAS) bias = fetch_bias(a, head, qpos - (kt0 + 16 * g));
 #pragma unroll
         for (int kb = 0; kb < 4; ++kb) {
             sc[kb] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
@@ -758,8 +762,9 @@ struct WaveAttn {
         if (!EARLY_V) fetch_values(0);
         // softmax on this lane's 16 scores (keys kt0 + 16g + 4kb + r); the row's four lanes share max and sum
         uint4 p_lo, p_hi;
-        const bool shaped = shapes_scores(a);
-        if (shaped) shape_scores(sc, kt0 + 16 * g, a, slope, qpos, [&](int i) { return bias.v[i >> 2][i & 3]; });
+        constexpr bool shaped = SHAPE != SHAPE_NONE;
+        if (SHAPE == SHAPE_CAP_SLOPE) cap_and_slope(sc, kt0 + 16 * g, a, slope, qpos);
+        if (SHAPE == SHAPE_BIAS) shape_with_bias(sc, kt0 + 16 * g, a, slope, qpos, [&](int i) { return bias.v[i >> 2][i & 3]; });
         const float alpha = softmax_step<true>(sc, kt0 + 16 * g, lo, hi, shaped ? LOG2E : a.scale * LOG2E, m, l, p_lo, p_hi, span.keep);
         const bool rescale = __builtin_amdgcn_ballot_w64(alpha != 1.f) != 0;
         float al[4] = {1.f, 1.f, 1.f, 1.f};
@@ -798,7 +803,7 @@ struct WaveAttn {
 };
 
 // prefill: item = up to 16 consecutive queries of one sequence; block = one wave = (item, head)
-template <int HD>
+template <int HD, int SHAPE>
 __global__ __launch_bounds__(64) void attn_mfma_tile_kernel(AttnArgs a) {
     const int item = blockIdx.x >> 2, sub = blockIdx.x & 3, h = blockIdx.y, lane = threadIdx.x, li = lane & 15, g = lane >> 4;
     const int kvh = h / (a.nh / a.nkv);
@@ -816,7 +821,7 @@ __global__ __launch_bounds__(64) void attn_mfma_tile_kernel(AttnArgs a) {
         lo = first_visible(a, hi);
         qrow = (const bf16*)a.q + (size_t)(tok0 + li) * a.ldq + (size_t)h * hd;
     }
-    WaveAttn<HD> w;
+    WaveAttn<HD, SHAPE> w;
     w.init(qrow, hd);
     const PageLookup pl = {bt, nullptr, 0, 0};
     const KeySpan span = {kv_begin, kv_end, a.keep_first};
@@ -830,7 +835,7 @@ __global__ __launch_bounds__(64) void attn_mfma_tile_kernel(AttnArgs a) {
         const float fr = __shfl(fin, row, 64);
         if (row < n) {
 #pragma unroll
-            for (int cb = 0; cb < WaveAttn<HD>::CB; ++cb) {
+            for (int cb = 0; cb < WaveAttn<HD, SHAPE>::CB; ++cb) {
                 const int d = 16 * cb + li;
                 if (d < a.vd) store_lane<bf16>(a, tok0 + row, h, d, w.o[cb][r] * fr);
             }
@@ -841,7 +846,7 @@ __global__ __launch_bounds__(64) void attn_mfma_tile_kernel(AttnArgs a) {
 // decode, several waves per block: block = (item, kv head x group block of 16 query heads, split);
 // its waves take the split's tiles of 64 keys in turn and their results are merged through LDS in
 // wave order.  With one split the block writes the output itself, no second launch.
-template <int HD, int MAX_THREADS>
+template <int HD, int MAX_THREADS, int SHAPE>
 __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(AttnArgs a) {
     extern __shared__ float wave_out[];      // [waves][rows][HD + 2]: o, then m and l
     // The grid is (heads, items, splits): blocks go to the eight XCDs in turn, so with the heads fastest every
@@ -886,7 +891,7 @@ __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(Att
     const int n = min(16, group - hb * 16);        // query heads in this block
     const int h0 = kvh * group + hb * 16;
     const bool empty = kv_begin >= kv_end;
-    WaveAttn<HD> w;
+    WaveAttn<HD, SHAPE> w;
     const bool row_ok = li < n;
     w.init(row_ok && !empty ? (const bf16*)a.q + (size_t)tok * a.ldq + (size_t)(h0 + li) * hd : nullptr, hd);
     if (!empty) {
@@ -909,14 +914,14 @@ __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(Att
             if (a.splits == 1) {
                 const float fin = finish_row<true>(a, h, m, l);
 #pragma unroll
-                for (int cb = 0; cb < WaveAttn<HD>::CB; ++cb) {
+                for (int cb = 0; cb < WaveAttn<HD, SHAPE>::CB; ++cb) {
                     const int d = 16 * cb + li;
                     if (d < a.vd) store_lane<bf16>(a, tok, h, d, w.o[cb][r] * fin);
                 }
             } else {
                 float* po = a.part_o + (((size_t)item * a.nh + h) * a.splits + split) * a.vd;
 #pragma unroll
-                for (int cb = 0; cb < WaveAttn<HD>::CB; ++cb) {
+                for (int cb = 0; cb < WaveAttn<HD, SHAPE>::CB; ++cb) {
                     const int d = 16 * cb + li;
                     if (d < a.vd) po[d] = m == NEG_INF ? 0.f : w.o[cb][r];
                 }
@@ -940,7 +945,7 @@ __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(Att
         const int row = 4 * g + r;
         if (row < n) {
 #pragma unroll
-            for (int cb = 0; cb < WaveAttn<HD>::CB; ++cb) mine[row * stride + 16 * cb + li] = w.o[cb][r];
+            for (int cb = 0; cb < WaveAttn<HD, SHAPE>::CB; ++cb) mine[row * stride + 16 * cb + li] = w.o[cb][r];
         }
     }
     __syncthreads();
@@ -998,36 +1003,22 @@ __global__ __launch_bounds__(MAX_THREADS) void attn_mfma_decode_block_kernel(Att
     }
 }
 
-// A head's row of biases for a block that walks over many tiles: a copy in LDS (dynamic, sized by the launch; a load from
-// memory inside the walk would be waited for behind the tiles that are on their way), or the row itself where it is too
-// long for that.
-#define BIAS_LDS_MAX 2048      // floats
-__device__ __forceinline__ bool bias_in_lds(const AttnArgs& a) { return bias_row_len(a) <= BIAS_LDS_MAX; }
+// A head's row of biases for a block that walks over many tiles is copied to LDS (dynamic, sized by the launch): a load from
+// memory inside the walk would be waited for behind the tiles that are on their way.  Rows longer than this are for the
+// kernels for any shape (beside the stages of the widest of these kernels, 132 KB, they would not fit).
+#define BIAS_LDS_MAX 6144      // floats
 __device__ __forceinline__ void stage_bias(const AttnArgs& a, int h, float* lds) {      // every thread; a barrier follows before its use
-    if (!a.bias || !bias_in_lds(a)) return;
     const float* row = a.bias + (size_t)h * bias_row_len(a);
     for (int i = threadIdx.x; i < bias_row_len(a); i += blockDim.x) lds[i] = row[i];
 }
-// the numbers of 16 consecutive keys, `distance` that of the first (one branch around all of them, so that the reads are
-// plain LDS or plain memory reads)
-__device__ __forceinline__ BiasRow read_bias(const AttnArgs& a, int h, const float* lds, int distance) {
-    if (!bias_in_lds(a)) return fetch_bias(a, h, distance);
-    BiasRow b;
-    const float* p = lds + bias_first(a, distance);
-#pragma unroll
-    for (int i = 0; i < 16; ++i) b.v[i >> 2][i & 3] = p[i];
-    return b;
-}
-static size_t bias_lds_bytes(const AttnArgs& a) {
-    return a.bias && bias_row_len(a) <= BIAS_LDS_MAX ? (size_t)bias_row_len(a) * sizeof(float) : 0;
-}
+static size_t bias_lds_bytes(const AttnArgs& a) { return a.bias ? (size_t)bias_row_len(a) * sizeof(float) : 0; }
 
 // Prefill with the keys and values of a tile shared through LDS: a block of four waves owns up
 // to 64 consecutive queries of one head (16 each); per tile of 64 keys the block stages K
 // (rows permuted so that the 16 keys an MFMA operand needs lie in consecutive rows) and the
 // transposed V once, and every wave takes its operands from there.  While a tile is multiplied
 // the next one is already on its way from memory into registers.
-template <int HD>
+template <int HD, int SHAPE>
 __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(AttnArgs a) {
     constexpr int KS = HD / 32, CB = HD / 16;
     constexpr int KROW = HD + 8;          // bf16 elements per staged key row (16 bytes of padding)
@@ -1072,7 +1063,7 @@ __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(
             w_lo_max = first_visible(a, w_hi);
         }
     }
-    const bool shaped = shapes_scores(a);
+    constexpr bool shaped = SHAPE != SHAPE_NONE;
     const float slope = a.slopes ? a.slopes[h] : 0.f;
     const float cs = shaped ? LOG2E : a.scale * LOG2E;
     float m = NEG_INF, l = 0.f;
@@ -1100,7 +1091,7 @@ __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(
     int first_blk, last_blk, unused;
     page_slot(a, kv_begin, first_blk, unused);
     page_slot(a, kv_end - 1, last_blk, unused);
-    stage_bias(a, h, bias_lds);
+    if (SHAPE == SHAPE_BIAS) stage_bias(a, h, bias_lds);
     const PageLookup pl = stage_pages(bt, page_copy, first_blk, last_blk);
     auto fetch = [&](uint4* kreg, uint4* vreg, int kt0) {
         size_t kbase[4], vbase[4];     // page and slot of each group of 16 keys of the tile (the same for all threads)
@@ -1189,10 +1180,10 @@ __global__ __launch_bounds__(256, HD > 128 ? 2 : 1) void attn_mfma_block_kernel(
         // tiles that every row of this wave sees whole need no mask
         const bool whole = kt0 >= w_lo_max && kt0 + 63 <= w_hi_min && kt0 >= kv_begin;
         uint4 p_lo, p_hi;
-        if (shaped) {
-            BiasRow bias = {};
-            if (a.bias) bias = read_bias(a, h, bias_lds, max(hi, 0) - (kt0 + 16 * g));
-            shape_scores(sc, kt0 + 16 * g, a, slope, hi, [&](int i) { return bias.v[i >> 2][i & 3]; });
+        if (SHAPE == SHAPE_CAP_SLOPE) cap_and_slope(sc, kt0 + 16 * g, a, slope, hi);
+        if (SHAPE == SHAPE_BIAS) {
+            const float* bias = bias_lds + bias_first(a, max(hi, 0) - (kt0 + 16 * g));
+            shape_with_bias(sc, kt0 + 16 * g, a, slope, hi, [&](int i) { return bias[i]; });
         }
         const float alpha = whole ? softmax_step<false>(sc, kt0 + 16 * g, lo, hi, cs, m, l, p_lo, p_hi)
                                   : softmax_step<true>(sc, kt0 + 16 * g, lo, hi, cs, m, l, p_lo, p_hi, span.keep);
@@ -1249,7 +1240,7 @@ typedef __attribute__((address_space(3))) void* fx_lds_ptr;
 // ones, group 1 the odd ones), each with stages, running maxima, sums and outputs of its own; group 1 hands its
 // results over through LDS at the end and group 0 merges them.  An item's chain of tiles is then half as long,
 // which is what bounds a prompt portion of few items over many keys.
-template <int HD, int NS, int W = 4, int G = 1>
+template <int HD, int NS, int W, int G, int SHAPE>
 __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(AttnArgs a) {      // two blocks on a CU, or one of two groups
     static_assert(G == 1 || (G == 2 && NS == 2), "one group, or two with two stages each");
     constexpr int KS = HD / 32, CB = HD / 16;
@@ -1296,7 +1287,7 @@ __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(Att
             w_lo_max = first_visible(a, w_hi);
         }
     }
-    const bool shaped = shapes_scores(a);
+    constexpr bool shaped = SHAPE != SHAPE_NONE;
     const float slope = a.slopes ? a.slopes[h] : 0.f;
     const float cs = shaped ? LOG2E : a.scale * LOG2E;
     float m = NEG_INF, l = 0.f;
@@ -1312,7 +1303,7 @@ __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(Att
     int first_blk, last_blk, unused;
     page_slot(a, kv_begin, first_blk, unused);
     page_slot(a, kv_end - 1, last_blk, unused);
-    stage_bias(a, h, bias_lds);
+    if (SHAPE == SHAPE_BIAS) stage_bias(a, h, bias_lds);
     const PageLookup pl = stage_pages(bt, page_copy, first_blk, last_blk);
     const KeySpan span = {kv_begin, kv_end, a.keep_first};
     const TileWalk walk = tile_walk(span);
@@ -1391,10 +1382,10 @@ __global__ __launch_bounds__(W * G * 64, W / 2) void attn_mfma_direct_kernel(Att
         }
         const bool whole = kt0 >= w_lo_max && kt0 + 63 <= w_hi_min && kt0 >= kv_begin;
         uint4 p_lo, p_hi;
-        if (shaped) {
-            BiasRow bias = {};
-            if (a.bias) bias = read_bias(a, h, bias_lds, max(hi, 0) - (kt0 + 16 * g));
-            shape_scores(sc, kt0 + 16 * g, a, slope, hi, [&](int i) { return bias.v[i >> 2][i & 3]; });
+        if (SHAPE == SHAPE_CAP_SLOPE) cap_and_slope(sc, kt0 + 16 * g, a, slope, hi);
+        if (SHAPE == SHAPE_BIAS) {
+            const float* bias = bias_lds + bias_first(a, max(hi, 0) - (kt0 + 16 * g));
+            shape_with_bias(sc, kt0 + 16 * g, a, slope, hi, [&](int i) { return bias[i]; });
         }
         const float alpha = whole ? softmax_step<false>(sc, kt0 + 16 * g, lo, hi, cs, m, l, p_lo, p_hi)
                                   : softmax_step<true>(sc, kt0 + 16 * g, lo, hi, cs, m, l, p_lo, p_hi, span.keep);
@@ -1471,6 +1462,16 @@ static bool mfma_ok(int dtype, int hd, int bs, const void* q, long ldq, const vo
            (((uintptr_t)q | (uintptr_t)k_pages | (uintptr_t)v_pages) % 16 == 0);
 }
 
+// f(the launch's shape as a compile-time constant)
+template <typename F>
+static void by_shape(const AttnArgs& a, F&& f) {
+    switch (shape_of(a)) {
+        case SHAPE_BIAS: f(std::integral_constant<int, SHAPE_BIAS>{}); break;
+        case SHAPE_CAP_SLOPE: f(std::integral_constant<int, SHAPE_CAP_SLOPE>{}); break;
+        default: f(std::integral_constant<int, SHAPE_NONE>{}); break;
+    }
+}
+
 // ---------------------------------------------------------------------------
 static int check_common(const char* who, int dtype, int nh, int nkv, int hd, int bs, int window, float scale, int vd = 0, int mask_chunk = 0,
                         int keep_first = 0) {
@@ -1510,6 +1511,7 @@ FX_API int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void*
     if (check_common("attn_tiles", dtype, nh, nkv, hd, bs, window, scale, vd, mask_chunk, keep_first)) return 1;
     FX_REQUIRE(tile_q == 64 || (tile_q == 128 && wide_items_ok(dtype, hd, bs) && mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd)),
                "attn_tiles: items of %d queries (64, or 128 where fx_attn_tile_queries says so)", tile_q);
+    FX_REQUIRE(tile_q == 64 || !bias || bias_n + 2 * BIAS_PAD <= BIAS_LDS_MAX, "attn_tiles: items of %d queries with biases for %d distances", tile_q, bias_n);
     if (n_items <= 0) return 0;
     AttnArgs a = {};
     a.q = q; a.ldq = ldq; a.out = out; a.ldo = ldo; a.k_pages = k_pages; a.v_pages = v_pages;
@@ -1537,27 +1539,26 @@ FX_API int fx_attn_tiles(void* stream, int dtype, const void* q, long ldq, void*
         attn_tile_kernel<float><<<grid, 64, 0, s>>>(a);
     else if (beyond)
         attn_tile_kernel<bf16, HD_MAX_ANY><<<grid, 64, 0, s>>>(a);
-    else if (mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd) && hd > 128) {
+    else if (mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd) && shm <= BIAS_LDS_MAX * sizeof(float)) by_shape(a, [&](auto shape) {
+        constexpr int SH = decltype(shape)::value;
         // the widest heads: tiles of 64 keys (34 KB) and their values (36 KB) staged in LDS for the block's 64 queries
-        attn_mfma_block_kernel<256><<<grid_blocks, 256, shm, s>>>(a);
-    } else if (mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd) && vd != hd) {
-        if (hd <= 64) attn_mfma_tile_kernel<64><<<grid, 64, 0, s>>>(a);
-        else attn_mfma_tile_kernel<128><<<grid, 64, 0, s>>>(a);
-    } else if (mfma_ok(dtype, hd, bs, q, ldq, k_pages, v_pages, vd)) {
-        if (tile_q == 128 && hd == 128 && two_groups) attn_mfma_direct_kernel<128, 2, 8, 2><<<grid_blocks, 1024, shm, s>>>(a);
-        else if (tile_q == 128 && hd == 64 && two_groups) attn_mfma_direct_kernel<64, 2, 8, 2><<<grid_blocks, 1024, shm, s>>>(a);
-        else if (tile_q == 128 && hd == 128) attn_mfma_direct_kernel<128, 2, 8><<<grid_blocks, 512, shm, s>>>(a);
-        else if (tile_q == 128) attn_mfma_direct_kernel<64, 2, 8><<<grid_blocks, 512, shm, s>>>(a);
-        else if (bs % 64 == 0 && hd == 128 && g_direct == 2 && two_groups) attn_mfma_direct_kernel<128, 2, 4, 2><<<grid_blocks, 512, shm, s>>>(a);
-        else if (bs % 64 == 0 && hd == 64 && g_direct == 2 && two_groups) attn_mfma_direct_kernel<64, 2, 4, 2><<<grid_blocks, 512, shm, s>>>(a);
-        else if (bs % 64 == 0 && hd == 128 && g_direct == 3) attn_mfma_direct_kernel<128, 3><<<grid_blocks, 256, shm, s>>>(a);
-        else if (bs % 64 == 0 && hd == 128 && g_direct) attn_mfma_direct_kernel<128, 2><<<grid_blocks, 256, shm, s>>>(a);
-        else if (bs % 64 == 0 && hd == 64 && g_direct) attn_mfma_direct_kernel<64, 2><<<grid_blocks, 256, shm, s>>>(a);
-        else if (hd <= 32) attn_mfma_block_kernel<32><<<grid_blocks, 256, shm, s>>>(a);
-        else if (hd <= 64) attn_mfma_block_kernel<64><<<grid_blocks, 256, shm, s>>>(a);
-        else if (hd <= 128) attn_mfma_block_kernel<128><<<grid_blocks, 256, shm, s>>>(a);
-        else return fx_fail("attn_tiles: no kernel for a head size of %d", hd);
-    } else
+        if (hd > 128) attn_mfma_block_kernel<256, SH><<<grid_blocks, 256, shm, s>>>(a);
+        else if (vd != hd && hd <= 64) attn_mfma_tile_kernel<64, SH><<<grid, 64, 0, s>>>(a);
+        else if (vd != hd) attn_mfma_tile_kernel<128, SH><<<grid, 64, 0, s>>>(a);
+        else if (tile_q == 128 && hd == 128 && two_groups) attn_mfma_direct_kernel<128, 2, 8, 2, SH><<<grid_blocks, 1024, shm, s>>>(a);
+        else if (tile_q == 128 && hd == 64 && two_groups) attn_mfma_direct_kernel<64, 2, 8, 2, SH><<<grid_blocks, 1024, shm, s>>>(a);
+        else if (tile_q == 128 && hd == 128) attn_mfma_direct_kernel<128, 2, 8, 1, SH><<<grid_blocks, 512, shm, s>>>(a);
+        else if (tile_q == 128) attn_mfma_direct_kernel<64, 2, 8, 1, SH><<<grid_blocks, 512, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 128 && g_direct == 2 && two_groups) attn_mfma_direct_kernel<128, 2, 4, 2, SH><<<grid_blocks, 512, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 64 && g_direct == 2 && two_groups) attn_mfma_direct_kernel<64, 2, 4, 2, SH><<<grid_blocks, 512, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 128 && g_direct == 3) attn_mfma_direct_kernel<128, 3, 4, 1, SH><<<grid_blocks, 256, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 128 && g_direct) attn_mfma_direct_kernel<128, 2, 4, 1, SH><<<grid_blocks, 256, shm, s>>>(a);
+        else if (bs % 64 == 0 && hd == 64 && g_direct) attn_mfma_direct_kernel<64, 2, 4, 1, SH><<<grid_blocks, 256, shm, s>>>(a);
+        else if (hd <= 32) attn_mfma_block_kernel<32, SH><<<grid_blocks, 256, shm, s>>>(a);
+        else if (hd <= 64) attn_mfma_block_kernel<64, SH><<<grid_blocks, 256, shm, s>>>(a);
+        else attn_mfma_block_kernel<128, SH><<<grid_blocks, 256, shm, s>>>(a);
+    });
+    else
         attn_tile_kernel<bf16><<<grid, 64, 0, s>>>(a);
     FX_CHECK_LAUNCH("attn_tiles");
     return 0;
@@ -1572,7 +1573,7 @@ static int attn_decode_launch(void* stream, int dtype, const void* q, long ldq, 
                               float* part_o, float* part_ml, int splits, int chunk, int waves, int vd = 0, int mask_chunk = 0,
                               int keep_first = 0, const float* sinks = nullptr, const void* gate = nullptr, long ldg = 0,
                               float softcap = 0.f, const float* slopes = nullptr, int gate_per_head = 0, const float* turns = nullptr,
-                           int gate_f32 = 0, const float* bias = nullptr, int bias_n = 0) {
+                              int gate_f32 = 0, const float* bias = nullptr, int bias_n = 0) {
     if (vd <= 0) vd = hd;
     AttnArgs a = {};
     a.gate_f32 = gate_f32 ? 1 : 0; a.bias = bias; a.bias_n = bias_n;
@@ -1617,10 +1618,13 @@ static int attn_decode_launch(void* stream, int dtype, const void* q, long ldq, 
         if (splits == 1 && 2 * n_blocks >= slots) nw = 1;
         if (waves > 0 && (size_t)waves * rows * (hdc + 2) * 4 <= 48 * 1024) nw = waves;      // the caller's choice
         const size_t shm = (size_t)nw * rows * (hdc + 2) * 4;
-        if (hd <= 32) attn_mfma_decode_block_kernel<32, 512><<<gridm, nw * 64, shm, s>>>(a);
-        else if (hd <= 64) attn_mfma_decode_block_kernel<64, 512><<<gridm, nw * 64, shm, s>>>(a);
-        else if (hd <= 128) attn_mfma_decode_block_kernel<128, 512><<<gridm, nw * 64, shm, s>>>(a);
-        else attn_mfma_decode_block_kernel<256, 256><<<gridm, nw * 64, shm, s>>>(a);
+        by_shape(a, [&](auto shape) {
+            constexpr int SH = decltype(shape)::value;
+            if (hd <= 32) attn_mfma_decode_block_kernel<32, 512, SH><<<gridm, nw * 64, shm, s>>>(a);
+            else if (hd <= 64) attn_mfma_decode_block_kernel<64, 512, SH><<<gridm, nw * 64, shm, s>>>(a);
+            else if (hd <= 128) attn_mfma_decode_block_kernel<128, 512, SH><<<gridm, nw * 64, shm, s>>>(a);
+            else attn_mfma_decode_block_kernel<256, 256, SH><<<gridm, nw * 64, shm, s>>>(a);
+        });
         if (splits > 1) attn_decode_merge_kernel<bf16><<<grid2, 128, splits * sizeof(float), s>>>(a);
     } else {
         attn_decode_kernel<bf16><<<grid, 64, 0, s>>>(a);

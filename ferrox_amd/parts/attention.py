@@ -383,7 +383,9 @@ class PagedAttention(Mixer):
         portion deep in a prompt: 603 against 784 us at 16 heads); else items of 128 if they still number about
         one evenly loaded block per CU (blocks of a portion that starts a prompt differ in work up to the portion's
         length in keys and count by their mean share of the longest; +8-26 % from 448 such blocks on); else 64."""
-        if ctx.recorded or self.v_dim != self.head_dim:      # (the kernels for unequal head sizes take items of 64)
+        if ctx.recorded or self.v_dim != self.head_dim or \
+                (self.distance_bias is not None and self.distance_bias.shape[1] > ops.BIAS_ROW_MAX):
+            # (the kernels for unequal head sizes, and for rows of biases that LDS does not hold, take items of 64)
             return 64
         widest = ops.attention_tile_queries(dtype, self.head_dim, block_size)
         if widest == 64:

@@ -50,13 +50,18 @@ class TokenEmbedding(Part):
         if self.position_table:
             self.positions = fetch(self.position_table).to(self.weight.dtype).contiguous()
 
-    def forward(self, token_ids, positions=None):
+    @property
+    def hands_rows(self) -> bool:
+        """Whether forward takes `rows`, a bfloat16 tensor that receives the rows once more, rounded."""
+        return self.norm is None
+
+    def forward(self, token_ids, positions=None, rows=None):
         if self.position_table:
-            return ops.embed(self.weight, token_ids, scale=self.scale, position_table=self.positions, positions=positions)
+            return ops.embed(self.weight, token_ids, scale=self.scale, position_table=self.positions, positions=positions, rows=rows)
         if self.norm is not None:
             weight, eps = self.norm.rms_params()
             return ops.embed_rmsnorm(self.weight, token_ids, weight, eps, scale=self.scale)
-        return ops.embed(self.weight, token_ids, scale=self.scale)
+        return ops.embed(self.weight, token_ids, scale=self.scale, rows=rows)
 
 
 @HEADS.register("linear_head")

@@ -126,6 +126,18 @@ def test_layer_norm_as_rows_join_the_stream(dtype, H):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_the_embedding_hands_out_its_rows_rounded(dtype):
+    from ferrox_amd import ops
+    gen = torch.Generator().manual_seed(3)
+    table, pos = torch.randn(30, 37, generator=gen).to(dtype).cuda(), torch.randn(8, 37, generator=gen).to(dtype).cuda()
+    ids, places = torch.tensor([3, 29, 0], dtype=torch.int32).cuda(), torch.tensor([7, 0, 2], dtype=torch.int32).cuda()
+    for kw in ({}, {"position_table": pos, "positions": places}):
+        rows = torch.empty(3, 37, dtype=torch.bfloat16, device="cuda")
+        h = ops.embed(table, ids, scale=2.5, rows=rows, **kw)
+        assert torch.equal(h, ops.embed(table, ids, scale=2.5, **kw)) and torch.equal(rows, h.bfloat16())
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_gated_products_of_every_kind_of_kernel(dtype):
     """The gate in the epilogues of grouped products (a head a group, gate columns beside other columns of wider rows) for
     few rows and many, of sizes that fit no vector, and of a plain product."""
@@ -279,14 +291,14 @@ def test_attention_kernels_with_distance_biases(dtype, hd, vd, bs, G):
     item = lambda x: torch.tensor(x, dtype=torch.int32, device="cuda")      # noqa: E731
     for window, n_bias, sinks, gate, cap, slope in ((40, 40, zeros, None, 0.0, False), (100, 30, zeros, "head", 0.0, False),
                                                     (0, 150, None, "element", 0.0, False), (70, 1, learned, None, 1.5, True),
-                                                    (0, 2500, zeros, "head", 0.0, False), (64, 64, None, None, 2.0, False)):
+                                                    (0, 6200, zeros, "head", 0.0, False), (64, 64, None, None, 2.0, False)):
         bias = torch.randn(H, n_bias, generator=gen) * 2
         want = attention_reference(q, k, v, 0.2, window, bias, sinks, gates[gate] if gate else None, cap, slopes if slope else None).view(n, -1)
         common = (H, G, hd, bs, window, 0.2)
         extra = dict(v_dim=vd, sinks=sinks.cuda() if sinks is not None else None, gate=gates[gate].cuda() if gate else None,
                      gate_per_head=gate == "head", softcap=cap, slopes=slopes.cuda() if slope else None,
                      distance_bias=ops.distance_bias_rows(bias).cuda())
-        for tile in sorted({64, ops.attention_tile_queries(dt, hd, bs) if vd == hd else 64}):
+        for tile in sorted({64, ops.attention_tile_queries(dt, hd, bs) if vd == hd and n_bias < ops.BIAS_ROW_MAX else 64}):
             for first in (0, 200):
                 starts = list(range(first, n, tile))
                 out = torch.full((n, H * vd), float("nan"), dtype=dt, device="cuda")
