@@ -10,43 +10,38 @@ FX_DEFINE_LAST_ERROR()
 
 // ---------------------------------------------------------------------------
 // embedding: h[t, :] = table[ids[t], :] * scale   (the reference has no scale, ferrox-models/src/decoder.rs:1279-1284;
-// a design that multiplies its embeddings by a constant does so here, in float32); with `rows`, the same rows once more in
-// bfloat16, for a first layer that reads the stream as it is
+// a design that multiplies its embeddings by a constant does so here, in float32)
 // ---------------------------------------------------------------------------
 template <typename W>
 __global__ void embed_kernel(const W* __restrict__ table, const int* __restrict__ ids,
                              float* __restrict__ h, int H, int V, float scale,
-                             const W* __restrict__ pos_table, const int* __restrict__ positions, int n_pos, bf16* __restrict__ rows) {
+                             const W* __restrict__ pos_table, const int* __restrict__ positions, int n_pos) {
     const int t = blockIdx.x;
-    auto put = [&](int c, float v) {
-        h[(size_t)t * H + c] = v;
-        if (rows) rows[(size_t)t * H + c] = float_to_bf16(v);
-    };
     int id = ids[t];
     const int pos = pos_table ? positions[t] : 0;
     if (id < 0 || id >= V || pos < 0 || (pos_table && pos >= n_pos)) {  // the host rejects such ids and places; never read outside a table
-        for (int c = threadIdx.x; c < H; c += blockDim.x) put(c, __int_as_float(0x7fc00000));
+        for (int c = threadIdx.x; c < H; c += blockDim.x) h[(size_t)t * H + c] = __int_as_float(0x7fc00000);
         return;
     }
     const W* row = table + (size_t)id * H;
     if (pos_table) {       // a learned vector per position joins the token's row (it is not scaled)
         const W* prow = pos_table + (size_t)pos * H;
-        for (int c = threadIdx.x; c < H; c += blockDim.x) put(c, to_float(row[c]) * scale + to_float(prow[c]));
+        for (int c = threadIdx.x; c < H; c += blockDim.x) h[(size_t)t * H + c] = to_float(row[c]) * scale + to_float(prow[c]);
         return;
     }
-    for (int c = threadIdx.x; c < H; c += blockDim.x) put(c, to_float(row[c]) * scale);
+    for (int c = threadIdx.x; c < H; c += blockDim.x) h[(size_t)t * H + c] = to_float(row[c]) * scale;
 }
 
 FX_API int fx_embed(void* stream, int w_dtype, const void* table, const int* ids, float* h,
-                    int T, int H, int V, float scale, const void* pos_table, const int* positions, int n_pos, void* rows) {
+                    int T, int H, int V, float scale, const void* pos_table, const int* positions, int n_pos) {
     FX_REQUIRE(T >= 0 && H > 0 && V > 0, "embed: bad sizes T=%d H=%d V=%d", T, H, V);
     FX_REQUIRE(!pos_table || (positions && n_pos > 0), "embed: a table of positions needs the tokens' positions");
     if (T == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     if (w_dtype == FX_F32)
-        embed_kernel<float><<<T, 256, 0, s>>>((const float*)table, ids, h, H, V, scale, (const float*)pos_table, positions, n_pos, (bf16*)rows);
+        embed_kernel<float><<<T, 256, 0, s>>>((const float*)table, ids, h, H, V, scale, (const float*)pos_table, positions, n_pos);
     else if (w_dtype == FX_BF16)
-        embed_kernel<bf16><<<T, 256, 0, s>>>((const bf16*)table, ids, h, H, V, scale, (const bf16*)pos_table, positions, n_pos, (bf16*)rows);
+        embed_kernel<bf16><<<T, 256, 0, s>>>((const bf16*)table, ids, h, H, V, scale, (const bf16*)pos_table, positions, n_pos);
     else
         return fx_fail("embed: unknown table dtype %d", w_dtype);
     FX_CHECK_LAUNCH("embed");

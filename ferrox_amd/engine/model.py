@@ -127,16 +127,11 @@ class Model:
     def forward(self, ctx: StepContext, caches: list):
         debug.region("embed")
         # (an embedding that adds something per position says so and gets the tokens' positions)
-        asks = {"positions": ctx.positions} if getattr(self.embedding, "uses_positions", False) else {}
-        # (a first block that reads the stream as it is gets its rows from the embedding's launch)
-        normed = None
-        first = self.blocks[self.schedule[0].layer] if self.schedule else None
-        if first is not None and first.chains_norms and getattr(first.first_norm, "as_is", False) and ctx.act_dtype == torch.bfloat16 \
-                and getattr(self.embedding, "hands_rows", False):
-            normed = asks["rows"] = torch.empty((ctx.n_tokens, self.spec.hidden_size), dtype=torch.bfloat16, device=ctx.device)
-        h = self.embedding.forward(ctx.token_ids, **asks)
+        h = self.embedding.forward(ctx.token_ids, positions=ctx.positions) if getattr(self.embedding, "uses_positions", False) \
+            else self.embedding.forward(ctx.token_ids)
         # blocks that chain their norms: the block before may already have applied this block's first norm
         # to the rows it finished (in the kernel that finished them)
+        normed = None
         for i, e in enumerate(self.schedule):
             block = self.blocks[e.layer]
             if block.chains_norms:

@@ -60,7 +60,7 @@ def _stream():
 
 
 _sigs = {
-    ("elementwise", "fx_embed"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p],
+    ("elementwise", "fx_embed"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int],
     ("elementwise", "fx_embed_rmsnorm"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_int, c_float],
     ("elementwise", "fx_angle_table"): [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int],
     ("elementwise", "fx_turned_kv_write"): [c_void_p, c_int, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p,
@@ -182,16 +182,12 @@ def _i32(t, what):
 
 # ---------------------------------------------------------------------------
 def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor | None = None, scale: float = 1.0,
-          position_table: torch.Tensor | None = None, positions: torch.Tensor | None = None,
-          rows: torch.Tensor | None = None) -> torch.Tensor:
-    """h[t] = table[ids[t]] * scale (+ position_table[positions[t]], a learned vector per position) as float32.  `rows`
-    (bfloat16 [T, H]) receives the same rows rounded."""
+          position_table: torch.Tensor | None = None, positions: torch.Tensor | None = None) -> torch.Tensor:
+    """h[t] = table[ids[t]] * scale (+ position_table[positions[t]], a learned vector per position) as float32."""
     V, H = table.shape
     T = ids.numel()
     if out is None:
         out = torch.empty((T, H), dtype=torch.float32, device=table.device)
-    if rows is not None and (rows.dtype != torch.bfloat16 or tuple(rows.shape) != (T, H) or not rows.is_contiguous()):
-        raise KernelError(f"embed: rounded rows go to a contiguous bfloat16 [{T}, {H}], not {tuple(rows.shape)} ({rows.dtype})")
     n_pos = 0
     if position_table is not None:
         if positions is None or positions.numel() < T or position_table.dtype != table.dtype or position_table.dim() != 2 \
@@ -200,8 +196,7 @@ def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor | None = Non
                               f"embedding table {tuple(table.shape)} ({table.dtype}) needs the tokens' positions")
         n_pos = position_table.shape[0]
     _call("elementwise", "fx_embed", _stream(), dtype_code(table.dtype), _p(table), _p(_i32(ids, "ids")), _p(out), T, H, V,
-          float(scale), _p(position_table), _p(_i32(positions, "positions")) if position_table is not None else None, n_pos,
-          _p(rows))
+          float(scale), _p(position_table), _p(_i32(positions, "positions")) if position_table is not None else None, n_pos)
     return out
 
 

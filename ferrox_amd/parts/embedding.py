@@ -50,18 +50,13 @@ class TokenEmbedding(Part):
         if self.position_table:
             self.positions = fetch(self.position_table).to(self.weight.dtype).contiguous()
 
-    @property
-    def hands_rows(self) -> bool:
-        """Whether forward takes `rows`, a bfloat16 tensor that receives the rows once more, rounded."""
-        return self.norm is None
-
-    def forward(self, token_ids, positions=None, rows=None):
+    def forward(self, token_ids, positions=None):
         if self.position_table:
-            return ops.embed(self.weight, token_ids, scale=self.scale, position_table=self.positions, positions=positions, rows=rows)
+            return ops.embed(self.weight, token_ids, scale=self.scale, position_table=self.positions, positions=positions)
         if self.norm is not None:
             weight, eps = self.norm.rms_params()
             return ops.embed_rmsnorm(self.weight, token_ids, weight, eps, scale=self.scale)
-        return ops.embed(self.weight, token_ids, scale=self.scale, rows=rows)
+        return ops.embed(self.weight, token_ids, scale=self.scale)
 
 
 @HEADS.register("linear_head")

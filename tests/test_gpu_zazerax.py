@@ -126,18 +126,6 @@ def test_layer_norm_as_rows_join_the_stream(dtype, H):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-def test_the_embedding_hands_out_its_rows_rounded(dtype):
-    from ferrox_amd import ops
-    gen = torch.Generator().manual_seed(3)
-    table, pos = torch.randn(30, 37, generator=gen).to(dtype).cuda(), torch.randn(8, 37, generator=gen).to(dtype).cuda()
-    ids, places = torch.tensor([3, 29, 0], dtype=torch.int32).cuda(), torch.tensor([7, 0, 2], dtype=torch.int32).cuda()
-    for kw in ({}, {"position_table": pos, "positions": places}):
-        rows = torch.empty(3, 37, dtype=torch.bfloat16, device="cuda")
-        h = ops.embed(table, ids, scale=2.5, rows=rows, **kw)
-        assert torch.equal(h, ops.embed(table, ids, scale=2.5, **kw)) and torch.equal(rows, h.bfloat16())
-
-
-@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_gated_products_of_every_kind_of_kernel(dtype):
     """The gate in the epilogues of grouped products (a head a group, gate columns beside other columns of wider rows) for
     few rows and many, of sizes that fit no vector, and of a plain product."""
