@@ -67,7 +67,7 @@ def test_rope_angle_in_float32_is_one_rounded_product():
     x = randn(16)
     near = plain.rope_neox(x, 2047, 1e4, "float32")
     assert torch.allclose(near, plain.rope_neox(x, 2047, 1e4), atol=1e-3) and not torch.allclose(
-        near, plain.rope_neox(x, 2047, 1e4), atol=1e-7)
+        near, plain.rope_neox(x, 2047, 1e4), rtol=0.0, atol=1e-7)
 
 
 def test_rope_scores_depend_on_distance_only():
